@@ -1,0 +1,206 @@
+"""A slow, whole-sequence implementation of the Surodra design, one function per mechanism, written from its equations
+and sharing no code with the package: the oracle of tests/test_surodra.py.  Everything runs in fp32 (or fp64) on the CPU
+over one whole sequence at a time; there is no cache, no batching and no portioning here.
+
+Notation: x residual [L, W]; N squashing norm; a layer computes x <- x + m mixer(N1 x), then x <- x + m ff(N2 x).
+"""
+import json
+import math
+import os
+
+import torch
+
+
+# ---- norms ---------------------------------------------------------------------------------------------------------
+def squash_norm(x, alpha, w, b):
+    """No statistics at all: every value is squashed on its own."""
+    return torch.tanh(alpha * x) * w + b
+
+
+def unit_rms(y, eps):
+    return y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps)
+
+
+def unit_vector(y):
+    return y / torch.sqrt((y * y).sum(-1, keepdim=True) + 1e-6)
+
+
+def silu(z):
+    return z * torch.sigmoid(z)
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1 + torch.tanh(math.sqrt(2 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+# ---- short causal convolution ----------------------------------------------------------------------------------------
+def short_conv(u, w):
+    """u [L, C], w [C, taps]:  y[t] = sum_j w[:, j] u[t - taps + 1 + j], zeros before the sequence."""
+    L, C = u.shape
+    taps = w.shape[1]
+    padded = torch.cat([torch.zeros(taps - 1, C, dtype=u.dtype), u])
+    y = torch.zeros_like(u)
+    for j in range(taps):
+        y = y + w[:, j] * padded[j: j + L]
+    return y
+
+
+# ---- rotation --------------------------------------------------------------------------------------------------------
+def rotate(x, rot):
+    """x [L, heads, D]: value i < dims / 2 and value i + dims / 2 form a pair, turned by position * f_i."""
+    dims = int((rot or {}).get("dims", 0) or 0)
+    if dims == 0:
+        return x
+    L, n = x.shape[0], dims // 2
+    f = torch.tensor([rot["base"] ** (-2.0 * i / dims) for i in range(n)], dtype=torch.float64)
+    if rot.get("scaling"):
+        f = f / rot["scaling"]["factor"]
+    ang = torch.arange(L, dtype=torch.float64)[:, None] * f[None, :]
+    c, s = torch.cos(ang).to(x.dtype)[:, None, :], torch.sin(ang).to(x.dtype)[:, None, :]
+    a, b = x[..., :n], x[..., n: dims]
+    return torch.cat([a * c - b * s, b * c + a * s, x[..., dims:]], dim=-1)
+
+
+# ---- recurrences, token by token -----------------------------------------------------------------------------------
+def decayed_memory(q, k, v, decay):
+    """q, k, decay [L, H, D], v [L, H, E]:  S_t = diag(decay_t) S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t."""
+    L, H, D = q.shape
+    S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype)
+    out = []
+    for t in range(L):
+        S = decay[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+        out.append((S * q[t][:, :, None]).sum(1))
+    return torch.stack(out)
+
+
+def delta_memory(q, k, v, g, beta):
+    """q, k [L, H, D], v [L, H, E], g, beta [L, H]: decay, correct the value read at k, write, read at q."""
+    L, H, D = q.shape
+    S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype)
+    out = []
+    for t in range(L):
+        S = g[t][:, None, None] * S
+        u = beta[t][:, None] * (v[t] - (S * k[t][:, :, None]).sum(1))
+        S = S + k[t][:, :, None] * u[:, None, :]
+        out.append((S * q[t][:, :, None]).sum(1))
+    return torch.stack(out)
+
+
+# ---- mixers ------------------------------------------------------------------------------------------------------------
+def delta_mixer(h, w, m, eps):
+    L = h.shape[0]
+    H, G, D, E = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q, k, v = (silu(short_conv(h @ w[n].T, w[n + ".conv"])) for n in ("q", "k", "v"))
+    q = unit_vector(q.view(L, G, D)) * D ** -0.5
+    k = unit_vector(k.view(L, G, D))
+    own = torch.arange(H) // (H // G)
+    beta = torch.sigmoid(h @ w["b"].T)
+    g = torch.exp(-torch.exp(w["A_log"]) * torch.log1p(torch.exp(h @ w["a"].T + w["dt_bias"])))
+    o = delta_memory(q[:, own], k[:, own], v.view(L, H, E), g, beta)
+    o = unit_rms(o, eps) * w["norm"] * silu(h @ w["g"].T).view(L, H, E)
+    return o.reshape(L, H * E) @ w["o"].T
+
+
+def sink_attention(h, w, m, eps):
+    L = h.shape[0]
+    H, G, D, E = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q = unit_rms(h @ w["q"].T, eps) * w["q.norm"]            # over the whole projection, not per head
+    k = unit_rms(h @ w["k"].T, eps) * w["k.norm"]
+    v = (h @ w["v"].T).view(L, G, E)
+    q, k = rotate(q.view(L, H, D), m.get("rot")), rotate(k.view(L, G, D), m.get("rot"))
+    seen = torch.arange(L)[None, :] <= torch.arange(L)[:, None]
+    gate = torch.sigmoid(h @ w["g"].T)
+    out = []
+    for n in range(H):
+        g = n // (H // G)
+        s = (q[:, n] @ k[:, g].T) * m["scale"]
+        s = s.masked_fill(~seen, float("-inf"))
+        top = torch.maximum(s.max(-1, keepdim=True).values, w["sink"][n])
+        e = torch.exp(s - top)
+        p = e / (e.sum(-1, keepdim=True) + torch.exp(w["sink"][n] - top))
+        out.append((p @ v[:, g]) * gate[:, n: n + 1])
+    return torch.cat(out, -1) @ w["o"].T
+
+
+def gated_linear_mixer(h, w, m, eps):
+    L = h.shape[0]
+    H, D, E = m["heads"], m["dim"], m["vdim"]
+    q = (h @ w["q"].T).view(L, H, D) * D ** -0.5
+    k = (h @ w["k"].T).view(L, H, D)
+    v = (h @ w["v"].T).view(L, H, E)
+    z = (h @ w["a1"].T) @ w["a2"].T + w["a2.b"]
+    alpha = torch.sigmoid(z) ** (1.0 / m["tau"])
+    o = unit_rms(decayed_memory(q, k, v, alpha.view(L, H, D)), eps) * w["norm"]
+    return (o.reshape(L, H * E) * silu(h @ w["g"].T)) @ w["o"].T
+
+
+def parallel_mixer(h, w, m, eps):
+    def part(side):
+        return {n[len(side) + 1:]: t for n, t in w.items() if n.startswith(side + ".")}
+    lw, rw = part("left"), part("right")
+    a = unit_rms(sink_attention(h, lw, m["left"], eps), eps) * lw["out"]
+    b = unit_rms(gated_linear_mixer(h, rw, m["right"], eps), eps) * rw["out"]
+    return 0.5 * (a + b)
+
+
+def retention_mixer(h, w, m, eps):
+    L = h.shape[0]
+    H, D, E = m["heads"], m["dim"], m["vdim"]
+    q = rotate((h @ w["q"].T).view(L, H, D), m.get("rot"))
+    k = rotate((h @ w["k"].T).view(L, H, D), m.get("rot")) * D ** -0.5
+    v = (h @ w["v"].T).view(L, H, E)
+    decay = torch.tensor(m["decay"], dtype=h.dtype)[None, :, None].expand(L, H, D)
+    o = unit_rms(decayed_memory(q, k, v, decay), eps)
+    return (o.reshape(L, H * E) * silu(h @ w["g"].T)) @ w["o"].T
+
+
+MIXERS = {"delta": delta_mixer, "parallel": parallel_mixer, "retention": retention_mixer}
+
+
+def feed_forward(h, w):
+    return (gelu_tanh(h @ w["gate"].T) * (h @ w["up"].T)) @ w["down"].T
+
+
+# ---- the stack -----------------------------------------------------------------------------------------------------------
+def run_list(n, loop):
+    """(layer, pass, is this the first layer of a pass?) in running order."""
+    if not loop:
+        return [(i, 0, False) for i in range(n)]
+    a, b = loop["start"], loop["stop"]
+    return [(i, 0, False) for i in range(a)] + \
+        [(i, t, i == a) for t in range(loop["times"]) for i in range(a, b)] + [(i, 0, False) for i in range(b, n)]
+
+
+def model_logits(tokens, weights, config, dtype=torch.float32, trail=None):
+    """tokens: list of ids.  Returns logits [L, vocab]; ``trail`` collects the residual after every layer run."""
+    W = {n: t.to(dtype) for n, t in weights.items()}
+    eps, mult = config["norm"]["eps"], config.get("residual_mult", 1.0)
+
+    def norm(x, name):
+        return squash_norm(x, W[name + ".alpha"], W[name], W[name + ".b"])
+
+    def sub(prefix):
+        return {n[len(prefix):]: t for n, t in W.items() if n.startswith(prefix)}
+    e = W["embed"][torch.tensor(tokens)]
+    x = e
+    for i, t, first in run_list(len(config["layers"]), config.get("loop")):
+        spec = config["layers"][i]
+        if first:
+            if t > 0:
+                x = x + e
+            x = x + W["loop.step"][t]
+        x = x + mult * MIXERS[spec["type"]](norm(x, f"l{i}.norm1"), sub(f"l{i}.mix."), spec["mixer"], eps)
+        if spec.get("mlp"):
+            x = x + mult * feed_forward(norm(x, f"l{i}.norm2"), sub(f"l{i}.mlp."))
+        if trail is not None:
+            trail.append(x.clone())
+    y = norm(x, "final.norm") @ W["head"].T * config.get("logit_scale", 1.0)
+    cap = config.get("logit_softcap")
+    return cap * torch.tanh(y / cap) if cap else y
+
+
+def load_folder(folder):
+    from safetensors.torch import load_file
+    with open(os.path.join(folder, "config.json")) as f:
+        config = json.load(f)
+    return config, load_file(os.path.join(folder, "model.safetensors"))

@@ -176,6 +176,9 @@ def load_hf_config(model: str, overrides: Optional[dict] = None) -> HFConfig:
     if d.get("architecture") == "Lefolorn":        # a layer list of three attention variants with parallel sub-layers
         from .models.lefolorn import normalise_config as lefolorn_config
         d = lefolorn_config(d, model if os.path.isdir(model) else None)
+    if d.get("architecture") == "Surodra":         # a looped layer list of recurrent mixers, some beside attention
+        from .models.surodra import normalise_config as surodra_config
+        d = surodra_config(d, model if os.path.isdir(model) else None)
     if d.get("model_type") in ("exaone", "telechat", "qwen", "chatglm"):
         from .models.renamed_decoders import normalise_config
         d = normalise_config(d)
@@ -343,7 +346,8 @@ class ModelConfig:
                          # encoder-decoder: the cross-attention cache is per-request state of the same kind
                          "WhisperForConditionalGeneration", "BartForConditionalGeneration", "BartModel",
                          "MllamaForConditionalGeneration", "Zamba2ForCausalLM", "Plamo2ForCausalLM",
-                         "Florence2ForConditionalGeneration", "NositarForCausalLM", "RapovikForCausalLM", "SevazenForCausalLM")
+                         "Florence2ForConditionalGeneration", "NositarForCausalLM", "RapovikForCausalLM", "SevazenForCausalLM",
+                         "SurodraForCausalLM")
                    for a in self.architectures)
 
     @property

@@ -37,6 +37,19 @@ def default_weight_loader(param: torch.Tensor, loaded: torch.Tensor) -> None:
     param.data.copy_(loaded)
 
 
+def row_padding(width: int, to: int = 16) -> int:
+    """Columns that fill a fused projection's rows up to a multiple of ``to`` values, so that its consumers can use
+    aligned 16-byte accesses whatever small pieces (gates, steps) the rows end in."""
+    return -int(width) % to
+
+
+def zero_tail_rows(layer: nn.Module, n: int) -> None:
+    """The weight rows behind such padding columns are zero (no checkpoint tensor fills them)."""
+    w = getattr(layer, "weight", None)
+    if n and w is not None and w.is_floating_point():
+        w.data[w.shape[0] - n:].zero_()
+
+
 class UnquantizedLinearMethod:
     def create_weights(self, layer: nn.Module, in_per_rank: int, out_per_rank: int, dtype: torch.dtype) -> None:
         w = nn.Parameter(torch.empty(out_per_rank, in_per_rank, dtype=dtype), requires_grad=False)

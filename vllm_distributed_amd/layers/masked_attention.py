@@ -4,7 +4,9 @@ on the projections, several score maps per head, window / chunk masks, sinks and
     q, k, v = W x + b                                   (optional biases; grouped query heads; key width D, value width Dv)
     q, k, v <- causal convolution over time, per channel (``conv_taps`` >= 1; no bias, no activation; one tap is a
                weight per channel)
-    q, k    <- q / rms(q) * q_norm, k / rms(k) * k_norm  per head and map (weights of size D shared by all heads)
+    q, k    <- q / rms(q) * q_norm, k / rms(k) * k_norm  per head and map (weights of size D shared by all heads), or,
+               with ``norm_over`` "projection", one root mean square over all of q and one over all of k (weights as
+               long as the projections)
     q, k    <- first ``rot_dims`` values of each map rotated, value i paired with i + rot_dims / 2 (``rot_pairing``
                "halves") or value 2i with 2i + 1 ("neighbours"), fp32 angles
     q       <- q * (1 + coef * ln(floor((p + 1) / every) + 1)) at position p (``q_temp`` = (coef, every))
@@ -19,7 +21,7 @@ on the projections, several score maps per head, window / chunk masks, sinks and
     maps == 2 (differential attention): a head's query / key rows hold two maps side by side, each an attention over
                the same values;  o = a1 - lam * a2,  lam = exp(lq1 . lk1) - exp(lq2 . lk2) + diff,
                then o / rms(o) * (1 - diff) over the head's Dv values
-    out     = W_o (o * sigmoid(W_g x))                   (``gate``)
+    out     = W_o (o * sigmoid(W_g x))                   (``gate``: True, one number per value, or "head", one per head)
 
 The layer owns pages of the ordinary paged KV cache (a full-attention layer to the scheduler and the KV-cache manager:
 keys that a window or chunk hides stay in their pages, the kernels never load them) and, with a convolution, a state
@@ -46,7 +48,8 @@ from ..models.mamba import StateSpaceLayer
 from ..parallel.state import get_tensor_model_parallel_world_size
 from ..sched.kv_cache_interface import FullAttentionSpec, KVCacheSpec
 from .hyper_connections import _fp32_param
-from .linear import MergedColumnParallelLinear, RowParallelLinear, set_weight_attrs
+from .linear import (MergedColumnParallelLinear, RowParallelLinear, row_padding, set_weight_attrs,
+                     zero_tail_rows)
 from .rotary import half_split_cos_sin
 
 
@@ -101,10 +104,11 @@ class ShortConvState(StateSpaceLayer):
 class MaskedSoftmaxAttention(nn.Module):
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, v_head_dim: int,
                  scale: float, eps: float, *, bias: bool = False, conv_taps: int = 0, window: int = 0, chunk: int = 0,
-                 sink: bool = False, maps: int = 1, diff: float = 0.0, gate: bool = False, rot_dims: int = 0,
+                 sink: bool = False, maps: int = 1, diff: float = 0.0, gate=False, rot_dims: int = 0,
                  rot_base: float = 10000.0, rot_scaling: Optional[dict] = None, users: int = 1, quant_config=None,
                  prefix: str = "", rot_pairing: str = "halves", q_temp: Optional[tuple] = None, softcap: float = 0.0,
-                 dist_bias: Optional[tuple] = None, sink_fixed: Optional[float] = None, v_mix: bool = False):
+                 dist_bias: Optional[tuple] = None, sink_fixed: Optional[float] = None, v_mix: bool = False,
+                 norm_over: str = "head"):
         super().__init__()
         if get_tensor_model_parallel_world_size() > 1:
             raise NotImplementedError("this attention layer runs with tensor_parallel_size=1")
@@ -132,15 +136,23 @@ class MaskedSoftmaxAttention(nn.Module):
         self.layer_name = prefix
         nq, nk, nv = H * maps * D, G * maps * D, G * Dv
         self.qkv_width = nq + nk + nv
-        sizes = [nq, nk, nv] + ([H * Dv] if gate else [])
+        if gate not in (False, True, "head"):
+            raise ValueError(f"{prefix}: gate {gate!r} (False, True or 'head')")
+        self.gate_width = (H if gate == "head" else H * Dv) if gate else 0
+        pad = row_padding(self.qkv_width + self.gate_width) if gate == "head" else 0
+        sizes = [nq, nk, nv] + ([self.gate_width] if gate else []) + ([pad] if pad else [])
         # one GEMM for everything that reads x: q | k | v (| gate); the gate's part of the bias stays zero
         self.in_proj = MergedColumnParallelLinear(hidden_size, sizes, bias=bias, quant_config=quant_config,
                                                   prefix=f"{prefix}.in_proj")
+        zero_tail_rows(self.in_proj, pad)
         self.has_gate = bool(gate)
         self.o_proj = RowParallelLinear(H * Dv, hidden_size, bias=False, quant_config=quant_config,
                                         prefix=f"{prefix}.o_proj")
-        self.q_norm = _fp32_param((D,))
-        self.k_norm = _fp32_param((D,))
+        if norm_over not in ("head", "projection"):
+            raise ValueError(f"{prefix}: norms over {norm_over!r} ('head' or 'projection')")
+        self.whole_norm = norm_over == "projection"
+        self.q_norm = _fp32_param((nq if self.whole_norm else D,))
+        self.k_norm = _fp32_param((nk if self.whole_norm else D,))
         if sink_fixed is not None:
             self.register_buffer("sink", torch.full((H,), float(sink_fixed), dtype=torch.float32), persistent=False)
         else:
@@ -226,10 +238,12 @@ class MaskedSoftmaxAttention(nn.Module):
         p = self.in_proj(x)
         T = p.shape[0]
         W = self.qkv_width
-        gate = p[:, W:] if self.has_gate else None
+        gate = p[:, W: W + self.gate_width] if self.has_gate else None
         if md is None or kv.k_cache is None:              # memory-profiling run: the projections carry the footprint
             o = p[:, : H * maps * D].reshape(T, H, maps * D)[..., :1].expand(T, H, Dv).reshape(T, H * Dv)
-            return self.o_proj((o * gate if gate is not None else o).contiguous())
+            if gate is not None:
+                o = o * (gate if gate.shape[1] == H * Dv else gate[:, :1])
+            return self.o_proj(o.contiguous())
         n = md.num_actual_tokens
         S = md.num_decode_seqs + md.num_prefill_seqs
         qsl, lens = md.query_start_loc[:S + 1], md.seq_lens[:S]
@@ -242,7 +256,7 @@ class MaskedSoftmaxAttention(nn.Module):
         elif self.taps == 1:
             qkv = (p[:n, :W].float() * self.conv_weight.float().view(1, -1)).to(p.dtype)
         g_rows = gate[:n] if gate is not None else None
-        extras = dict(pairing=self.rot_pairing, q_temp=self.q_temp)
+        extras = dict(pairing=self.rot_pairing, q_temp=self.q_temp, whole_norm=self.whole_norm)
         if self.vmix is not None:
             if lent is None:
                 raise ValueError(f"{self.layer_name}: value mixing needs the forward pass's dictionary")

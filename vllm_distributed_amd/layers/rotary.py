@@ -63,7 +63,7 @@ _HALF_SPLIT_TABLES: dict = {}
 
 def half_split_cos_sin(max_len: int, rot_dim: int, base: float, scaling: Optional[dict], device) -> torch.Tensor:
     """fp32 [max_len, rot_dim] for kernels that rotate in fp32: cos(p f_i) for i < rot_dim / 2, then sin(p f_i), with
-    f_i = base^(-2i / rot_dim) rescaled by ``scaling``: None, {"kind": "llama3", factor, low, high, original} or
+    f_i = base^(-2i / rot_dim) rescaled by ``scaling``: None, {"kind": "linear", factor} (every f_i divided by it), {"kind": "llama3", factor, low, high, original} or
     {"kind": "yarn", factor, original, fast, slow, magnitude} (cos and sin times ``magnitude``).  Angles are formed in
     fp64 and rounded once."""
     sc = dict(scaling or {})
@@ -83,6 +83,8 @@ def half_split_cos_sin(max_len: int, rot_dim: int, base: float, scaling: Optiona
             inv = yarn_freqs(inv, float(sc["factor"]), rot_dim, float(base), int(sc["original"]),
                              float(sc.get("fast", 32)), float(sc.get("slow", 1)))
             mag = float(sc.get("magnitude", yarn_mscale(float(sc["factor"]))))
+        elif kind == "linear":
+            inv = inv / float(sc["factor"])
         elif kind is not None:
             raise ValueError(f"unknown frequency scaling {kind!r}")
         ang = torch.outer(torch.arange(max_len, dtype=torch.float64), inv)

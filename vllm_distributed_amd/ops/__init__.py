@@ -1552,6 +1552,131 @@ def gated_delta_rule(qkv: torch.Tensor, a_raw: torch.Tensor, b_raw: torch.Tensor
     return out
 
 
+RECURRENT_STEP_TOKENS = 16        # sequences with more new tokens than this take the chunk-parallel forms
+
+
+def gated_delta_rule_head(qkv: torch.Tensor, a_raw: torch.Tensor, b_raw: torch.Tensor, gate: torch.Tensor,
+                          a_log: torch.Tensor, dt_bias: torch.Tensor, norm_w: torch.Tensor, state: torch.Tensor,
+                          query_start_loc: torch.Tensor, seq_lens: torch.Tensor, slot_table: torch.Tensor,
+                          H: int, G: int, D: int, Dv: int, eps: float, max_query_len: int,
+                          first_long_seq: int = 0) -> torch.Tensor:
+    """Gated delta rule with ONE decay per head over a ragged batch (see ops/csrc/delta_rule.hip): g = exp(-exp(a_log) *
+    softplus(a_raw + dt_bias)), output gate silu(gate).  qkv [T, 2*G*D + H*Dv] (convolved q | k | v), a_raw [T, H],
+    b_raw [T, H], gate [T, H*Dv] in the activation type (row strides arbitrary); a_log [H], dt_bias [H], norm_w [Dv]
+    fp32; state fp32 [slots, H, Dv, D] (transposed), updated in place; sequence s uses slot ``slot_table[s, 0]`` and
+    starts from zero when all its tokens are in this batch.  ``first_long_seq``: sequences before it bring at most
+    ``RECURRENT_STEP_TOKENS`` tokens each."""
+    if not _dev(qkv) or D > 1024:
+        return R.gated_delta_rule(qkv, a_raw, b_raw, gate, a_log, dt_bias, norm_w, state, query_start_loc, seq_lens,
+                                  slot_table, H, G, D, Dv, eps, per_head=True)
+    T, S = qkv.shape[0], seq_lens.shape[0]
+    for t, n in ((qkv, 2 * G * D + H * Dv), (a_raw, H), (b_raw, H), (gate, H * Dv)):
+        assert t.stride(1) == 1 and t.dtype == qkv.dtype and t.shape == (T, n)
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, Dv, D)
+    for t, n in ((a_log, H), (dt_bias, H), (norm_w, Dv)):
+        assert t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n
+    out = torch.empty((T, H * Dv), dtype=qkv.dtype, device=qkv.device)
+    o_raw = scratch = None
+    if max_query_len > RECURRENT_STEP_TOKENS and D <= 256 and first_long_seq < S:
+        o_raw = torch.empty((T, H * Dv), dtype=torch.float32, device=qkv.device)
+        scratch = torch.empty(N.lib().vda_delta_head_scratch(T, S - first_long_seq, H, G, D), dtype=torch.float32,
+                              device=qkv.device)
+    N.call("vda_gated_delta_rule_head", out.data_ptr(), out.stride(0), N.ptr(o_raw), N.ptr(scratch), qkv.data_ptr(),
+           qkv.stride(0), a_raw.data_ptr(), a_raw.stride(0), b_raw.data_ptr(), b_raw.stride(0), gate.data_ptr(),
+           gate.stride(0), a_log.data_ptr(), dt_bias.data_ptr(), norm_w.data_ptr(), state.data_ptr(),
+           query_start_loc.data_ptr(), seq_lens.data_ptr(), slot_table.data_ptr(), slot_table.stride(0), T, S,
+           int(first_long_seq), H, G, D, Dv, max(int(max_query_len), 1), float(eps), N.dt(qkv.dtype), N.stream())
+    return out
+
+
+# ---- linear attention with decay ---------------------------------------------------------------------------------
+def linear_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor,
+                     norm_w: Optional[torch.Tensor], state: torch.Tensor, query_start_loc: torch.Tensor,
+                     seq_lens: torch.Tensor, slot_table: torch.Tensor, H: int, D: int, Dv: int, eps: float,
+                     max_query_len: int, *, log_decay: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None,
+                     z_bias: Optional[torch.Tensor] = None, tau: float = 1.0, cos_sin: Optional[torch.Tensor] = None,
+                     positions: Optional[torch.Tensor] = None, rot: int = 0, q_scale: float = 1.0,
+                     k_scale: float = 1.0, first_long_seq: int = 0) -> torch.Tensor:
+    """S <- diag(decay) S + k v^T, o = S^T q per head over a ragged batch, then o / rms(o) * norm_w * silu(gate) (see
+    ops/csrc/linear_attention.hip).  q, k [T, H*D], v, gate [T, H*Dv] in the activation type (row strides arbitrary);
+    the first ``rot`` values of every q / k head are rotated (halves; cos_sin fp32 [positions, rot]), q times q_scale, k
+    times k_scale, all in fp32.  Decay: exp(log_decay[h]) (fp32 [H]) or sigmoid(z + z_bias)^(1 / tau) per key channel
+    (z [T, H*D], z_bias fp32 [H*D] or None).  norm_w fp32 [Dv] or None.  state fp32 [slots, H, Dv, D] (transposed),
+    updated in place; sequence s uses slot ``slot_table[s, 0]`` and starts from zero when all its tokens are in this
+    batch.  ``first_long_seq``: sequences before it bring at most ``RECURRENT_STEP_TOKENS`` tokens each."""
+    if not _dev(q) or D > 1024:
+        return R.linear_attention(q, k, v, gate, norm_w, state, query_start_loc, seq_lens, slot_table, H, D, Dv, eps,
+                                  log_decay, z, z_bias, tau, cos_sin, positions, rot, q_scale, k_scale)
+    T, S = q.shape[0], seq_lens.shape[0]
+    assert (log_decay is None) != (z is None)
+    for t, n in ((q, H * D), (k, H * D), (v, H * Dv), (gate, H * Dv), (z, H * D)):
+        assert t is None or (t.stride(1) == 1 and t.dtype == q.dtype and t.shape == (T, n))
+    for t, n in ((norm_w, Dv), (log_decay, H), (z_bias, H * D)):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n)
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, Dv, D)
+    assert rot == 0 or (cos_sin.dtype == torch.float32 and cos_sin.is_contiguous() and cos_sin.shape[1] == rot
+                        and positions.dtype == torch.int64 and positions.shape[0] >= T)
+    out = torch.empty((T, H * Dv), dtype=q.dtype, device=q.device)
+    o_raw = scratch = None
+    C = 64
+    if max_query_len > RECURRENT_STEP_TOKENS and D <= 256 and first_long_seq < S:
+        fused = bool(N.lib().vda_linear_attention_fused(D, Dv))
+        if not fused:
+            o_raw = torch.empty((T, H * Dv), dtype=torch.float32, device=q.device)
+        if T // 128 * H >= 1024:          # enough workgroups: longer chunks move less state
+            C = 128
+        scratch = torch.empty(N.lib().vda_linear_attention_scratch(T, S - first_long_seq, C, H, D, Dv),
+                              dtype=torch.float32, device=q.device)
+    N.call("vda_linear_attention", out.data_ptr(), out.stride(0), N.ptr(o_raw), N.ptr(scratch), q.data_ptr(), q.stride(0),
+           k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), N.ptr(z), z.stride(0) if z is not None else 0,
+           N.ptr(z_bias), 1.0 / float(tau), N.ptr(log_decay), gate.data_ptr(), gate.stride(0), N.ptr(cos_sin),
+           N.ptr(positions), int(rot), float(q_scale), float(k_scale), N.ptr(norm_w), float(eps), state.data_ptr(),
+           query_start_loc.data_ptr(), seq_lens.data_ptr(), slot_table.data_ptr(), slot_table.stride(0), T, S,
+           int(first_long_seq), H, D, Dv, max(int(max_query_len), 1), C, N.dt(q.dtype), N.stream())
+    return out
+
+
+# ---- fp32 residual under a squashing norm (Dynamic Tanh) ----------------------------------------------------------
+def residual_squash_norm(x: torch.Tensor, branches: list, coef: float, eps: float, alpha: Optional[torch.Tensor],
+                         weight: Optional[torch.Tensor], bias: Optional[torch.Tensor], out_dtype: torch.dtype,
+                         extra: Optional[torch.Tensor] = None, step: Optional[torch.Tensor] = None
+                         ) -> Optional[torch.Tensor]:
+    """One pass over the fp32 residual ``x`` [T, W], in place: x += coef * sum over ``branches`` of y (tuples (y, None)) or
+    y / rms(y) * w (tuples (y, w), w fp32 [W]; at most two branches, y [T, W] in the activation type); then x += ``extra``
+    [T, W] (activation type) and x += ``step`` (fp32 [W]).  With ``weight``: returns tanh(alpha * x) * weight + bias
+    (alpha fp32 of one element, weight and bias fp32 [W]) in ``out_dtype``."""
+    T, W = x.shape
+    if not _dev(x) or len(branches) > 2:
+        return R.residual_squash_norm(x, branches, coef, eps, alpha, weight, bias, out_dtype, extra, step)
+    assert x.dtype == torch.float32 and x.is_contiguous()
+    for y, w in branches:
+        assert y.shape == (T, W) and y.stride(1) == 1 and y.dtype == out_dtype
+        assert w is None or (w.dtype == torch.float32 and w.is_contiguous() and w.numel() == W)
+    assert extra is None or (extra.shape == (T, W) and extra.stride(1) == 1 and extra.dtype == out_dtype)
+    for t, n in ((step, W), (alpha, 1), (weight, W), (bias, W)):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n)
+    h = torch.empty((T, W), dtype=out_dtype, device=x.device) if weight is not None else None
+    args = []
+    for y, w in branches:
+        args += [y.data_ptr(), y.stride(0), N.ptr(w)]
+    args += [None, 0, None] * (2 - len(branches))
+    N.call("vda_residual_squash_norm", x.data_ptr(), len(branches), *args, float(coef), float(eps), N.ptr(extra),
+           extra.stride(0) if extra is not None else 0, N.ptr(step), N.ptr(alpha), N.ptr(weight), N.ptr(bias), N.ptr(h),
+           h.stride(0) if h is not None else 0, T, W, N.dt(out_dtype), N.stream())
+    return h
+
+
+def scaled_softcap(x: torch.Tensor, scale: float = 1.0, cap: float = 0.0) -> torch.Tensor:
+    """cap * tanh(scale * x / cap) in fp32 (cap 0: scale * x), one launch."""
+    if not _dev(x) or x.dim() != 2:
+        return R.scaled_softcap(x, scale, cap)
+    assert x.stride(1) == 1
+    out = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    N.call("vda_scaled_softcap", out.data_ptr(), x.data_ptr(), x.stride(0), x.shape[0], x.shape[1], float(scale),
+           float(cap), N.dt(x.dtype), N.stream())
+    return out
+
+
 # ---- fp32 residual with a norm after and before every sub-layer ------------------------------------------------
 def residual_norms(x: torch.Tensor, y: Optional[torch.Tensor] = None, w_post: Optional[torch.Tensor] = None,
                    w_pre: Optional[torch.Tensor] = None, eps: float = 1e-6, out_dtype: Optional[torch.dtype] = None,
@@ -1724,7 +1849,7 @@ def qk_norm_rope_cache(qkv: torch.Tensor, H: int, G: int, D: int, Dv: int, maps:
                        eps: float, k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor],
                        slot_mapping: torch.Tensor, by_map: bool = False, pairing: str = "halves",
                        q_temp: Optional[tuple] = None, v_first: Optional[torch.Tensor] = None,
-                       v_lam: Optional[torch.Tensor] = None) -> torch.Tensor:
+                       v_lam: Optional[torch.Tensor] = None, whole_norm: bool = False) -> torch.Tensor:
     """qkv [T, >= H*maps*D + G*maps*D + G*Dv] (queries, keys, values side by side; further columns are ignored).  Every
     D-wide map of every query / key head is divided by its root mean square, multiplied by q_weight / k_weight (fp32
     [D]), and its first ``rot`` values are rotated in the half-split layout (value i pairs with i + rot / 2; cos_sin fp32
@@ -1735,12 +1860,16 @@ def qk_norm_rope_cache(qkv: torch.Tensor, H: int, G: int, D: int, Dv: int, maps:
     group) as [T, H * maps, D].
     ``pairing`` "neighbours": the rotation pairs value 2i with 2i + 1 (same table layout).  ``q_temp`` = (coef, every):
     the queries at position p are multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  ``v_first`` [T, G * Dv] (row
-    stride arbitrary) with ``v_lam`` (fp32, one element): the cached values are (1 - lam) v + lam v_first."""
+    stride arbitrary) with ``v_lam`` (fp32, one element): the cached values are (1 - lam) v + lam v_first.
+    ``whole_norm``: all query values of a token are divided by ONE root mean square (and all key values by one), the
+    weights have a value of their own per projection row (q_weight fp32 [H*maps*D], k_weight fp32 [G*maps*D])."""
     used = (H + G) * maps * D + G * Dv
     if not _dev(qkv):
         assert not by_map
         return R.qk_norm_rope_cache(qkv[:, :used], H, G, D, Dv, maps, q_weight, k_weight, cos_sin, positions, rot, eps,
-                                    k_cache, v_cache, slot_mapping, pairing, q_temp, v_first, v_lam)
+                                    k_cache, v_cache, slot_mapping, pairing, q_temp, v_first, v_lam, whole_norm)
+    assert q_weight.numel() == (H * maps * D if whole_norm else D)
+    assert k_weight.numel() == (G * maps * D if whole_norm else D)
     assert pairing in ("halves", "neighbours")
     if v_first is not None:
         assert v_first.dtype == qkv.dtype and v_first.stride(1) == 1 and v_first.shape[0] >= qkv.shape[0] \
@@ -1758,7 +1887,8 @@ def qk_norm_rope_cache(qkv: torch.Tensor, H: int, G: int, D: int, Dv: int, maps:
            k_weight.data_ptr(), N.ptr(cos_sin), positions.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
            slot_mapping.data_ptr(), T, H, G, D, Dv, maps, rot, bs, float(eps), int(by_map),
            int(pairing == "neighbours"), float(q_temp[0]) if q_temp else 0.0, int(q_temp[1]) if q_temp else 0,
-           N.ptr(v_first), v_first.stride(0) if v_first is not None else 0, N.ptr(v_lam), N.dt(qkv.dtype), N.stream())
+           N.ptr(v_first), v_first.stride(0) if v_first is not None else 0, N.ptr(v_lam), int(whole_norm),
+           N.dt(qkv.dtype), N.stream())
     return qn
 
 
@@ -1814,10 +1944,10 @@ def masked_softmax_attention_mfma(qn: torch.Tensor, k_cache: torch.Tensor, v_cac
     if maps == 1 and gate is None:
         return a.view(T, H * Dv)
     out = torch.empty((T, H * Dv), dtype=qn.dtype, device=qn.device)
-    assert gate is None or (gate.dtype == qn.dtype and gate.stride(1) == 1 and gate.shape == (T, H * Dv))
+    assert gate is None or (gate.dtype == qn.dtype and gate.stride(1) == 1 and gate.shape in ((T, H * Dv), (T, H)))
     N.call("vda_map_combine", out.data_ptr(), a.data_ptr(), N.ptr(lam), N.ptr(gate),
-           gate.stride(0) if gate is not None else 0, T, H, G, Dv, int(maps), float(eps), float(out_scale),
-           N.dt(qn.dtype), N.stream())
+           gate.stride(0) if gate is not None else 0, int(gate is not None and gate.shape[1] != H * Dv), T, H, G, Dv,
+           int(maps), float(eps), float(out_scale), N.dt(qn.dtype), N.stream())
     return out
 
 
@@ -1832,7 +1962,8 @@ def masked_softmax_attention(qn: torch.Tensor, k_cache: torch.Tensor, v_cache: t
     v_cache [blocks, G, Dv, bs]).  Key j is visible to the query at position i when j <= i, i - j < window (window > 0)
     and j // chunk == i // chunk (chunk > 0).  ``sink`` fp32 [H]: exp(sink[h]) joins head h's denominator.  maps == 2:
     two score maps per head over the same values, o = a1 - lam * a2 (``lam``: fp32 tensor of one element), then
-    o / rms(o) * out_scale over Dv.  ``gate`` [T, H * Dv] (row stride arbitrary): the result times sigmoid(gate).
+    o / rms(o) * out_scale over Dv.  ``gate`` [T, H * Dv] or [T, H], one number per head (row stride arbitrary): the
+    result times sigmoid(gate).
     ``softcap`` > 0: score <- softcap * tanh(score / softcap).  ``dist_bias`` fp32 [far + 1, H]: row min(i - j, far) joins
     the (capped) scores of every head.
     Returns [T, H * Dv] in ``out_dtype`` (default: qn's type).  Scores, softmax and sums in fp32."""
@@ -1848,12 +1979,12 @@ def masked_softmax_attention(qn: torch.Tensor, k_cache: torch.Tensor, v_cache: t
     assert qn.dtype == k_cache.dtype == v_cache.dtype == out_dtype and k_cache.shape[1:] == (G, bs, MD)
     assert sink is None or (sink.dtype == torch.float32 and sink.numel() == H)
     assert maps == 1 or (lam is not None and lam.dtype == torch.float32 and lam.is_cuda)
-    assert gate is None or (gate.dtype == qn.dtype and gate.stride(1) == 1 and gate.shape[1] == H * Dv)
+    assert gate is None or (gate.dtype == qn.dtype and gate.stride(1) == 1 and gate.shape[1] in (H * Dv, H))
     out = torch.zeros((T, H * Dv), dtype=out_dtype, device=qn.device)
     N.call("vda_masked_softmax_attention", out.data_ptr(), qn.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
            block_table.data_ptr(), block_table.stride(0), seq_lens.data_ptr(), query_start_loc.data_ptr(),
-           N.ptr(sink), N.ptr(lam), N.ptr(gate), gate.stride(0) if gate is not None else 0, float(scale), int(window),
-           int(chunk), int(maps), float(eps), float(out_scale), seq_lens.shape[0], H, G, MD // maps, Dv, bs,
+           N.ptr(sink), N.ptr(lam), N.ptr(gate), gate.stride(0) if gate is not None else 0,
+           int(gate is not None and gate.shape[1] != H * Dv), float(scale), int(window), int(chunk), int(maps), float(eps), float(out_scale), seq_lens.shape[0], H, G, MD // maps, Dv, bs,
            max(int(max_query_len), 1), float(softcap), N.ptr(dist_bias),
            dist_bias.shape[0] - 1 if dist_bias is not None else 0, N.dt(out_dtype), N.stream())
     return out

@@ -15,23 +15,25 @@
 //            over the sixteen lanes with DPP row operations.  The prepared vectors of 32 tokens sit in LDS while
 //            the next 32 are on their way from memory, so a step is one short dependent chain of register work.
 //   epilogue normalises the read-out over the head's columns, applies the weight and the gate.
+// With ONE decay per head (vda_gated_delta_rule_head: g = exp(-exp(a_log) softplus(a + dt_bias)), gate silu) two other
+// kernels do the work:
+//   step     sequences with at most 16 new tokens: one workgroup per (sequence, head) does everything -- unit vectors,
+//            gates, the recurrence token by token with the state read and written once, output norm and gate;
+//   chunked  longer ones, sixteen tokens at a time on the fp32 matrix instruction.  With b the running sum of log g,
+//            M_ij = beta_i e^(b_i - b_j) k_i.k_j (j < i) and T = (I + M)^-1 diag(beta), a block's writes are
+//                U = T (V - diag(e^b) K S),   O = diag(e^b) Q S + P U,   P_ij = e^(b_i - b_j) q_i.k_j (j <= i)
+//                S <- e^b_n S + K^T diag(e^(b_n - b)) U
+//            T, P and the unit vectors of every block are made in parallel (delta_block_prepare); the walk over the blocks
+//            keeps S in the accumulators of one wave per (sequence, head, 16 columns) and passes every product on in
+//            registers (recurrent.h); norm and gate follow in a launch of their own.
 // The batch description is the one of the other recurrent kernels (qsl, seq_lens, slot in column 0 of the table;
 // a sequence carries state in when seq_len - new_tokens > 0), so prompts, portions of prompts, single decoded
 // tokens and mixtures of them are one code path, and the state after a token does not depend on how the
 // sequence was cut.
-#include "common.h"
+#include "recurrent.h"
 
 __device__ __forceinline__ float dr_softplus(float v) { return v > 20.f ? v : log1pf(expf(v)); }
 __device__ __forceinline__ float dr_sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
-
-// sum over the 16 lanes of a DPP row, result in every lane
-__device__ __forceinline__ float row16_sum(float v) {
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x141, 0xF, 0xF, true));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x140, 0xF, 0xF, true));
-  return v;
-}
 
 // grid: tokens; one wave per (token, vector): G query vectors, G key vectors (with their dot products), H decays
 template <typename T>
@@ -293,6 +295,417 @@ VDA_EXPORT int vda_gated_delta_rule(void* out, long o_stride, float* o_raw, floa
   else if (dtype == VDA_F16) L2(f16_t);
   else L2(float);
 #undef L2
+  VDA_CHECK_LAUNCH();
+  return 0;
+}
+
+// ---- one decay per head --------------------------------------------------------------------------------------------
+struct DeltaHeadArgs {
+  const void* qkv;              // [T, 2 G D + H Dv] convolved q | k | v
+  long qkv_stride;
+  const void *a_raw, *b_raw, *gate;
+  long a_stride, b_stride, g_stride;
+  const float *a_log, *dt_bias, *norm_w;
+  float eps;
+  float* state;                 // [slots, H, Dv, D]
+  void* out;
+  long o_stride;
+  float* o_raw;                 // [T, H * Dv]
+  const int *qsl, *seq_lens, *slot_table;
+  long st_stride;
+  int H, G, D, Dv, seq0, limit;
+  float* qhat;                  // [blocks, G, 16, DP]
+  float* khat;                  // [blocks, G, 16, DP]
+  float* khatT;                 // [blocks, G, DP, 16]
+  float* mats;                  // [blocks, H, DELTA_MAT]: T (16 x 16), P (16 x 16), e^b (16), e^(b_n - b) (16)
+};
+#define DELTA_MAT 544
+
+// grid (H, S); columns over groups of sixteen lanes as in lin_step_kernel
+template <typename T, int NR>
+__global__ __launch_bounds__(256) void delta_step_kernel(const DeltaHeadArgs a, const int tile) {
+  constexpr int NCG = NR <= 8 ? 4 : NR <= 16 ? 2 : 1;
+  constexpr int DP = 16 * NR;
+  extern __shared__ __align__(16) float lds[];
+  const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x;
+  const int sl = a.seq_lens[s];
+  if (sl <= 0) return;
+  const int t0 = a.qsl[s], L = a.qsl[s + 1] - t0;
+  if (L <= 0 || L > a.limit) return;
+  const int D = a.D, Dv = a.Dv, G = a.G, c = h / (a.H / G);
+  float* qs = lds;                                     // [tile][DP] unit vectors
+  float* ks = qs + tile * DP;
+  float* vs = ks + tile * DP;                          // [tile][Dv]
+  float* os = vs + tile * Dv;                          // [tile][Dv]
+  float* sc = os + tile * Dv;                          // [tile][4]: decay, beta, q^ . k^
+  const int part = tid & 15, sub = tid >> 4, lane = tid & 63, wave = tid >> 6;
+  const bool carry = sl - L > 0;
+  const bool vs4 = (D & 3) == 0;
+  float* Sb = a.state + ((long)a.slot_table[s * a.st_stride] * a.H + h) * (long)Dv * D;
+  const float q_scale = 1.f / sqrtf((float)D), a_scale = expf(a.a_log[h]), dtb = a.dt_bias[h];
+  const T* qkv = (const T*)a.qkv;
+  float S[NCG][NR];
+  auto load_group = [&](int c0, bool live) {
+#pragma unroll
+    for (int n = 0; n < NCG; ++n) {
+      const int col = c0 + n * 16 + sub;
+      rec_load_column<NR>(S[n], Sb + (long)(col < Dv ? col : Dv - 1) * D, part, D, live && col < Dv, vs4);
+    }
+  };
+  load_group(0, carry);
+  for (int b = 0; b < L; b += tile) {
+    const int nt = min(tile, L - b);
+    if (b > 0) { __syncthreads(); load_group(0, true); }
+    for (int tt = wave; tt < nt; tt += 4) {            // one wave per token: unit vectors and scalars
+      const long t = t0 + b + tt;
+      const T* qr = qkv + t * a.qkv_stride + (long)c * D;
+      const T* kr = qkv + t * a.qkv_stride + (long)(G + c) * D;
+      float sq = 0.f, sk = 0.f, dot = 0.f;
+      for (int d = lane; d < D; d += 64) {
+        const float x = (float)qr[d], y = (float)kr[d];
+        sq += x * x;
+        sk += y * y;
+        dot += x * y;
+      }
+      sq = wave_sum(sq);
+      sk = wave_sum(sk);
+      dot = wave_sum(dot);
+      const float rq = q_scale / sqrtf(sq + 1e-6f), rk = 1.f / sqrtf(sk + 1e-6f);
+      for (int d = lane; d < DP; d += 64) {
+        qs[tt * DP + d] = d < D ? (float)qr[d] * rq : 0.f;
+        ks[tt * DP + d] = d < D ? (float)kr[d] * rk : 0.f;
+      }
+      if (lane == 0) {
+        sc[tt * 4] = expf(-a_scale * rec_softplus((float)((const T*)a.a_raw)[t * a.a_stride + h] + dtb));
+        sc[tt * 4 + 1] = rec_sigmoid((float)((const T*)a.b_raw)[t * a.b_stride + h]);
+        sc[tt * 4 + 2] = dot * rq * rk;
+      }
+    }
+    for (int e = tid; e < nt * Dv; e += 256) {
+      const int tt = e / Dv, cc = e - tt * Dv;
+      vs[e] = (float)qkv[(long)(t0 + b + tt) * a.qkv_stride + (long)2 * G * D + (long)h * Dv + cc];
+    }
+    __syncthreads();
+    for (int c0 = 0; c0 < Dv; c0 += 16 * NCG) {
+      for (int tt = 0; tt < nt; ++tt) {
+        float kr[NR], qr[NR];
+        rec_lane_row<NR>(kr, ks + tt * DP, part);
+        rec_lane_row<NR>(qr, qs + tt * DP, part);
+        const float g = sc[tt * 4], beta = sc[tt * 4 + 1], qk = sc[tt * 4 + 2];
+#pragma unroll
+        for (int n = 0; n < NCG; ++n) {
+          const int col = c0 + n * 16 + sub;
+          float r = 0.f, p = 0.f;
+#pragma unroll
+          for (int i = 0; i < NR; ++i) {
+            S[n][i] *= g;
+            r += S[n][i] * kr[i];
+            p += S[n][i] * qr[i];
+          }
+          r = row16_sum(r);
+          p = row16_sum(p);
+          const float u = beta * (vs[tt * Dv + (col < Dv ? col : Dv - 1)] - r);
+#pragma unroll
+          for (int i = 0; i < NR; ++i) S[n][i] += kr[i] * u;
+          if (part == 0 && col < Dv) os[tt * Dv + col] = p + qk * u;
+        }
+      }
+#pragma unroll
+      for (int n = 0; n < NCG; ++n) {
+        const int col = c0 + n * 16 + sub;
+        if (col < Dv) rec_store_column<NR>(S[n], Sb + (long)col * D, part, D, vs4);
+      }
+      if (c0 + 16 * NCG < Dv) load_group(c0 + 16 * NCG, carry || b > 0);
+    }
+    __syncthreads();
+    for (int tt = wave; tt < nt; tt += 4) {
+      const long t = t0 + b + tt;
+      const float* o = os + tt * Dv;
+      float ss = 0.f;
+      for (int cc = lane; cc < Dv; cc += 64) ss += o[cc] * o[cc];
+      ss = wave_sum(ss);
+      const float rs = 1.f / sqrtf(ss / (float)Dv + a.eps);
+      for (int cc = lane; cc < Dv; cc += 64) {
+        const float zg = (float)((const T*)a.gate)[t * a.g_stride + (long)h * Dv + cc];
+        ((T*)a.out)[t * a.o_stride + (long)h * Dv + cc] = (T)(o[cc] * rs * a.norm_w[cc] * zg * rec_sigmoid(zg));
+      }
+    }
+  }
+}
+
+// Blocks of sixteen tokens counted from every sequence's first new token; block index t0 / 16 + (s - seq0) + block.
+// grid (blocks of the longest sequence, sequences, G): unit vectors of the block's q / k head, then, per value head that
+// reads it, the block's matrices.
+template <typename T, int DT>
+__global__ __launch_bounds__(256) void delta_block_prepare_kernel(const DeltaHeadArgs a) {
+  constexpr int DP = DT * 16, QP = DP + 4;
+  __shared__ __align__(16) float qs[16 * QP], ks[16 * QP];
+  __shared__ float M[4][16 * 17];
+  const int srel = blockIdx.y, s = a.seq0 + srel, tid = threadIdx.x;
+  if (a.seq_lens[s] <= 0) return;
+  const int t0 = a.qsl[s], L = a.qsl[s + 1] - t0, tb = blockIdx.x * 16;
+  if (L <= a.limit || tb >= L) return;
+  const int n = min(16, L - tb), D = a.D, G = a.G, c = blockIdx.z;
+  const int lane = tid & 63, wave = tid >> 6, lo = lane & 15, g = lane >> 4;
+  const long blk = (long)(t0 / 16) + srel + blockIdx.x;
+  const float q_scale = 1.f / sqrtf((float)D);
+  float* qh = a.qhat + (blk * G + c) * 16 * DP;
+  float* kh = a.khat + (blk * G + c) * 16 * DP;
+  float* kt = a.khatT + (blk * G + c) * 16 * DP;
+  for (int tt = wave; tt < 16; tt += 4) {
+    const T* qr = (const T*)a.qkv + (long)(t0 + tb + tt) * a.qkv_stride + (long)c * D;
+    const T* kr = qr + (long)G * D;
+    float sq = 0.f, sk = 0.f;
+    if (tt < n)
+      for (int d = lane; d < D; d += 64) {
+        const float x = (float)qr[d], y = (float)kr[d];
+        sq += x * x;
+        sk += y * y;
+      }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    const float rq = q_scale / sqrtf(sq + 1e-6f), rk = 1.f / sqrtf(sk + 1e-6f);
+    for (int d = lane; d < DP; d += 64) {
+      const bool ok = tt < n && d < D;
+      const float x = ok ? (float)qr[d] * rq : 0.f, y = ok ? (float)kr[d] * rk : 0.f;
+      qs[tt * QP + d] = x;
+      ks[tt * QP + d] = y;
+      qh[tt * DP + d] = x;
+      kh[tt * DP + d] = y;
+    }
+  }
+  __syncthreads();
+  for (int e = tid; e < DP * 4; e += 256) {            // transposed keys, four tokens per store
+    const int d = e >> 2, j = (e & 3) * 4;
+    *reinterpret_cast<f32x4*>(kt + d * 16 + j) =
+        f32x4{ks[j * QP + d], ks[(j + 1) * QP + d], ks[(j + 2) * QP + d], ks[(j + 3) * QP + d]};
+  }
+  // k_i . k_j and q_i . k_j: accumulator register r = [i = 4 g + r][j = lo]
+  f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt) {
+    const f32x4 ka = *reinterpret_cast<const f32x4*>(ks + lo * QP + dt * 16 + 4 * g);
+    const f32x4 qa = *reinterpret_cast<const f32x4*>(qs + lo * QP + dt * 16 + 4 * g);
+    kk = mfma_f32_k16(ka, ka, kk);
+    qk = mfma_f32_k16(qa, ka, qk);
+  }
+  const int rep = a.H / G;
+  float* Mw = M[wave];
+  for (int hh = wave; hh < ((rep + 3) & ~3); hh += 4) {          // every wave makes the same number of turns
+    const bool live = hh < rep;
+    const int h = c * rep + (live ? hh : rep - 1);
+    float* m = a.mats + (blk * a.H + h) * DELTA_MAT;
+    // lane token lo: log decay, running sum over the tokens (all four groups of sixteen lanes alike), beta
+    const long t = t0 + tb + min(lo, n - 1);
+    float b = lo < n ? -expf(a.a_log[h]) * rec_softplus((float)((const T*)a.a_raw)[t * a.a_stride + h] + a.dt_bias[h]) : 0.f;
+    const float beta = lo < n ? rec_sigmoid((float)((const T*)a.b_raw)[t * a.b_stride + h]) : 0.f;
+#pragma unroll
+    for (int o = 1; o < 16; o <<= 1) {
+      const float up = __shfl(b, (lane & 48) | (lo >= o ? lo - o : lo), 64);
+      if (lo >= o) b += up;
+    }
+    const float bn = __shfl(b, 15, 64);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = 4 * g + r;
+      const float bi = __shfl(b, i, 64), betai = __shfl(beta, i, 64);
+      const float f = lo <= i ? expf(bi - b) : 0.f;
+      Mw[i * 17 + lo] = lo < i ? betai * f * kk[r] : 0.f;
+      if (live) m[256 + i * 16 + lo] = f * qk[r];
+    }
+    __syncthreads();
+    // (I + M)^-1, one column per lane by forward substitution, times beta of the column
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == lo ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < i; ++j) v -= Mw[i * 17 + j] * x[j];
+      x[i] = v;
+    }
+    if (live && g == 0) {
+#pragma unroll
+      for (int i = 0; i < 16; ++i) m[i * 16 + lo] = x[i] * beta;
+      m[512 + lo] = expf(b);
+      m[528 + lo] = expf(bn - b);
+    }
+    __syncthreads();
+  }
+}
+
+// grid (column tiles, H, sequences), one wave each: walks the blocks of its sequence with S in accumulators
+template <typename T, int DT>
+__global__ __launch_bounds__(64) void delta_block_walk_kernel(const DeltaHeadArgs a) {
+  constexpr int DP = DT * 16;
+  const int srel = blockIdx.z, s = a.seq0 + srel, lane = threadIdx.x, lo = lane & 15, g = lane >> 4;
+  const int sl = a.seq_lens[s];
+  if (sl <= 0) return;
+  const int t0 = a.qsl[s], L = a.qsl[s + 1] - t0;
+  if (L <= a.limit) return;
+  const int h = blockIdx.y, D = a.D, Dv = a.Dv, H = a.H, G = a.G, c = h / (H / G);
+  const int col = blockIdx.x * 16 + lo;
+  const bool has_col = col < Dv;
+  const bool vs4 = (D & 3) == 0;
+  float* Scol = a.state + (((long)a.slot_table[s * a.st_stride] * H + h) * Dv + (has_col ? col : Dv - 1)) * (long)D;
+  f32x4 S[DT];
+  const bool carry = sl - L > 0;
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt) S[dt] = load4<float>(Scol + dt * 16 + 4 * g, carry ? D - dt * 16 - 4 * g : 0, vs4);
+  const int nb = (L + 15) / 16;
+  const long blk0 = (long)(t0 / 16) + srel;
+  const T* vp = (const T*)a.qkv + (long)t0 * a.qkv_stride + (long)2 * G * D + (long)h * Dv + (has_col ? col : Dv - 1);
+
+  struct Block {
+    f32x4 k[DT], q[DT], kt[DT], tm, pm, eb, ek, v;
+    float en;
+  };
+  auto fetch = [&](Block& f, int bi) {
+    const float* kh = a.khat + ((blk0 + bi) * G + c) * 16 * DP + lo * DP + 4 * g;
+    const float* qh = a.qhat + ((blk0 + bi) * G + c) * 16 * DP + lo * DP + 4 * g;
+    const float* kt = a.khatT + ((blk0 + bi) * G + c) * 16 * DP + lo * 16 + 4 * g;
+    const float* m = a.mats + ((blk0 + bi) * H + h) * DELTA_MAT;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      f.k[dt] = *reinterpret_cast<const f32x4*>(kh + dt * 16);
+      f.q[dt] = *reinterpret_cast<const f32x4*>(qh + dt * 16);
+      f.kt[dt] = *reinterpret_cast<const f32x4*>(kt + dt * 256);
+    }
+    f.tm = *reinterpret_cast<const f32x4*>(m + lo * 16 + 4 * g);
+    f.pm = *reinterpret_cast<const f32x4*>(m + 256 + lo * 16 + 4 * g);
+    f.eb = *reinterpret_cast<const f32x4*>(m + 512 + 4 * g);
+    f.ek = *reinterpret_cast<const f32x4*>(m + 528 + 4 * g);
+    f.en = m[512 + 15];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int tt = bi * 16 + 4 * g + r;
+      f.v[r] = tt < L ? (float)vp[(long)tt * a.qkv_stride] : 0.f;
+    }
+  };
+  auto run = [&](const Block& f, int bi) {
+    f32x4 ka = {0.f, 0.f, 0.f, 0.f}, kb = ka, qa = ka, qb = ka;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      if (dt & 1) {
+        kb = mfma_f32_k16(f.k[dt], S[dt], kb);
+        qb = mfma_f32_k16(f.q[dt], S[dt], qb);
+      } else {
+        ka = mfma_f32_k16(f.k[dt], S[dt], ka);
+        qa = mfma_f32_k16(f.q[dt], S[dt], qa);
+      }
+    }
+    const f32x4 rhs = f.v - f.eb * (ka + kb);
+    f32x4 u = {0.f, 0.f, 0.f, 0.f};
+    u = mfma_f32_k16(f.tm, rhs, u);
+    const f32x4 o = mfma_f32_k16(f.pm, u, f.eb * (qa + qb));
+    u *= f.ek;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) S[dt] = mfma_f32_k16(f.kt[dt], u, S[dt] * f.en);
+    if (has_col) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int tt = bi * 16 + 4 * g + r;
+        if (tt < L) a.o_raw[((long)(t0 + tt) * H + h) * Dv + col] = o[r];
+      }
+    }
+  };
+  if constexpr (DT <= 8) {               // the next block is on its way while this one is computed
+    Block f0, f1;
+    fetch(f0, 0);
+    for (int bi = 0; bi < nb; bi += 2) {
+      if (bi + 1 < nb) fetch(f1, bi + 1);
+      run(f0, bi);
+      if (bi + 2 < nb) fetch(f0, bi + 2);
+      if (bi + 1 < nb) run(f1, bi + 1);
+    }
+  } else {                               // wide keys: the registers hold one block
+    Block f0;
+    for (int bi = 0; bi < nb; ++bi) {
+      fetch(f0, bi);
+      run(f0, bi);
+    }
+  }
+  if (has_col) {
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) store4(Scol + dt * 16 + 4 * g, S[dt], D - dt * 16 - 4 * g, vs4);
+  }
+}
+
+static int delta_dt(int D) { return D <= 32 ? 2 : D <= 64 ? 4 : D <= 128 ? 8 : 16; }
+
+// floats of scratch the chunked form needs for T tokens of S sequences
+VDA_EXPORT long vda_delta_head_scratch(int T, int S, int H, int G, int D) {
+  const long blocks = (long)T / 16 + S + 1;
+  return blocks * ((long)G * 3 * 16 * delta_dt(D) * 16 + (long)H * DELTA_MAT);
+}
+
+VDA_EXPORT int vda_gated_delta_rule_head(void* out, long o_stride, float* o_raw, float* scratch, const void* qkv,
+                                         long qkv_stride, const void* a_raw, long a_stride, const void* b_raw,
+                                         long b_stride, const void* gate, long g_stride, const float* a_log,
+                                         const float* dt_bias, const float* norm_w, float* state, const int* qsl,
+                                         const int* seq_lens, const int* slot_table, long st_stride, int T, int S,
+                                         int seq0, int H, int G, int D, int Dv, int max_q, float eps, int dtype,
+                                         hipStream_t st) {
+  if (S <= 0 || T <= 0) return 0;
+  if (H <= 0 || G <= 0 || H % G || D < 1 || D > 1024 || Dv < 1 || seq0 < 0 || seq0 > S) return -1;
+  const bool chunked = D <= 256 && max_q > 16 && scratch && o_raw && seq0 < S;
+  DeltaHeadArgs a;
+  a.qkv = qkv; a.qkv_stride = qkv_stride; a.a_raw = a_raw; a.b_raw = b_raw; a.gate = gate; a.a_stride = a_stride;
+  a.b_stride = b_stride; a.g_stride = g_stride; a.a_log = a_log; a.dt_bias = dt_bias; a.norm_w = norm_w; a.eps = eps;
+  a.state = state; a.out = out; a.o_stride = o_stride; a.o_raw = o_raw; a.qsl = qsl; a.seq_lens = seq_lens;
+  a.slot_table = slot_table; a.st_stride = st_stride; a.H = H; a.G = G; a.D = D; a.Dv = Dv; a.seq0 = seq0;
+  a.limit = chunked ? 16 : 0x7fffffff;
+  const int DT = delta_dt(D);
+  const long blocks = (long)T / 16 + (S - seq0) + 1;
+  a.qhat = scratch;
+  a.khat = scratch ? a.qhat + blocks * G * 16 * (DT * 16) : nullptr;
+  a.khatT = scratch ? a.khat + blocks * G * 16 * (DT * 16) : nullptr;
+  a.mats = scratch ? a.khatT + blocks * G * 16 * (DT * 16) : nullptr;
+  int NR = 1;
+  while (16 * NR < D) NR *= 2;
+  int tile = max_q < 16 ? max_q : 16;
+  auto step_lds = [&](int tl) { return ((size_t)tl * 2 * 16 * NR + (size_t)2 * tl * Dv + 4 * tl) * 4; };
+  while (tile > 1 && step_lds(tile) > 48 * 1024) tile >>= 1;
+  if (step_lds(tile) > 60 * 1024) return -2;
+  const size_t slds = step_lds(tile);
+#define STEP(TT, NN) hipLaunchKernelGGL((delta_step_kernel<TT, NN>), dim3(H, S), dim3(256), slds, st, a, tile)
+#define STEPS(TT)                                                                                                      \
+  switch (NR) {                                                                                                        \
+    case 1: STEP(TT, 1); break;                                                                                        \
+    case 2: STEP(TT, 2); break;                                                                                        \
+    case 4: STEP(TT, 4); break;                                                                                        \
+    case 8: STEP(TT, 8); break;                                                                                        \
+    case 16: STEP(TT, 16); break;                                                                                      \
+    case 32: STEP(TT, 32); break;                                                                                      \
+    default: STEP(TT, 64); break;                                                                                      \
+  }
+  if (dtype == VDA_BF16) { STEPS(bf16_t) }
+  else if (dtype == VDA_F16) { STEPS(f16_t) }
+  else if (dtype == VDA_F32) { STEPS(float) }
+  else return -3;
+#undef STEPS
+#undef STEP
+  VDA_CHECK_LAUNCH();
+  if (!chunked) return 0;
+  const dim3 gp((max_q + 15) / 16, S - seq0, G), gw((Dv + 15) / 16, H, S - seq0);
+#define CK(TT, DD)                                                                                                     \
+  do {                                                                                                                 \
+    hipLaunchKernelGGL((delta_block_prepare_kernel<TT, DD>), gp, dim3(256), 0, st, a);                                 \
+    hipLaunchKernelGGL((delta_block_walk_kernel<TT, DD>), gw, dim3(64), 0, st, a);                                     \
+  } while (0)
+#define CA(TT) do { if (DT == 2) CK(TT, 2); else if (DT == 4) CK(TT, 4); else if (DT == 8) CK(TT, 8); else CK(TT, 16); } while (0)
+  if (dtype == VDA_BF16) CA(bf16_t);
+  else if (dtype == VDA_F16) CA(f16_t);
+  else CA(float);
+#undef CA
+#undef CK
+  VDA_CHECK_LAUNCH();
+  const dim3 ge((unsigned)(((long)max_q * H + 3) / 4), S - seq0);
+#define EP(TT) hipLaunchKernelGGL((head_norm_silu_kernel<TT>), ge, dim3(256), 0, st, (TT*)out, o_stride, o_raw,        \
+                                  (const TT*)gate, g_stride, norm_w, qsl, seq_lens, seq0, a.limit, H, Dv, eps)
+  if (dtype == VDA_BF16) EP(bf16_t);
+  else if (dtype == VDA_F16) EP(f16_t);
+  else EP(float);
+#undef EP
   VDA_CHECK_LAUNCH();
   return 0;
 }

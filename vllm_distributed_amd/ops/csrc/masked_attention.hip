@@ -1,7 +1,8 @@
 // Softmax attention on the paged cache with the pieces several decoder designs combine freely:
 //   * per-head RMS norms of queries and keys with a learned weight, then a rotation of the first `rot` values of a
 //     head, value i paired with value i + rot / 2 (half-split) or value 2i with 2i + 1 (neighbours), angles from an
-//     fp32 cos | sin table;
+//     fp32 cos | sin table; or ONE norm over all query heads of a token and one over all key heads (`whole`), with
+//     weights as long as the projections;
 //   * a query temperature: queries at position p times 1 + coef * ln(floor((p + 1) / every) + 1);
 //   * value mixing: v <- (1 - lam) v + lam v_first with the values another layer made of the same token, before the
 //     cache write;
@@ -13,7 +14,7 @@
 //   * masks: causal, and on top a sliding window (i - j < window) and / or chunks counted from the sequence's start
 //     (j / chunk == i / chunk);
 //   * a sink per head: exp(sink[h]) joins the softmax denominator, with no key and no value;
-//   * an output gate: the result times the sigmoid of a second projection.
+//   * an output gate: the result times the sigmoid of a second projection, per value or one number per head.
 //
 // Cache layout: k_cache [blocks, G, bs, maps * D] (a head's maps side by side in one row), v_cache [blocks, G, Dv, bs].
 // For the matrix-core kernels of attention.hip every map is a key head of its own instead (`by_map`): k_cache
@@ -38,7 +39,26 @@ struct QkExtras {
   const void* v_first;     // [T, G * Dv] values of the same tokens from an earlier layer, or null
   long v_first_stride;
   const float* v_lam;      // one value: v <- (1 - lam) v + lam v_first
+  int whole;               // one norm over all queries, one over all keys; q_w, k_w as long as the projections
 };
+
+// 1 / rms of all query values and of all key values of a token (q | k side by side in `row`), every thread of the block
+template <typename T>
+__device__ __forceinline__ void whole_row_norms(const T* row, int q_len, int k_len, float eps, float& rq, float& rk) {
+  __shared__ float red[2][4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  float sq = 0.f, sk = 0.f;
+  for (int e = tid; e < q_len; e += 256) { const float v = (float)row[e]; sq += v * v; }
+  for (int e = tid; e < k_len; e += 256) { const float v = (float)row[q_len + e]; sk += v * v; }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if (lane == 0) { red[0][wave] = sq; red[1][wave] = sk; }
+  __syncthreads();
+  sq = red[0][0] + red[0][1] + red[0][2] + red[0][3];
+  sk = red[1][0] + red[1][1] + red[1][2] + red[1][3];
+  rq = 1.f / sqrtf(sq / (float)q_len + eps);
+  rk = 1.f / sqrtf(sk / (float)k_len + eps);
+}
 
 __device__ __forceinline__ float query_temperature(const QkExtras& x, long p) {
   if (x.q_every <= 0) return 1.f;
@@ -66,18 +86,23 @@ __global__ __launch_bounds__(256) void qk_norm_rope_cache_kernel(
   const long slot = slot_mapping[t];
   const float qt = query_temperature(x, positions[t]);
   const int nq = H * maps, nk = G * maps;
+  float rq = 1.f, rk = 1.f;
+  if (x.whole) whole_row_norms<T>(row, nq * D, nk * D, eps, rq, rk);
   // one wave per D-wide unit: the query maps first, then the key maps
   for (int u = wave; u < nq + nk; u += 4) {
     const bool is_q = u < nq;
     const T* src = row + (long)u * D;             // q units and k units are contiguous in the row
-    const float* w = is_q ? q_w : k_w;
-    float ss = 0.f;
-    for (int d = lane; d < D; d += 64) {
-      const float v = (float)src[d];
-      ss += v * v;
+    const float* w = (is_q ? q_w : k_w) + (x.whole ? (long)(is_q ? u : u - nq) * D : 0);
+    float rs = is_q ? rq : rk;
+    if (!x.whole) {
+      float ss = 0.f;
+      for (int d = lane; d < D; d += 64) {
+        const float v = (float)src[d];
+        ss += v * v;
+      }
+      ss = wave_sum(ss);
+      rs = 1.f / sqrtf(ss / (float)D + eps);
     }
-    ss = wave_sum(ss);
-    const float rs = 1.f / sqrtf(ss / (float)D + eps);
     T* dst;
     if (is_q) {
       int uo = u;                                 // query unit = head * maps + map
@@ -132,19 +157,21 @@ __global__ __launch_bounds__(256) void qk_norm_rope_cache_vec_kernel(
   const long slot = slot_mapping[t];
   const float qt = query_temperature(xo, positions[t]);
   const int nq = H * maps, nk = G * maps, total = nq + nk;
+  float rq = 1.f, rk = 1.f;
+  if (xo.whole) whole_row_norms<T>(row, nq * D, nk * D, eps, rq, rk);
   for (int u0 = 0; u0 < total; u0 += UPB) {
     const int u = u0 + tid / LPU;
     const bool live = u < total;
     const int uc = live ? u : total - 1;
     const bool is_q = uc < nq;
     const V8 v = ld16<V8>(row + (long)uc * D + d0);
-    const float* w = (is_q ? q_w : k_w) + d0;
+    const float* w = (is_q ? q_w : k_w) + d0 + (xo.whole ? (long)(is_q ? uc : uc - nq) * D : 0);
     float x[8], ss = 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) { x[i] = (float)v[i]; ss += x[i] * x[i]; }
 #pragma unroll
     for (int o = LPU / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
-    const float rs = 1.f / sqrtf(ss / (float)D + eps);
+    const float rs = xo.whole ? (is_q ? rq : rk) : 1.f / sqrtf(ss / (float)D + eps);
 #pragma unroll
     for (int i = 0; i < 8; ++i) x[i] *= rs * w[i];
     if (rot > 0 && xo.neighbours) {                  // uniform: a pair sits in one lane
@@ -204,11 +231,11 @@ VDA_EXPORT int vda_qk_norm_rope_cache(void* qn, const void* qkv, long qkv_stride
                                       const float* cos_sin, const long* positions, void* k_cache, void* v_cache,
                                       const long* slot_mapping, int T, int H, int G, int D, int Dv, int maps, int rot,
                                       int bs, float eps, int by_map, int neighbours, float q_coef, int q_every,
-                                      const void* v_first, long v_first_stride, const float* v_lam, int dtype,
-                                      hipStream_t st) {
+                                      const void* v_first, long v_first_stride, const float* v_lam, int whole,
+                                      int dtype, hipStream_t st) {
   if (T <= 0) return 0;
   if (rot < 0 || rot > D || (rot & 1) || maps < 1 || (rot > 0 && !cos_sin) || (v_first && !v_lam)) return -1;
-  const QkExtras xo{neighbours, q_coef, q_every, v_first, v_first_stride, v_lam};
+  const QkExtras xo{neighbours, q_coef, q_every, v_first, v_first_stride, v_lam, whole};
   // half-split pairs: the partner sits rot / 16 lanes away; neighbours: inside the lane's own eight values
   const bool vec = (D == 32 || D == 64 || D == 128 || D == 256) && (neighbours ? rot % 8 == 0 : (rot / 2) % 8 == 0) &&
                    qkv_stride % 8 == 0 &&
@@ -250,8 +277,9 @@ struct MaskedAttnArgs {
   const int* qsl;
   const float* sink;         // [H] or null
   const float* lam;          // one value (maps == 2)
-  const void* gate;          // [T, H * Dv] pre-activations or null
+  const void* gate;          // [T, H * Dv] or [T, H] (gate_heads) pre-activations or null
   long gate_stride;
+  int gate_heads;            // one gate per head
   const float* dist_bias;    // [far + 1, H] or null: row min(i - j, far) joins the scores
   int far;
   float scale, eps, out_scale, softcap;
@@ -431,7 +459,7 @@ __global__ __launch_bounds__(256) void masked_softmax_attention_kernel(const Mas
     }
     for (int d = lane; d < Dv; d += 64) {
       float o = maps == 2 ? (a1[d] - lam * a1[Dv + d]) * rsn : a1[d];
-      if (gate) o *= 1.f / (1.f + expf(-(float)gate[tok * a.gate_stride + col + d]));
+      if (gate) o *= 1.f / (1.f + expf(-(float)gate[tok * a.gate_stride + (a.gate_heads ? h0 + hl : col + d)]));
       out[tok * ((long)a.H * Dv) + col + d] = (T)o;
     }
   }
@@ -440,8 +468,8 @@ __global__ __launch_bounds__(256) void masked_softmax_attention_kernel(const Mas
 VDA_EXPORT int vda_masked_softmax_attention(void* out, const void* qn, const void* k_cache, const void* v_cache,
                                             const int* block_table, long bt_stride, const int* seq_lens,
                                             const int* qsl, const float* sink, const float* lam, const void* gate,
-                                            long gate_stride, float scale, int window, int chunk, int maps, float eps,
-                                            float out_scale, int S, int H, int G, int D, int Dv, int bs, int max_q,
+                                            long gate_stride, int gate_heads, float scale, int window, int chunk,
+                                            int maps, float eps, float out_scale, int S, int H, int G, int D, int Dv, int bs, int max_q,
                                             float softcap, const float* dist_bias, int far, int dtype,
                                             hipStream_t st) {
   if (S <= 0 || max_q <= 0) return 0;
@@ -477,7 +505,7 @@ VDA_EXPORT int vda_masked_softmax_attention(void* out, const void* qn, const voi
   MaskedAttnArgs a;
   a.out = out; a.qn = qn; a.k_cache = k_cache; a.v_cache = v_cache; a.block_table = block_table;
   a.bt_stride = bt_stride; a.seq_lens = seq_lens; a.qsl = qsl; a.sink = sink; a.lam = lam; a.gate = gate;
-  a.gate_stride = gate_stride; a.scale = scale; a.eps = eps; a.out_scale = out_scale; a.window = window;
+  a.gate_stride = gate_stride; a.gate_heads = gate_heads; a.scale = scale; a.eps = eps; a.out_scale = out_scale; a.window = window;
   a.chunk = chunk; a.maps = maps; a.H = H; a.G = G; a.D = D; a.Dv = Dv; a.bs = bs; a.HG = HG; a.BQ = BQ; a.BK = BK;
   a.softcap = softcap; a.dist_bias = dist_bias; a.far = far;
   dim3 grid((max_q + BQ - 1) / BQ, S, G * ((R + HG - 1) / HG)), block(256);
@@ -510,7 +538,7 @@ VDA_EXPORT int vda_masked_softmax_attention(void* out, const void* qn, const voi
 template <typename T>
 __global__ __launch_bounds__(256) void map_combine_kernel(T* __restrict__ out, const T* __restrict__ a,
                                                           const float* __restrict__ lam_p, const T* __restrict__ gate,
-                                                          long gate_stride, long n_rows, int H, int G, int Dv,
+                                                          long gate_stride, int gate_heads, long n_rows, int H, int G, int Dv,
                                                           int maps, float eps, float out_scale) {
   const long row = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= n_rows) return;
@@ -532,18 +560,18 @@ __global__ __launch_bounds__(256) void map_combine_kernel(T* __restrict__ out, c
   }
   for (int d = lane; d < Dv; d += 64) {
     float o = maps == 2 ? ((float)a1[d] - lam * (float)a2[d]) * rsn : (float)a1[d];
-    if (gate) o *= 1.f / (1.f + expf(-(float)gate[t * gate_stride + (long)h * Dv + d]));
+    if (gate) o *= 1.f / (1.f + expf(-(float)gate[t * gate_stride + (gate_heads ? (long)h : (long)h * Dv + d)]));
     out[row * Dv + d] = (T)o;
   }
 }
 
-VDA_EXPORT int vda_map_combine(void* out, const void* a, const float* lam, const void* gate, long gate_stride, int T,
-                               int H, int G, int Dv, int maps, float eps, float out_scale, int dtype, hipStream_t st) {
+VDA_EXPORT int vda_map_combine(void* out, const void* a, const float* lam, const void* gate, long gate_stride,
+                               int gate_heads, int T, int H, int G, int Dv, int maps, float eps, float out_scale, int dtype, hipStream_t st) {
   if (T <= 0) return 0;
   if (H % G || maps < 1 || maps > 2 || (maps == 2 && !lam)) return -1;
   const long rows = (long)T * H;
 #define L(TT) hipLaunchKernelGGL((map_combine_kernel<TT>), dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, st,         \
-                                 (TT*)out, (const TT*)a, lam, (const TT*)gate, gate_stride, rows, H, G, Dv, maps, eps, \
+                                 (TT*)out, (const TT*)a, lam, (const TT*)gate, gate_stride, gate_heads, rows, H, G, Dv, maps, eps, \
                                  out_scale)
   if (dtype == VDA_BF16) L(bf16_t);
   else if (dtype == VDA_F16) L(f16_t);

@@ -748,3 +748,173 @@ VDA_EXPORT int vda_fp32_rows_dot(float* out, const void* x, long x_stride, const
   VDA_CHECK_LAUNCH();
   return 0;
 }
+
+// fp32 residual under a squashing norm (no statistics): one pass over the row,
+//     x += coef * sum over the sub-layer's branches of (y  or  y / rms(y) * w)      in place
+//     x += extra (a row in the activation type) + step (one fp32 row for all tokens)
+//     h  = tanh(alpha * x) * nw + nb                                                 the next sub-layer's input
+// Branches with a weight are divided by their root mean square over the row first (two parallel mixers whose outputs are
+// normed before they are summed); their rows are read once for the sums and, from cache, once more for the update.
+struct SquashArgs {
+  float* x;
+  const void* y[2];
+  long y_stride[2];
+  const float* w[2];
+  int nbranch;
+  float coef, eps;
+  const void* extra;
+  long extra_stride;
+  const float* step;
+  const float* alpha;
+  const float* nw;
+  const float* nb;
+  void* h;
+  long h_stride;
+  int W;
+};
+
+// tanh through one exponential: 1 - 2 / (e^2z + 1), with the odd series where the difference would cancel
+__device__ __forceinline__ float squash_tanh(float z) {
+  const float a = fabsf(z);
+  if (a < 0.25f) {
+    const float q = z * z;
+    return z * (1.f + q * (-0.33333334f + q * (0.13333334f + q * (-0.053968254f + q * (0.021869488f - q * 0.008863236f)))));
+  }
+  const float e = expf(fminf(2.f * a, 80.f));
+  return copysignf(1.f - 2.f / (e + 1.f), z);
+}
+
+template <typename T, int VEC, int BLOCK>
+__global__ __launch_bounds__(BLOCK) void residual_squash_norm_kernel(const SquashArgs a) {
+  using V = T __attribute__((ext_vector_type(VEC)));
+  using F = float __attribute__((ext_vector_type(VEC)));
+  __shared__ float red[2][BLOCK / 64];
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x, W = a.W;
+  float rs[2] = {1.f, 1.f};
+  bool any = false;
+  for (int b = 0; b < a.nbranch; ++b) any |= a.w[b] != nullptr;
+  if (any) {
+    for (int b = 0; b < a.nbranch; ++b) {
+      if (!a.w[b]) continue;
+      const T* yr = (const T*)a.y[b] + t * a.y_stride[b];
+      float ss = 0.f;
+      for (int c = tid * VEC; c < W; c += BLOCK * VEC) {
+        const V v = *reinterpret_cast<const V*>(yr + c);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) ss += (float)v[i] * (float)v[i];
+      }
+      ss = wave_sum(ss);
+      if ((tid & 63) == 0) red[b][tid >> 6] = ss;
+    }
+    __syncthreads();
+    for (int b = 0; b < a.nbranch; ++b) {
+      if (!a.w[b]) continue;
+      float ss = 0.f;
+#pragma unroll
+      for (int k = 0; k < BLOCK / 64; ++k) ss += red[b][k];
+      rs[b] = 1.f / sqrtf(ss / (float)W + a.eps);
+    }
+  }
+  const float al = a.h ? *a.alpha : 0.f;
+  float* xr = a.x + t * W;
+  for (int c = tid * VEC; c < W; c += BLOCK * VEC) {
+    F x = *reinterpret_cast<const F*>(xr + c);
+    F add;
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) add[i] = 0.f;
+    for (int b = 0; b < a.nbranch; ++b) {
+      const V y = *reinterpret_cast<const V*>((const T*)a.y[b] + t * a.y_stride[b] + c);
+      if (a.w[b]) {
+        const F w = *reinterpret_cast<const F*>(a.w[b] + c);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) add[i] += (float)y[i] * rs[b] * w[i];
+      } else {
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) add[i] += (float)y[i];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) x[i] += a.coef * add[i];
+    if (a.extra) {
+      const V e = *reinterpret_cast<const V*>((const T*)a.extra + t * a.extra_stride + c);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) x[i] += (float)e[i];
+    }
+    if (a.step) {
+      const F e = *reinterpret_cast<const F*>(a.step + c);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) x[i] += e[i];
+    }
+    if (a.nbranch > 0 || a.extra || a.step) *reinterpret_cast<F*>(xr + c) = x;
+    if (a.h) {
+      const F w = *reinterpret_cast<const F*>(a.nw + c), bb = *reinterpret_cast<const F*>(a.nb + c);
+      V o;
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) o[i] = (T)(squash_tanh(al * x[i]) * w[i] + bb[i]);
+      *reinterpret_cast<V*>((T*)a.h + t * a.h_stride + c) = o;
+    }
+  }
+}
+
+VDA_EXPORT int vda_residual_squash_norm(float* x, int nbranch, const void* y0, long y0_stride, const float* w0,
+                                        const void* y1, long y1_stride, const float* w1, float coef, float eps,
+                                        const void* extra, long extra_stride, const float* step, const float* alpha,
+                                        const float* nw, const float* nb, void* h, long h_stride, int T, int W,
+                                        int dtype, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (nbranch < 0 || nbranch > 2 || (nbranch > 0 && !y0) || (nbranch > 1 && !y1) || (h && (!alpha || !nw || !nb)))
+    return -1;
+  const SquashArgs a{x, {y0, y1}, {y0_stride, y1_stride}, {w0, w1}, nbranch, coef, eps, extra, extra_stride, step,
+                     alpha, nw, nb, h, h_stride, W};
+  const uintptr_t al = dtype == VDA_F32 ? 16 : 8;          // four values of the activation type
+  const bool vec = W % 4 == 0 && y0_stride % 4 == 0 && y1_stride % 4 == 0 && extra_stride % 4 == 0 &&
+                   h_stride % 4 == 0 && !((uintptr_t)y0 % al) && !((uintptr_t)y1 % al) && !((uintptr_t)extra % al) &&
+                   !((uintptr_t)h % al) && !((uintptr_t)x % 16) && !((uintptr_t)w0 % 16) && !((uintptr_t)w1 % 16) &&
+                   !((uintptr_t)step % 16) && !((uintptr_t)nw % 16) && !((uintptr_t)nb % 16);
+#define L3(TT, VV, BB) hipLaunchKernelGGL((residual_squash_norm_kernel<TT, VV, BB>), dim3(T), dim3(BB), 0, st, a)
+#define L(TT)                                                          \
+  do {                                                                 \
+    if (vec && W <= 512) L3(TT, 4, 128);                               \
+    else if (vec) L3(TT, 4, 256);                                      \
+    else L3(TT, 1, 256);                                               \
+  } while (0)
+  if (dtype == VDA_BF16) L(bf16_t);
+  else if (dtype == VDA_F16) L(f16_t);
+  else if (dtype == VDA_F32) L(float);
+  else return -3;
+#undef L
+#undef L3
+  VDA_CHECK_LAUNCH();
+  return 0;
+}
+
+// out = cap * tanh(scale * in / cap) in fp32 (cap <= 0: scale * in): logits on their way to the sampler
+template <typename T>
+__global__ __launch_bounds__(256) void scaled_softcap_kernel(float* __restrict__ out, const T* __restrict__ in,
+                                                             long in_stride, long rows, int cols, float scale,
+                                                             float cap) {
+  const long n = rows * cols;
+  const float k = cap > 0.f ? scale / cap : scale;
+  for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) {
+    const long r = i / cols;
+    const float v = (float)in[r * in_stride + (i - r * cols)] * k;
+    out[i] = cap > 0.f ? cap * squash_tanh(v) : v;
+  }
+}
+
+VDA_EXPORT int vda_scaled_softcap(float* out, const void* in, long in_stride, long rows, int cols, float scale,
+                                  float cap, int dtype, hipStream_t st) {
+  if (rows <= 0 || cols <= 0) return 0;
+  const long blocks = (rows * cols + 255) / 256;
+  const dim3 grid((unsigned)(blocks > 4096 ? 4096 : blocks));
+#define L(TT) hipLaunchKernelGGL((scaled_softcap_kernel<TT>), grid, dim3(256), 0, st, out, (const TT*)in, in_stride, \
+                                 rows, cols, scale, cap)
+  if (dtype == VDA_BF16) L(bf16_t);
+  else if (dtype == VDA_F16) L(f16_t);
+  else if (dtype == VDA_F32) L(float);
+  else return -3;
+#undef L
+  VDA_CHECK_LAUNCH();
+  return 0;
+}

@@ -70,10 +70,10 @@ _SIGS = {
     "vda_moe_pairs": [P, L, P, P, L, P, P, P, P, I, I, I, I, I, I, F, I, I, P],
     "vda_residual_layer_norm": [P, P, L, P, P, P, L, F, I, I, I, P, L, P, L, P],
     "vda_fp32_rows_dot": [P, P, L, P, P, I, I, I, I, P],
-    "vda_qk_norm_rope_cache": [P, P, L, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, I, F, I, P, L, P, I, P],
-    "vda_map_combine": [P, P, P, P, L, I, I, I, I, I, F, F, I, P],
-    "vda_masked_softmax_attention": [P, P, P, P, P, L, P, P, P, P, P, L, F, I, I, I, F, F, I, I, I, I, I, I, I, F, P, I,
-                                     I, P],
+    "vda_qk_norm_rope_cache": [P, P, L, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, I, F, I, P, L, P, I, I, P],
+    "vda_map_combine": [P, P, P, P, L, I, I, I, I, I, I, F, F, I, P],
+    "vda_masked_softmax_attention": [P, P, P, P, P, L, P, P, P, P, P, L, I, F, I, I, I, F, F, I, I, I, I, I, I, I, F, P,
+                                     I, I, P],
     "vda_moe_gate_up": [P, P, P, P, P, P, I, I, I, I, I, L, I, I, I, I, F, P],
     "vda_moe_down": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
     "vda_moe_up_act": [P, P, P, P, P, I, I, I, I, I, L, I, I, I, P],
@@ -108,9 +108,21 @@ _SIGS = {
     "vda_sigmoid_attention_mfma_ok": [I, I, I, I, I, I],
     "vda_gated_delta_rule": [P, L, P, P, P, L, P, L, P, L, P, L, P, P, P, P, P, P, P, L, I, I, I, I, I, I, F, I, P],
     "vda_delta_rule_padded_dim": [I],
+    "vda_gated_delta_rule_head": [P, L, P, P, P, L, P, L, P, L, P, L, P, P, P, P, P, P, P, L, I, I, I, I, I, I, I, I, F,
+                                  I, P],
+    "vda_delta_head_scratch": [I, I, I, I, I],
+    "vda_linear_attention": [P, L, P, P, P, L, P, L, P, L, P, L, P, F, P, P, L, P, P, I, F, F, P, F, P, P, P, P, L, I, I, I,
+                             I, I, I, I, I, I, P],
+    "vda_linear_attention_scratch": [I, I, I, I, I, I],
+    "vda_linear_attention_fused": [I, I],
+    "vda_residual_squash_norm": [P, I, P, L, P, P, L, P, F, F, P, L, P, P, P, P, P, L, I, I, I, P],
+    "vda_scaled_softcap": [P, P, L, L, I, F, F, I, P],
     "vda_selective_scan": [P, P, P, P, P, P, P, P, P, P, P, P, P, L, I, I, I, L, L, L, L, L, L, I, I, I, I, I, I, P, P,
                            I, P],
 }
+
+# functions that answer with a size instead of a status
+_LONG_RESULTS = ("vda_delta_head_scratch", "vda_linear_attention_scratch")
 
 
 def library_path() -> str:
@@ -135,7 +147,7 @@ def lib() -> ctypes.CDLL:
             if fn is None:
                 continue       # optional symbol (e.g. MoE kernels are registered by their module)
             fn.argtypes = sig
-            fn.restype = c_int
+            fn.restype = c_long if name in _LONG_RESULTS else c_int
     return _LIB
 
 

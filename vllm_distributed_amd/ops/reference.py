@@ -665,12 +665,13 @@ def sigmoid_window_attention(qn, k_cache, v_cache, block_table, seq_lens, qsl, t
 
 # ---- gated delta rule with one decay per key channel ---------------------------------------------------
 def gated_delta_rule(qkv, a_raw, b_raw, gate_raw, a_log, dt_bias, norm_w, state, qsl, seq_lens, slot_table,
-                     H: int, G: int, D: int, Dv: int, eps: float):
+                     H: int, G: int, D: int, Dv: int, eps: float, per_head: bool = False):
     """qkv [T, 2*G*D + H*Dv] (after the short convolution), a_raw [T, H*D], b_raw [T, H], gate_raw [T, H*Dv];
     state fp32 [slots, H, Dv, D] (S transposed), updated in place.  Per token and head (q, k of head h // (H / G)):
     q <- q / sqrt(|q|^2 + 1e-6) / sqrt(D), k <- k / sqrt(|k|^2 + 1e-6), decay = exp(-exp(a_log[h]) *
     softplus(a_raw + dt_bias)); S <- decay[:, None] * S; u = sigmoid(b) * (v - S^T k); S <- S + k u^T; o = S^T q;
-    out = o / rms(o) * norm_w * sigmoid(gate_raw)."""
+    out = o / rms(o) * norm_w * sigmoid(gate_raw).
+    ``per_head``: one decay per head (a_raw [T, H], dt_bias [H]) and silu(gate_raw) as the output gate."""
     T = qkv.shape[0]
     out = torch.zeros((T, H, Dv), dtype=torch.float32, device=qkv.device)
     rep = H // G
@@ -682,7 +683,7 @@ def gated_delta_rule(qkv, a_raw, b_raw, gate_raw, a_log, dt_bias, norm_w, state,
     q, k = q.repeat_interleave(rep, 1), k.repeat_interleave(rep, 1)
     beta = torch.sigmoid(b_raw.float())
     decay = torch.exp(-torch.exp(a_log.float()).view(1, H, 1)
-                      * torch.nn.functional.softplus(a_raw.float() + dt_bias.float()).view(T, H, D))
+                      * torch.nn.functional.softplus(a_raw.float() + dt_bias.float()).view(T, H, 1 if per_head else D))
     for s in range(seq_lens.shape[0]):
         sl = int(seq_lens[s])
         t0, t1 = int(qsl[s]), int(qsl[s + 1])
@@ -698,8 +699,73 @@ def gated_delta_rule(qkv, a_raw, b_raw, gate_raw, a_log, dt_bias, norm_w, state,
             out[t] = torch.einsum("hdv,hd->hv", S, q[t])
         state[slot] = S.transpose(1, 2)
     o = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()
-    o = o * torch.sigmoid(gate_raw.float().view(T, H, Dv))
+    z = gate_raw.float().view(T, H, Dv)
+    o = o * (F.silu(z) if per_head else torch.sigmoid(z))
     return o.view(T, H * Dv).to(qkv.dtype)
+
+
+# ---- linear attention with decay ---------------------------------------------------------------------------------
+def linear_attention(q, k, v, gate, norm_w, state, qsl, seq_lens, slot_table, H: int, D: int, Dv: int, eps: float,
+                     log_decay, z, z_bias, tau: float, cos_sin, positions, rot: int, q_scale: float, k_scale: float):
+    """q, k [T, H*D], v, gate [T, H*Dv]; state fp32 [slots, H, Dv, D] (S transposed), updated in place.  q and k rotated
+    (halves) and scaled in fp32; per token and head S <- diag(decay) S + k v^T, o = S^T q with decay =
+    exp(log_decay[h]) or sigmoid(z + z_bias)^(1 / tau) per key channel; out = o / rms(o) * norm_w * silu(gate)."""
+    T = q.shape[0]
+    qf, kf = q.float().reshape(T, H, D), k.float().reshape(T, H, D)
+    vf = v.float().reshape(T, H, Dv)
+    if rot > 0:
+        cs = cos_sin[positions[:T].long()]
+        cos, sin = cs[:, None, : rot // 2], cs[:, None, rot // 2: rot]
+        qf, kf = rotate_halves(qf, cos, sin, rot), rotate_halves(kf, cos, sin, rot)
+    qf, kf = qf * q_scale, kf * k_scale
+    if z is not None:
+        zf = z.float() + (z_bias.float() if z_bias is not None else 0.0)
+        decay = torch.exp(F.logsigmoid(zf) / tau).view(T, H, D)
+    else:
+        decay = torch.exp(log_decay.float()).view(1, H, 1).expand(T, H, D)
+    out = torch.zeros((T, H, Dv), dtype=torch.float32, device=q.device)
+    for s in range(seq_lens.shape[0]):
+        sl = int(seq_lens[s])
+        t0, t1 = int(qsl[s]), int(qsl[s + 1])
+        if sl <= 0 or t1 <= t0:
+            continue
+        slot = int(slot_table[s, 0])
+        S = state[slot].transpose(1, 2).clone() if sl - (t1 - t0) > 0 else \
+            torch.zeros((H, D, Dv), dtype=torch.float32, device=q.device)
+        for t in range(t0, t1):
+            S = decay[t].unsqueeze(-1) * S + kf[t].unsqueeze(-1) * vf[t].unsqueeze(1)
+            out[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+        state[slot] = S.transpose(1, 2)
+    o = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps)
+    if norm_w is not None:
+        o = o * norm_w.float()
+    return (o.view(T, H * Dv) * F.silu(gate.float())).to(q.dtype)
+
+
+# ---- fp32 residual under a squashing norm -----------------------------------------------------------------------
+def residual_squash_norm(x, branches, coef: float, eps: float, alpha, weight, bias, out_dtype, extra=None, step=None):
+    """x fp32 [T, W], in place: x += coef * sum of the branches (y, w): y, or y / rms(y) * w; x += extra + step; with
+    ``weight`` returns tanh(alpha * x) * weight + bias in ``out_dtype``."""
+    total = None
+    for y, w in branches:
+        f = y.float()
+        if w is not None:
+            f = f * torch.rsqrt(f.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+        total = f if total is None else total + f
+    if total is not None:
+        x += coef * total
+    if extra is not None:
+        x += extra.float()
+    if step is not None:
+        x += step.float()
+    if weight is None:
+        return None
+    return (torch.tanh(alpha.float() * x) * weight.float() + bias.float()).to(out_dtype)
+
+
+def scaled_softcap(x, scale: float, cap: float):
+    f = x.float() * scale
+    return cap * torch.tanh(f / cap) if cap > 0 else f
 
 
 # ---- fp32 residual with a norm after and before every sub-layer ---------------------------------------------
@@ -878,7 +944,7 @@ def position_temperature(positions, coef: float, every: int):
 
 def qk_norm_rope_cache(qkv, H: int, G: int, D: int, Dv: int, maps: int, q_weight, k_weight, cos_sin, positions,
                        rot: int, eps: float, k_cache, v_cache, slot_mapping, pairing: str = "halves", q_temp=None,
-                       v_first=None, v_lam=None):
+                       v_first=None, v_lam=None, whole_norm: bool = False):
     """qkv [T, H*maps*D + G*maps*D + G*Dv].  Every D-wide map of every query / key head is divided by its root mean
     square, multiplied by q_weight / k_weight [D] and its first ``rot`` values are rotated (cos_sin fp32 [positions, rot],
     cosines then sines; ``pairing``: value i with i + rot / 2, "halves", or 2i with 2i + 1, "neighbours").  ``q_temp`` =
@@ -893,8 +959,12 @@ def qk_norm_rope_cache(qkv, H: int, G: int, D: int, Dv: int, maps: int, q_weight
     if v_first is not None:
         lam = v_lam.float().reshape(())
         v = ((1.0 - lam) * v.float() + lam * v_first[:T].float().view(T, G, Dv))
-    q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * q_weight.float()
-    k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * k_weight.float()
+    if whole_norm:          # one root mean square over all query (key) values of a token
+        q = q * torch.rsqrt(q.pow(2).mean((-2, -1), keepdim=True) + eps) * q_weight.float().view(H * maps, D)
+        k = k * torch.rsqrt(k.pow(2).mean((-2, -1), keepdim=True) + eps) * k_weight.float().view(G * maps, D)
+    else:
+        q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * q_weight.float()
+        k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * k_weight.float()
     if rot > 0:
         cs = cos_sin[positions[:T].long()]
         cos, sin = cs[:, None, : rot // 2], cs[:, None, rot // 2: rot]
@@ -974,7 +1044,8 @@ def masked_softmax_attention(qn, k_cache, v_cache, block_table, seq_lens, qsl, s
         out[t0:t1] = o.reshape(L, H, Dv)
     out = out.view(T, H * Dv)
     if gate is not None:
-        out = out * torch.sigmoid(gate[:T].float())
+        g = torch.sigmoid(gate[:T].float())
+        out = out * (g.repeat_interleave(Dv, 1) if g.shape[1] != H * Dv else g)
     return out.to(out_dtype)
 
 
