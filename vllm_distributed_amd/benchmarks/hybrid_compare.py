@@ -1,10 +1,11 @@
-"""Prefill and decode throughput of a Nositar, Rapovik, Sevazen or Lefolorn stack beside the closest existing models of
+"""Prefill and decode throughput of a Nositar, Rapovik, Sevazen, Lefolorn or Surodra stack beside the closest existing models of
 equal size, random weights.
 
     python bench.py --compare-nositar [--sizes small,medium] [--batch 32] [--input-len 2048] [--output-len 64]
     python bench.py --compare-rapovik [...]        (rapovik beside jamba-moe)
     python bench.py --compare-sevazen [...]        (sevazen beside mixtral-swa)
     python bench.py --compare-lefolorn [...]       (lefolorn beside sevazen and mixtral-swa)
+    python bench.py --compare-surodra [...]        (surodra beside nositar and jamba)
 
 Per size three engines run one after the other, each in a process of its own (``--one`` is the child's entry):
   nositar      alternating sigmoid head-mixing attention (window + kept first tokens) and gated delta-rule layers,
@@ -22,6 +23,8 @@ Per size three engines run one after the other, each in a process of its own (``
                in turn; both sub-layers of a layer read one group norm of the fp32 residual and join it behind layer
                scales and per-channel sigmoid gates; every layer has 8 routed gated experts and 2 identity outputs (two
                choices per token, from the better of two groups) plus a shared expert
+  surodra      delta-rule, attention-beside-gated-linear-attention and retention mixers in turn under squashing norms over an
+               fp32 residual; GELU-gated feed-forwards; the whole list is the looped part, run once
   mixtral-swa  a Mixtral stack of the same width, depth and heads with the same sliding window and 8 routed gated
                experts (two per token) of equal weight count
 Prefill: ``batch`` prompts of ``input-len`` tokens, one generated token.  Decode: the same requests generating
@@ -155,7 +158,27 @@ def lefolorn_config(s: dict) -> dict:
             "layers": [dict((lat, bias, cap)[i % 3], mlp=moe) for i in range(s["layers"])]}
 
 
-MODELS = {"lefolorn": lefolorn_config, "sevazen": sevazen_config, "mixtral-swa": mixtral_swa_config, "nositar": nositar_config, "llama-swa": llama_config, "jamba": jamba_config, "jamba-moe": jamba_moe_config,
+def surodra_config(s: dict) -> dict:
+    """Gated delta rule (heads of 128 x 128, as many values as the width), attention (heads of the other stacks, a quarter of
+    each rotated, NO window) beside gated linear attention (keys of half the width in heads of 64, values of the width in
+    heads of 128), and retention (heads of 128 x 128) in turn."""
+    w, d = s["width"], s["dim"]
+    hh = max(w // 128, 1)
+    mlp = {"kind": "dense", "ff": s["ff"]}
+    delta = {"type": "delta", "mlp": mlp, "mixer": {"heads": hh, "kv_heads": hh, "dim": 128, "vdim": 128, "conv": 4}}
+    par = {"type": "parallel", "mlp": mlp,
+           "mixer": {"left": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5,
+                              "rot": {"base": 500000.0, "dims": d // 4, "scaling": {"factor": 8.0}}},
+                     "right": {"heads": hh, "dim": 64, "vdim": 128, "tau": 16.0, "decay_rank": 16}}}
+    ret = {"type": "retention", "mlp": mlp,
+           "mixer": {"heads": hh, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-5 - 5 * i / hh) for i in range(hh)],
+                     "rot": {"base": 10000.0, "dims": 128}}}
+    return {"architecture": "Surodra", "vocab": s["vocab"], "width": w, "norm": {"eps": 1e-6}, "residual_mult": 0.3,
+            "logit_scale": 0.5, "logit_softcap": 15.0, "loop": {"start": 0, "stop": s["layers"], "times": 1},
+            "layers": [(delta, par, ret)[i % 3] for i in range(s["layers"])]}
+
+
+MODELS = {"surodra": surodra_config, "lefolorn": lefolorn_config, "sevazen": sevazen_config, "mixtral-swa": mixtral_swa_config, "nositar": nositar_config, "llama-swa": llama_config, "jamba": jamba_config, "jamba-moe": jamba_moe_config,
           "rapovik": rapovik_config}
 
 

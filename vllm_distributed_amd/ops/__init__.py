@@ -1623,7 +1623,7 @@ def linear_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: to
         fused = bool(N.lib().vda_linear_attention_fused(D, Dv))
         if not fused:
             o_raw = torch.empty((T, H * Dv), dtype=torch.float32, device=q.device)
-        if T // 128 * H >= 1024:          # enough workgroups: longer chunks move less state
+        if T // 128 * H >= 1:          # enough workgroups: longer chunks move less state
             C = 128
         scratch = torch.empty(N.lib().vda_linear_attention_scratch(T, S - first_long_seq, C, H, D, Dv),
                               dtype=torch.float32, device=q.device)

@@ -24,8 +24,8 @@
 //                U = T (V - diag(e^b) K S),   O = diag(e^b) Q S + P U,   P_ij = e^(b_i - b_j) q_i.k_j (j <= i)
 //                S <- e^b_n S + K^T diag(e^(b_n - b)) U
 //            T, P and the unit vectors of every block are made in parallel (delta_block_prepare); the walk over the blocks
-//            keeps S in the accumulators of one wave per (sequence, head, 16 columns) and passes every product on in
-//            registers (recurrent.h); norm and gate follow in a launch of their own.
+//            keeps S of sixteen columns in a wave's accumulators and passes every product on in registers
+//            (recurrent.h); norm and gate follow in a launch of their own.
 // The batch description is the one of the other recurrent kernels (qsl, seq_lens, slot in column 0 of the table;
 // a sequence carries state in when seq_len - new_tokens > 0), so prompts, portions of prompts, single decoded
 // tokens and mixtures of them are one code path, and the state after a token does not depend on how the
@@ -314,10 +314,10 @@ struct DeltaHeadArgs {
   const int *qsl, *seq_lens, *slot_table;
   long st_stride;
   int H, G, D, Dv, seq0, limit;
-  float* qhat;                  // [blocks, G, 16, DP]
-  float* khat;                  // [blocks, G, 16, DP]
-  float* khatT;                 // [blocks, G, DP, 16]
-  float* mats;                  // [blocks, H, DELTA_MAT]: T (16 x 16), P (16 x 16), e^b (16), e^(b_n - b) (16)
+  // what the walk reads, every matrix in the order its operand registers are filled ([lane][4], see recurrent.h):
+  float* vecs;                  // [blocks, G, 3, DT, 256]: unit keys, unit queries (token = lane % 16), keys with rows and
+                                //   columns exchanged (channel = lane % 16)
+  float* mats;                  // [blocks, H, DELTA_MAT]: T, P (256 each), e^b (16), e^(b_n - b) (16)
 };
 #define DELTA_MAT 544
 
@@ -449,9 +449,7 @@ __global__ __launch_bounds__(256) void delta_block_prepare_kernel(const DeltaHea
   const int lane = tid & 63, wave = tid >> 6, lo = lane & 15, g = lane >> 4;
   const long blk = (long)(t0 / 16) + srel + blockIdx.x;
   const float q_scale = 1.f / sqrtf((float)D);
-  float* qh = a.qhat + (blk * G + c) * 16 * DP;
-  float* kh = a.khat + (blk * G + c) * 16 * DP;
-  float* kt = a.khatT + (blk * G + c) * 16 * DP;
+  float* vec = a.vecs + (blk * G + c) * 3 * 16 * DP;
   for (int tt = wave; tt < 16; tt += 4) {
     const T* qr = (const T*)a.qkv + (long)(t0 + tb + tt) * a.qkv_stride + (long)c * D;
     const T* kr = qr + (long)G * D;
@@ -470,15 +468,15 @@ __global__ __launch_bounds__(256) void delta_block_prepare_kernel(const DeltaHea
       const float x = ok ? (float)qr[d] * rq : 0.f, y = ok ? (float)kr[d] * rk : 0.f;
       qs[tt * QP + d] = x;
       ks[tt * QP + d] = y;
-      qh[tt * DP + d] = x;
-      kh[tt * DP + d] = y;
     }
   }
   __syncthreads();
-  for (int e = tid; e < DP * 4; e += 256) {            // transposed keys, four tokens per store
-    const int d = e >> 2, j = (e & 3) * 4;
-    *reinterpret_cast<f32x4*>(kt + d * 16 + j) =
-        f32x4{ks[j * QP + d], ks[(j + 1) * QP + d], ks[(j + 2) * QP + d], ks[(j + 3) * QP + d]};
+  for (int e = tid; e < DT * 64; e += 256) {
+    const int dt = e >> 6, tok = e & 15, g4 = (e >> 4 & 3) * 4;
+    *reinterpret_cast<f32x4*>(vec + e * 4) = *reinterpret_cast<const f32x4*>(ks + tok * QP + dt * 16 + g4);
+    *reinterpret_cast<f32x4*>(vec + 16 * DP + e * 4) = *reinterpret_cast<const f32x4*>(qs + tok * QP + dt * 16 + g4);
+    const float* kc = ks + g4 * QP + dt * 16 + tok;
+    *reinterpret_cast<f32x4*>(vec + 32 * DP + e * 4) = f32x4{kc[0], kc[QP], kc[2 * QP], kc[3 * QP]};
   }
   // k_i . k_j and q_i . k_j: accumulator register r = [i = 4 g + r][j = lo]
   f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
@@ -511,7 +509,7 @@ __global__ __launch_bounds__(256) void delta_block_prepare_kernel(const DeltaHea
       const float bi = __shfl(b, i, 64), betai = __shfl(beta, i, 64);
       const float f = lo <= i ? expf(bi - b) : 0.f;
       Mw[i * 17 + lo] = lo < i ? betai * f * kk[r] : 0.f;
-      if (live) m[256 + i * 16 + lo] = f * qk[r];
+      if (live) m[256 + ((lo >> 2) * 16 + i) * 4 + (lo & 3)] = f * qk[r];
     }
     __syncthreads();
     // (I + M)^-1, one column per lane by forward substitution, times beta of the column
@@ -525,7 +523,7 @@ __global__ __launch_bounds__(256) void delta_block_prepare_kernel(const DeltaHea
     }
     if (live && g == 0) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) m[i * 16 + lo] = x[i] * beta;
+      for (int i = 0; i < 16; ++i) m[((lo >> 2) * 16 + i) * 4 + (lo & 3)] = x[i] * beta;
       m[512 + lo] = expf(b);
       m[528 + lo] = expf(bn - b);
     }
@@ -533,18 +531,24 @@ __global__ __launch_bounds__(256) void delta_block_prepare_kernel(const DeltaHea
   }
 }
 
-// grid (column tiles, H, sequences), one wave each: walks the blocks of its sequence with S in accumulators
+// grid (H, sequences, groups of 64 columns): walks the blocks of its sequence, S of sixteen columns per wave in
+// accumulators.  A block's operands (read by all four waves) sit in one of two LDS buffers while those of the next two
+// blocks are on their way from memory; one barrier per block.  The column group is the slowest grid index, so that workgroups that
+// read the same blocks tend to share an L2.
 template <typename T, int DT>
-__global__ __launch_bounds__(64) void delta_block_walk_kernel(const DeltaHeadArgs a) {
-  constexpr int DP = DT * 16;
-  const int srel = blockIdx.z, s = a.seq0 + srel, lane = threadIdx.x, lo = lane & 15, g = lane >> 4;
+__global__ __launch_bounds__(256) void delta_block_walk_kernel(const DeltaHeadArgs a) {
+  constexpr int DP = DT * 16, NV = 48 * DP, BUF = NV + DELTA_MAT;
+  constexpr int PF = (NV / 4 + 255) / 256;             // float4 of the vectors per thread and block
+  extern __shared__ __align__(16) float lds[];
+  const int srel = blockIdx.y, s = a.seq0 + srel, tid = threadIdx.x;
+  const int lane = tid & 63, wave = tid >> 6, lo = lane & 15, g = lane >> 4;
   const int sl = a.seq_lens[s];
   if (sl <= 0) return;
   const int t0 = a.qsl[s], L = a.qsl[s + 1] - t0;
   if (L <= a.limit) return;
-  const int h = blockIdx.y, D = a.D, Dv = a.Dv, H = a.H, G = a.G, c = h / (H / G);
-  const int col = blockIdx.x * 16 + lo;
-  const bool has_col = col < Dv;
+  const int h = blockIdx.x, D = a.D, Dv = a.Dv, H = a.H, G = a.G, c = h / (H / G);
+  const int tile0 = blockIdx.z * 64 + wave * 16, col = tile0 + lo;
+  const bool busy = tile0 < Dv, has_col = col < Dv;
   const bool vs4 = (D & 3) == 0;
   float* Scol = a.state + (((long)a.slot_table[s * a.st_stride] * H + h) * Dv + (has_col ? col : Dv - 1)) * (long)D;
   f32x4 S[DT];
@@ -555,73 +559,97 @@ __global__ __launch_bounds__(64) void delta_block_walk_kernel(const DeltaHeadArg
   const long blk0 = (long)(t0 / 16) + srel;
   const T* vp = (const T*)a.qkv + (long)t0 * a.qkv_stride + (long)2 * G * D + (long)h * Dv + (has_col ? col : Dv - 1);
 
-  struct Block {
-    f32x4 k[DT], q[DT], kt[DT], tm, pm, eb, ek, v;
-    float en;
+  const float* vec0 = a.vecs + (blk0 * G + c) * NV + tid * 4;
+  const float* mat0 = a.mats + (blk0 * H + h) * DELTA_MAT + tid * 4;
+  struct Fetched {
+    f32x4 vec[PF], mat;
+    T v[4];
   };
-  auto fetch = [&](Block& f, int bi) {
-    const float* kh = a.khat + ((blk0 + bi) * G + c) * 16 * DP + lo * DP + 4 * g;
-    const float* qh = a.qhat + ((blk0 + bi) * G + c) * 16 * DP + lo * DP + 4 * g;
-    const float* kt = a.khatT + ((blk0 + bi) * G + c) * 16 * DP + lo * 16 + 4 * g;
-    const float* m = a.mats + ((blk0 + bi) * H + h) * DELTA_MAT;
+  auto fetch = [&](Fetched& f, int bi) {               // nothing here waits for the data
+    const float* vp4 = vec0 + (long)bi * G * NV;
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      f.k[dt] = *reinterpret_cast<const f32x4*>(kh + dt * 16);
-      f.q[dt] = *reinterpret_cast<const f32x4*>(qh + dt * 16);
-      f.kt[dt] = *reinterpret_cast<const f32x4*>(kt + dt * 256);
-    }
-    f.tm = *reinterpret_cast<const f32x4*>(m + lo * 16 + 4 * g);
-    f.pm = *reinterpret_cast<const f32x4*>(m + 256 + lo * 16 + 4 * g);
-    f.eb = *reinterpret_cast<const f32x4*>(m + 512 + 4 * g);
-    f.ek = *reinterpret_cast<const f32x4*>(m + 528 + 4 * g);
-    f.en = m[512 + 15];
+    for (int n = 0; n < PF; ++n)
+      if ((n + 1) * 1024 <= NV || tid * 4 + n * 1024 < NV) f.vec[n] = *reinterpret_cast<const f32x4*>(vp4 + n * 1024);
+    if (tid < DELTA_MAT / 4) f.mat = *reinterpret_cast<const f32x4*>(mat0 + (long)bi * H * DELTA_MAT);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int tt = bi * 16 + 4 * g + r;
-      f.v[r] = tt < L ? (float)vp[(long)tt * a.qkv_stride] : 0.f;
-    }
+    for (int r = 0; r < 4; ++r) f.v[r] = vp[(long)min(bi * 16 + 4 * g + r, L - 1) * a.qkv_stride];
   };
-  auto run = [&](const Block& f, int bi) {
-    f32x4 ka = {0.f, 0.f, 0.f, 0.f}, kb = ka, qa = ka, qb = ka;
+  f32x4 v;
+  auto stage = [&](const Fetched& f, int bi) {         // block bi into its buffer, its values into v
+    float* buf = lds + (bi & 1) * BUF;
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      if (dt & 1) {
-        kb = mfma_f32_k16(f.k[dt], S[dt], kb);
-        qb = mfma_f32_k16(f.q[dt], S[dt], qb);
-      } else {
-        ka = mfma_f32_k16(f.k[dt], S[dt], ka);
-        qa = mfma_f32_k16(f.q[dt], S[dt], qa);
+    for (int n = 0; n < PF; ++n)
+      if ((n + 1) * 1024 <= NV || tid * 4 + n * 1024 < NV) *reinterpret_cast<f32x4*>(buf + tid * 4 + n * 1024) = f.vec[n];
+    if (tid < DELTA_MAT / 4) *reinterpret_cast<f32x4*>(buf + NV + tid * 4) = f.mat;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = bi * 16 + 4 * g + r < L ? (float)f.v[r] : 0.f;
+  };
+  auto run = [&](int bi) {
+    const float* buf = lds + (bi & 1) * BUF;
+    if (busy) {
+      f32x4 ka = {0.f, 0.f, 0.f, 0.f}, kb = ka, qa = ka, qb = ka;
+      // four accumulators in turn: a product never waits for the one right before it
+#pragma unroll
+      for (int dt = 0; dt < DT; dt += 2) {
+        const f32x4 k0 = *reinterpret_cast<const f32x4*>(buf + (dt * 64 + lane) * 4);
+        const f32x4 k1 = *reinterpret_cast<const f32x4*>(buf + (dt * 64 + 64 + lane) * 4);
+        const f32x4 q0 = *reinterpret_cast<const f32x4*>(buf + 16 * DP + (dt * 64 + lane) * 4);
+        const f32x4 q1 = *reinterpret_cast<const f32x4*>(buf + 16 * DP + (dt * 64 + 64 + lane) * 4);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          ka = mfma_f32(k0[r], S[dt][r], ka);
+          kb = mfma_f32(k1[r], S[dt + 1][r], kb);
+          qa = mfma_f32(q0[r], S[dt][r], qa);
+          qb = mfma_f32(q1[r], S[dt + 1][r], qb);
+        }
+      }
+      const f32x4 tm = *reinterpret_cast<const f32x4*>(buf + NV + lane * 4);
+      const f32x4 pm = *reinterpret_cast<const f32x4*>(buf + NV + 256 + lane * 4);
+      const f32x4 eb = *reinterpret_cast<const f32x4*>(buf + NV + 512 + 4 * g);
+      const f32x4 ek = *reinterpret_cast<const f32x4*>(buf + NV + 528 + 4 * g);
+      const float en = buf[NV + 512 + 15];
+      const f32x4 rhs = v - eb * (ka + kb);
+      f32x4 u = {0.f, 0.f, 0.f, 0.f};
+      u = mfma_f32_k16(tm, rhs, u);
+      const f32x4 o = mfma_f32_k16(pm, u, eb * (qa + qb));
+      u *= ek;
+#pragma unroll
+      for (int dt = 0; dt < DT; dt += 2) {
+        const f32x4 kt0 = *reinterpret_cast<const f32x4*>(buf + 32 * DP + (dt * 64 + lane) * 4);
+        const f32x4 kt1 = *reinterpret_cast<const f32x4*>(buf + 32 * DP + (dt * 64 + 64 + lane) * 4);
+        S[dt] *= en;
+        S[dt + 1] *= en;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          S[dt] = mfma_f32(kt0[r], u[r], S[dt]);
+          S[dt + 1] = mfma_f32(kt1[r], u[r], S[dt + 1]);
+        }
+      }
+      if (has_col) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int tt = bi * 16 + 4 * g + r;
+          if (tt < L) a.o_raw[((long)(t0 + tt) * H + h) * Dv + col] = o[r];
+        }
       }
     }
-    const f32x4 rhs = f.v - f.eb * (ka + kb);
-    f32x4 u = {0.f, 0.f, 0.f, 0.f};
-    u = mfma_f32_k16(f.tm, rhs, u);
-    const f32x4 o = mfma_f32_k16(f.pm, u, f.eb * (qa + qb));
-    u *= f.ek;
-#pragma unroll
-    for (int dt = 0; dt < DT; ++dt) S[dt] = mfma_f32_k16(f.kt[dt], u, S[dt] * f.en);
-    if (has_col) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int tt = bi * 16 + 4 * g + r;
-        if (tt < L) a.o_raw[((long)(t0 + tt) * H + h) * Dv + col] = o[r];
-      }
-    }
   };
-  if constexpr (DT <= 8) {               // the next block is on its way while this one is computed
-    Block f0, f1;
-    fetch(f0, 0);
-    for (int bi = 0; bi < nb; bi += 2) {
-      if (bi + 1 < nb) fetch(f1, bi + 1);
-      run(f0, bi);
-      if (bi + 2 < nb) fetch(f0, bi + 2);
-      if (bi + 1 < nb) run(f1, bi + 1);
-    }
-  } else {                               // wide keys: the registers hold one block
-    Block f0;
-    for (int bi = 0; bi < nb; ++bi) {
-      fetch(f0, bi);
-      run(f0, bi);
+  // two blocks ahead in registers, one ahead in LDS
+  Fetched fa, fb;
+  fetch(fa, 0);
+  if (nb > 1) fetch(fb, 1);
+  stage(fa, 0);
+  __syncthreads();
+  for (int bi = 0; bi < nb; bi += 2) {
+    if (bi + 2 < nb) fetch(fa, bi + 2);
+    run(bi);
+    if (bi + 1 < nb) stage(fb, bi + 1);
+    __syncthreads();
+    if (bi + 1 < nb) {
+      if (bi + 3 < nb) fetch(fb, bi + 3);
+      run(bi + 1);
+      if (bi + 2 < nb) stage(fa, bi + 2);
+      __syncthreads();
     }
   }
   if (has_col) {
@@ -656,10 +684,8 @@ VDA_EXPORT int vda_gated_delta_rule_head(void* out, long o_stride, float* o_raw,
   a.limit = chunked ? 16 : 0x7fffffff;
   const int DT = delta_dt(D);
   const long blocks = (long)T / 16 + (S - seq0) + 1;
-  a.qhat = scratch;
-  a.khat = scratch ? a.qhat + blocks * G * 16 * (DT * 16) : nullptr;
-  a.khatT = scratch ? a.khat + blocks * G * 16 * (DT * 16) : nullptr;
-  a.mats = scratch ? a.khatT + blocks * G * 16 * (DT * 16) : nullptr;
+  a.vecs = scratch;
+  a.mats = scratch ? scratch + blocks * G * 48 * (DT * 16) : nullptr;
   int NR = 1;
   while (16 * NR < D) NR *= 2;
   int tile = max_q < 16 ? max_q : 16;
@@ -686,11 +712,17 @@ VDA_EXPORT int vda_gated_delta_rule_head(void* out, long o_stride, float* o_raw,
 #undef STEP
   VDA_CHECK_LAUNCH();
   if (!chunked) return 0;
-  const dim3 gp((max_q + 15) / 16, S - seq0, G), gw((Dv + 15) / 16, H, S - seq0);
+  const dim3 gp((max_q + 15) / 16, S - seq0, G), gw(H, S - seq0, (Dv + 63) / 64);
+  const size_t wlds = (size_t)2 * (48 * DT * 16 + DELTA_MAT) * 4;
 #define CK(TT, DD)                                                                                                     \
   do {                                                                                                                 \
+    if (wlds > 48 * 1024) {                                                                                            \
+      hipError_t e_ = hipFuncSetAttribute((const void*)delta_block_walk_kernel<TT, DD>,                                \
+                                          hipFuncAttributeMaxDynamicSharedMemorySize, (int)wlds);                      \
+      if (e_ != hipSuccess) return (int)e_;                                                                            \
+    }                                                                                                                  \
     hipLaunchKernelGGL((delta_block_prepare_kernel<TT, DD>), gp, dim3(256), 0, st, a);                                 \
-    hipLaunchKernelGGL((delta_block_walk_kernel<TT, DD>), gw, dim3(64), 0, st, a);                                     \
+    hipLaunchKernelGGL((delta_block_walk_kernel<TT, DD>), gw, dim3(256), wlds, st, a);                                 \
   } while (0)
 #define CA(TT) do { if (DT == 2) CK(TT, 2); else if (DT == 4) CK(TT, 4); else if (DT == 8) CK(TT, 8); else CK(TT, 16); } while (0)
   if (dtype == VDA_BF16) CA(bf16_t);

@@ -11,7 +11,7 @@
 // Sequences with few new tokens (decoding, short portions):
 //   step   one workgroup per (sequence, head), token by token, everything in one launch: the state is read and written
 //          once, norm and gate included.
-// Longer ones, chunk-parallel (fp32 matrix instructions, see recurrent.h): a sequence is cut into chunks of C tokens,
+// Longer ones (when the rows allow 4-value accesses; otherwise `step` walks them too), chunk-parallel (fp32 matrix instructions, see recurrent.h): a sequence is cut into chunks of C tokens,
 //   chunk<OUT = false>   per (chunk, head): the state the chunk alone would build, and its total decay
 //   carry                per (sequence, head): the state at every chunk's start, one after the other (elementwise)
 //   chunk<OUT = true>    per (chunk, head): from that state, sixteen tokens at a time:
@@ -47,8 +47,7 @@ struct LinArgs {
   float* chunk_decay;           // [chunks, H, DP] (channel decays)
   int limit;                    // sequences with at most this many new tokens belong to `step`, others to `chunk`
   int col_groups;
-  int vec;                      // D % 4 == 0 and all rows aligned for 4-value loads
-  int vec_v;                    // likewise for Dv
+  int vec;                      // D % 4 == 0 and all q / k / z rows aligned for 4-value loads
 };
 
 // values d .. d + 3 of a q or k row of head h at token t: rotated, unscaled, zeros from D on
@@ -195,18 +194,24 @@ __global__ __launch_bounds__(256) void lin_step_kernel(const LinArgs a, const in
 
 // ---- chunk-parallel form -------------------------------------------------------------------------------------------
 // grid (chunks of the longest sequence, sequences, heads x column groups); wave w holds columns
-// (w * ET .. w * ET + ET - 1) * 16 of the group, all D rows of them in accumulators
+// (w * ET .. w * ET + ET - 1) * 16 of the group, all D rows of them in accumulators.  Rows are aligned for 4-value
+// accesses and D, Dv and rot / 2 are multiples of 4.
+// Staging layout: thread -> token tid / 16, values d0 + 64 m with d0 = 4 * (tid % 16).  The next sixteen tokens' rows are
+// on their way from memory, unconverted, while these are computed; a block's output leaves LDS in the staging phase of
+// the next one, so two barriers (four with channel decays) separate everything.
 template <typename T, int DT, int ET, bool CHAN, bool OUT>
-__global__ __launch_bounds__(256) void lin_chunk_kernel(const LinArgs a) {
-  constexpr int DP = DT * 16, QP = DP + 4, TP = 20, CW = 64 * ET;
+__global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_kernel(const LinArgs a) {
+  constexpr int DP = DT * 16, QP = DP + 4, TP = 20, CW = 64 * ET, OP = CW + 4;
+  constexpr int NI = (DP + 63) / 64, NVI = ET;
+  using V4 = typename Vec<T>::v4;
   extern __shared__ __align__(16) float lds[];
   float* ks = lds;                                     // [16][QP]
   float* kT = ks + 16 * QP;                            // [DP][TP]   k_j e^(b_n - b_j), transposed
   float* vT = kT + DP * TP;                            // [CW][TP]
   float* qs = vT + CW * TP;                            // [16][QP]   (OUT)
-  float* bc = qs + (OUT ? 16 * QP : 0);                // [16][QP]   (CHAN) running sums of log decays
+  float* os = qs + (OUT ? 16 * QP : 0);                // [16][OP]   (OUT)
+  float* bc = os + (OUT ? 16 * OP : 0);                // [16][QP]   (CHAN) running sums of log decays
   float* dec = bc + (CHAN ? 16 * QP : 0);              // [DP]       (CHAN) e^b_n
-  float* red = dec + (CHAN ? DP : 0);                  // [4][16]    (OUT)
   const int srel = blockIdx.y, s = a.seq0 + srel, tid = threadIdx.x;
   const int sl = a.seq_lens[s];
   if (sl <= 0) return;
@@ -224,71 +229,171 @@ __global__ __launch_bounds__(256) void lin_chunk_kernel(const LinArgs a) {
   const long cidx = ((long)(t0 / C) + srel + c) * H + h;
   float* cst = a.chunk_state + cidx * coltiles * (DT * 256);
   float* Sb = a.state + ((long)a.slot_table[s * a.st_stride] * H + h) * (long)Dv * D;
-  const bool vs4 = (D & 3) == 0;
   f32x4 S[ET][DT];
+  const bool from_chunk = OUT && nch > 1, from_slot = OUT && nch == 1 && sl - L > 0;
 #pragma unroll
-  for (int e = 0; e < ET; ++e)
+  for (int e = 0; e < ET; ++e) {
+    const int ct = tile0 + e, col = ct * 16 + lo;
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) S[e][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  if (OUT) {
-#pragma unroll
-    for (int e = 0; e < ET; ++e) {
-      const int ct = tile0 + e, col = ct * 16 + lo;
-      if (ct >= coltiles) continue;
-#pragma unroll
-      for (int dt = 0; dt < DT; ++dt) {
-        if (nch > 1) S[e][dt] = *reinterpret_cast<const f32x4*>(cst + ((long)(ct * DT + dt) * 64 + lane) * 4);
-        else if (sl - L > 0 && col < Dv) S[e][dt] = load4<float>(Sb + (long)col * D + dt * 16 + 4 * g, D - dt * 16 - 4 * g, vs4);
-      }
+    for (int dt = 0; dt < DT; ++dt) {
+      const int d = dt * 16 + 4 * g;
+      S[e][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (from_chunk && ct < coltiles) S[e][dt] = *reinterpret_cast<const f32x4*>(cst + ((ct * DT + dt) * 64 + lane) * 4);
+      if (from_slot && col < Dv && d < D) S[e][dt] = *reinterpret_cast<const f32x4*>(Sb + (long)col * D + d);
     }
   }
   const float ld = CHAN ? 0.f : a.log_decay[h];
   float tot = 0.f;                                     // CHAN, thread d: sum of channel d's log decays over the chunk
-  const int end = min(L, c * C + C);
-  for (int tb = c * C; tb < end; tb += 16) {
+  float pf[4], of[4];                                  // e^(b_i - b_j) of this lane's pairs, e^b_i of its rows
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    pf[r] = 4 * g + r <= lo ? expf(ld * (float)(lo - 4 * g - r)) : 0.f;
+    of[r] = expf(ld * (float)(4 * g + r + 1));
+  }
+  const int tt = tid >> 4, d0 = (tid & 15) * 4, half = a.rot >> 1;
+  const T* kp = (const T*)a.k + (long)h * D + t0 * a.k_stride;
+  const T* qp = (const T*)a.q + (long)h * D + t0 * a.q_stride;
+  const T* vp = (const T*)a.v + (long)h * Dv + t0 * a.v_stride + col0;
+  const T* zp = CHAN ? (const T*)a.z + (long)h * D + t0 * a.z_stride : nullptr;
+  const T* gp = (const T*)a.gate + (long)h * Dv + t0 * a.g_stride;
+  V4 rk[NI], rk2[NI], rq[NI], rq2[NI], rz[NI], rv[NVI], rg[NVI];
+  int pos = 0;
+  auto fetch = [&](int tb) {
+    const long t = min(tb + tt, L - 1);
+    if (!CHAN && a.rot > 0) pos = (int)a.positions[t0 + t];
+#pragma unroll
+    for (int m = 0; m < NI; ++m) {
+      const int d = d0 + 64 * m, dc = d < D ? d : 0;
+      rk[m] = *reinterpret_cast<const V4*>(kp + t * a.k_stride + dc);
+      if (OUT) rq[m] = *reinterpret_cast<const V4*>(qp + t * a.q_stride + dc);
+      if (CHAN) rz[m] = *reinterpret_cast<const V4*>(zp + t * a.z_stride + dc);
+      if (!CHAN && a.rot > 0) {
+        const int dp = d < a.rot ? (d < half ? d + half : d - half) : dc;
+        rk2[m] = *reinterpret_cast<const V4*>(kp + t * a.k_stride + dp);
+        if (OUT) rq2[m] = *reinterpret_cast<const V4*>(qp + t * a.q_stride + dp);
+      }
+    }
+#pragma unroll
+    for (int m = 0; m < NVI; ++m) {
+      const int cc = d0 + 64 * m;
+      rv[m] = *reinterpret_cast<const V4*>(vp + t * a.v_stride + (col0 + cc < Dv ? cc : 0));
+    }
+  };
+  // rows tb .. tb + 15 of the output: norm over the head's columns, weight, gate (or the plain sums)
+  auto emit = [&](int tb) {
+    if (tb + tt >= min(L, c * C + C)) return;
+    const long t = tb + tt;
+    f32x4 o[NVI];
+    float ss = 0.f;
+#pragma unroll
+    for (int m = 0; m < NVI; ++m) {
+      o[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (col0 + d0 + 64 * m < Dv) o[m] = *reinterpret_cast<const f32x4*>(os + tt * OP + d0 + 64 * m);
+      ss += o[m][0] * o[m][0] + o[m][1] * o[m][1] + o[m][2] * o[m][2] + o[m][3] * o[m][3];
+    }
+    if (a.o_raw) {
+#pragma unroll
+      for (int m = 0; m < NVI; ++m)
+        if (col0 + d0 + 64 * m < Dv)
+          *reinterpret_cast<f32x4*>(a.o_raw + ((t0 + t) * H + h) * Dv + col0 + d0 + 64 * m) = o[m];
+      return;
+    }
+    ss = row16_sum(ss);                                // a token's columns sit in sixteen neighbouring lanes
+    const float rs = 1.f / sqrtf(ss / (float)Dv + a.eps);
+#pragma unroll
+    for (int m = 0; m < NVI; ++m) {
+      const int cc = d0 + 64 * m;
+      if (cc >= Dv) continue;
+      f32x4 w = {1.f, 1.f, 1.f, 1.f};
+      if (a.norm_w) w = *reinterpret_cast<const f32x4*>(a.norm_w + cc);
+      V4 y;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float zg = (float)rg[m][i];
+        y[i] = (T)(o[m][i] * rs * w[i] * zg * rec_sigmoid(zg));
+      }
+      *reinterpret_cast<V4*>((T*)a.out + (t0 + t) * a.o_stride + (long)h * Dv + cc) = y;
+    }
+  };
+  const int first = c * C, end = min(L, first + C);
+  fetch(first);
+  for (int tb = first; tb < end; tb += 16) {
     const int n = min(16, end - tb);
+    const bool on = tt < n;
+    f32x4 rc[NI], rs[NI];
+    if (!CHAN && a.rot > 0) {
+      const float* cs = a.cos_sin + pos * (long)a.rot;
+#pragma unroll
+      for (int m = 0; m < NI; ++m) {
+        const int d = d0 + 64 * m, ci = d < a.rot ? (d < half ? d : d - half) : 0;
+        rc[m] = *reinterpret_cast<const f32x4*>(cs + ci);
+        rs[m] = *reinterpret_cast<const f32x4*>(cs + half + ci);
+      }
+    }
     __syncthreads();
-    for (int e = tid; e < 16 * (DP / 4); e += 256) {
-      const int tt = e / (DP / 4), d = (e - tt * (DP / 4)) * 4;
-      const long t = t0 + tb + tt;
-      f32x4 k = {0.f, 0.f, 0.f, 0.f}, q = k, b = k;
-      if (tt < n) {
-        k = lin_row4<T>(a, (const T*)a.k + t * a.k_stride + (long)h * D, d, t) * a.k_scale;
-        if (OUT) q = lin_row4<T>(a, (const T*)a.q + t * a.q_stride + (long)h * D, d, t) * a.q_scale;
-        if (CHAN) b = lin_log_decay4<T>(a, t, h, d);
+    if (OUT && tb > first) emit(tb - 16);
+    const float f = CHAN ? 0.f : expf(ld * (float)max(n - 1 - tt, 0));
+#pragma unroll
+    for (int m = 0; m < NI; ++m) {
+      const int d = d0 + 64 * m;
+      if (DP < 64 && d >= DP) continue;
+      f32x4 k, q = {0.f, 0.f, 0.f, 0.f}, b = q;
+      const bool live = on && d < D, turn = !CHAN && d < a.rot;
+      const float sg = d < half ? -1.f : 1.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        float y = (float)rk[m][i];
+        if (turn) y = y * rc[m][i] + sg * (float)rk2[m][i] * rs[m][i];
+        k[i] = live ? y * a.k_scale : 0.f;
+        if (OUT) {
+          float x = (float)rq[m][i];
+          if (turn) x = x * rc[m][i] + sg * (float)rq2[m][i] * rs[m][i];
+          q[i] = live ? x * a.q_scale : 0.f;
+        }
       }
       *reinterpret_cast<f32x4*>(ks + tt * QP + d) = k;
       if (OUT) *reinterpret_cast<f32x4*>(qs + tt * QP + d) = q;
       if (CHAN) {
+        if (live) {
+          f32x4 zb = {0.f, 0.f, 0.f, 0.f};
+          if (a.z_bias) zb = *reinterpret_cast<const f32x4*>(a.z_bias + (long)h * D + d);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) b[i] = rec_logsigmoid((float)rz[m][i] + zb[i]) * a.inv_tau;
+        }
         *reinterpret_cast<f32x4*>(bc + tt * QP + d) = b;
       } else {
-        const float f = expf(ld * (float)(n - 1 - tt));          // tokens beyond n have k = 0
 #pragma unroll
-        for (int i = 0; i < 4; ++i) kT[(d + i) * TP + tt] = tt < n ? k[i] * f : 0.f;
+        for (int i = 0; i < 4; ++i) kT[(d + i) * TP + tt] = k[i] * f;
       }
     }
-    for (int e = tid; e < 16 * (CW / 4); e += 256) {
-      const int tt = e / (CW / 4), cc = (e - tt * (CW / 4)) * 4;
-      f32x4 v = {0.f, 0.f, 0.f, 0.f};
-      if (tt < n)
-        v = load4<T>((const T*)a.v + (long)(t0 + tb + tt) * a.v_stride + (long)h * Dv + col0 + cc, Dv - col0 - cc, a.vec_v);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) vT[(cc + i) * TP + tt] = v[i];
+    for (int m = 0; m < NVI; ++m) {
+      const int cc = d0 + 64 * m;
+      const bool live = on && col0 + cc < Dv;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) vT[(cc + i) * TP + tt] = live ? (float)rv[m][i] : 0.f;
     }
-    f32x4 pt = {0.f, 0.f, 0.f, 0.f}, pt2 = pt;         // P^T: [j = 4 g + r][i = lo]
-    if (CHAN) {
-      __syncthreads();
-      int strong = 0;
-      if (tid < DP) {
-        float run = 0.f;
+    if (OUT && !a.o_raw) {                             // this block's gates; used when its output leaves
+      const long t = min(tb + tt, L - 1);
 #pragma unroll
-        for (int tt = 0; tt < 16; ++tt) {
-          run += bc[tt * QP + tid];
-          bc[tt * QP + tid] = run;
-        }
-        dec[tid] = expf(run);
-        tot += run;
-        strong = run < -40.f;
+      for (int m = 0; m < NVI; ++m) rg[m] = *reinterpret_cast<const V4*>(gp + t * a.g_stride + (d0 + 64 * m < Dv ? d0 + 64 * m : 0));
+    }
+    if (tb + 16 < end) fetch(tb + 16);
+    __syncthreads();
+    f32x4 pt = {0.f, 0.f, 0.f, 0.f}, pt2 = pt;         // P^T: [j = 4 g + r][i = lo]
+    int strong = 0;
+    if (CHAN) {
+      if (tid < DP) {
+        float run[16];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) run[j] = bc[j * QP + tid];
+#pragma unroll
+        for (int j = 1; j < 16; ++j) run[j] += run[j - 1];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) bc[j * QP + tid] = run[j];
+        dec[tid] = expf(run[15]);
+        tot += run[15];
+        strong = run[15] < -40.f;
       }
       strong = __syncthreads_or(strong);
       if (OUT && strong) {
@@ -305,8 +410,10 @@ __global__ __launch_bounds__(256) void lin_chunk_kernel(const LinArgs a) {
         }
         __syncthreads();
       }
-      for (int e = tid; e < 16 * (DP / 4); e += 256) {
-        const int tt = e / (DP / 4), d = (e - tt * (DP / 4)) * 4;
+#pragma unroll
+      for (int m = 0; m < NI; ++m) {
+        const int d = d0 + 64 * m;
+        if (DP < 64 && d >= DP) continue;
         const f32x4 b = *reinterpret_cast<const f32x4*>(bc + tt * QP + d), bn = *reinterpret_cast<const f32x4*>(bc + 15 * QP + d);
         f32x4 k = *reinterpret_cast<const f32x4*>(ks + tt * QP + d);
 #pragma unroll
@@ -323,129 +430,89 @@ __global__ __launch_bounds__(256) void lin_chunk_kernel(const LinArgs a) {
         }
       }
       __syncthreads();
-      if (OUT && busy) {
-        if (!strong) {
-#pragma unroll
-          for (int dt = 0; dt < DT; ++dt) {
-            const f32x4 ka = *reinterpret_cast<const f32x4*>(ks + lo * QP + dt * 16 + 4 * g);
-            const f32x4 qb = *reinterpret_cast<const f32x4*>(qs + lo * QP + dt * 16 + 4 * g);
-            if (dt & 1) pt2 = mfma_f32_k16(ka, qb, pt2); else pt = mfma_f32_k16(ka, qb, pt);
-          }
-          pt += pt2;
-        }
-#pragma unroll
-        for (int r = 0; r < 4; ++r) pt[r] = 4 * g + r <= lo ? pt[r] : 0.f;
-      }
-    } else {
-      __syncthreads();
-      if (OUT && busy) {
-#pragma unroll
-        for (int dt = 0; dt < DT; ++dt) {
-          const f32x4 ka = *reinterpret_cast<const f32x4*>(ks + lo * QP + dt * 16 + 4 * g);
-          const f32x4 qb = *reinterpret_cast<const f32x4*>(qs + lo * QP + dt * 16 + 4 * g);
-          if (dt & 1) pt2 = mfma_f32_k16(ka, qb, pt2); else pt = mfma_f32_k16(ka, qb, pt);
-        }
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int j = 4 * g + r;
-          pt[r] = j <= lo ? (pt[r] + pt2[r]) * expf(ld * (float)(lo - j)) : 0.f;
-        }
-      }
     }
+    if (!busy) continue;
     f32x4 v4[ET];
 #pragma unroll
     for (int e = 0; e < ET; ++e) v4[e] = *reinterpret_cast<const f32x4*>(vT + ((wave * ET + e) * 16 + lo) * TP + 4 * g);
     if (OUT) {
-      f32x4 O[ET];
-      if (busy) {
+      if (!CHAN || !strong) {
 #pragma unroll
-        for (int e = 0; e < ET; ++e) {
-          f32x4 o2 = {0.f, 0.f, 0.f, 0.f};
-          O[e] = o2;
-#pragma unroll
-          for (int dt = 0; dt < DT; ++dt) {
-            const f32x4 qa = *reinterpret_cast<const f32x4*>(qs + lo * QP + dt * 16 + 4 * g);
-            if (dt & 1) o2 = mfma_f32_k16(qa, S[e][dt], o2); else O[e] = mfma_f32_k16(qa, S[e][dt], O[e]);
-          }
-          O[e] += o2;
-          if (!CHAN) {
-#pragma unroll
-            for (int r = 0; r < 4; ++r) O[e][r] *= expf(ld * (float)(4 * g + r + 1));
-          }
-          O[e] = mfma_f32_k16(pt, v4[e], O[e]);
+        for (int dt = 0; dt < DT; dt += 2) {
+          const float* kr = ks + lo * QP + dt * 16 + 4 * g;
+          const float* qr = qs + lo * QP + dt * 16 + 4 * g;
+          mfma_f32_k16_two(*(const f32x4*)kr, *(const f32x4*)qr, pt, *(const f32x4*)(kr + 16), *(const f32x4*)(qr + 16), pt2);
         }
-      } else {
+        pt += pt2;
 #pragma unroll
-        for (int e = 0; e < ET; ++e) O[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int r = 0; r < 4; ++r) pt[r] = CHAN ? (4 * g + r <= lo ? pt[r] : 0.f) : pt[r] * pf[r];
       }
-      if (a.o_raw) {
+      f32x4 O[ET], o2[ET];
 #pragma unroll
-        for (int e = 0; e < ET; ++e) {
-          const int col = (tile0 + e) * 16 + lo;
+      for (int e = 0; e < ET; ++e) O[e] = o2[e] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int r = 0; r < 4; ++r)
-            if (4 * g + r < n && col < Dv)
-              a.o_raw[((long)(t0 + tb + 4 * g + r) * H + h) * Dv + col] = O[e][r];
-        }
-      } else {
-        // columns beyond Dv hold zeros: they add nothing to the sums
+      for (int dt = 0; dt < DT; dt += 2) {
+        const f32x4 q0 = *reinterpret_cast<const f32x4*>(qs + lo * QP + dt * 16 + 4 * g);
+        const f32x4 q1 = *reinterpret_cast<const f32x4*>(qs + lo * QP + dt * 16 + 16 + 4 * g);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          float ss = 0.f;
-#pragma unroll
-          for (int e = 0; e < ET; ++e) ss += O[e][r] * O[e][r];
-          ss = row16_sum(ss);
-          if (lo == 0) red[wave * 16 + 4 * g + r] = ss;
-        }
-        __syncthreads();
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int i = 4 * g + r;
-          if (i >= n) continue;
-          const float ss = red[i] + red[16 + i] + red[32 + i] + red[48 + i];
-          const float rs = 1.f / sqrtf(ss / (float)Dv + a.eps);
-          const long t = t0 + tb + i;
+        for (int r = 0; r < 4; ++r)
 #pragma unroll
           for (int e = 0; e < ET; ++e) {
-            const int col = (tile0 + e) * 16 + lo;
-            if (col >= Dv) continue;
-            const float zg = (float)((const T*)a.gate)[t * a.g_stride + (long)h * Dv + col];
-            ((T*)a.out)[t * a.o_stride + (long)h * Dv + col] =
-                (T)(O[e][r] * rs * (a.norm_w ? a.norm_w[col] : 1.f) * zg * rec_sigmoid(zg));
+            O[e] = mfma_f32(q0[r], S[e][dt][r], O[e]);
+            o2[e] = mfma_f32(q1[r], S[e][dt + 1][r], o2[e]);
           }
+      }
+#pragma unroll
+      for (int e = 0; e < ET; ++e) {
+        O[e] += o2[e];
+        if (!CHAN) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) O[e][r] *= of[r];
         }
+        O[e] = mfma_f32_k16(pt, v4[e], O[e]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) os[(4 * g + r) * OP + (wave * ET + e) * 16 + lo] = O[e][r];
       }
     }
-    if (busy) {
-      const float dn = CHAN ? 0.f : expf(ld * (float)n);
+    const float dn = CHAN ? 0.f : expf(ld * (float)n);
 #pragma unroll
-      for (int dt = 0; dt < DT; ++dt) {
-        const f32x4 ka = *reinterpret_cast<const f32x4*>(kT + (dt * 16 + lo) * TP + 4 * g);
-        f32x4 d4;
-        if (CHAN) d4 = *reinterpret_cast<const f32x4*>(dec + dt * 16 + 4 * g);
-        else d4 = f32x4{dn, dn, dn, dn};
-#pragma unroll
-        for (int e = 0; e < ET; ++e) S[e][dt] = mfma_f32_k16(ka, v4[e], S[e][dt] * d4);
+    for (int dt = 0; dt < DT; dt += 2) {
+      const f32x4 k0 = *reinterpret_cast<const f32x4*>(kT + (dt * 16 + lo) * TP + 4 * g);
+      const f32x4 k1 = *reinterpret_cast<const f32x4*>(kT + (dt * 16 + 16 + lo) * TP + 4 * g);
+      f32x4 g0 = {dn, dn, dn, dn}, g1 = g0;
+      if (CHAN) {
+        g0 = *reinterpret_cast<const f32x4*>(dec + dt * 16 + 4 * g);
+        g1 = *reinterpret_cast<const f32x4*>(dec + dt * 16 + 16 + 4 * g);
       }
+#pragma unroll
+      for (int e = 0; e < ET; ++e) {
+        S[e][dt] *= g0;
+        S[e][dt + 1] *= g1;
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int e = 0; e < ET; ++e) {
+          S[e][dt] = mfma_f32(k0[r], v4[e][r], S[e][dt]);
+          S[e][dt + 1] = mfma_f32(k1[r], v4[e][r], S[e][dt + 1]);
+        }
     }
   }
-  if (!OUT) {
-    if (CHAN && cg == 0 && tid < DP) a.chunk_decay[cidx * DP + tid] = expf(tot);
+  if (OUT) {
+    __syncthreads();
+    emit((end - 1 - first) / 16 * 16 + first);
+    if (c != nch - 1) return;
+  } else if (CHAN && cg == 0 && tid < DP) {
+    a.chunk_decay[cidx * DP + tid] = expf(tot);
+  }
 #pragma unroll
-    for (int e = 0; e < ET; ++e) {
-      const int ct = tile0 + e;
-      if (ct >= coltiles) continue;
+  for (int e = 0; e < ET; ++e) {
+    const int ct = tile0 + e, col = ct * 16 + lo;
 #pragma unroll
-      for (int dt = 0; dt < DT; ++dt)
-        *reinterpret_cast<f32x4*>(cst + ((long)(ct * DT + dt) * 64 + lane) * 4) = S[e][dt];
-    }
-  } else if (c == nch - 1) {
-#pragma unroll
-    for (int e = 0; e < ET; ++e) {
-      const int col = (tile0 + e) * 16 + lo;
-      if (col >= Dv) continue;
-#pragma unroll
-      for (int dt = 0; dt < DT; ++dt) store4(Sb + (long)col * D + dt * 16 + 4 * g, S[e][dt], D - dt * 16 - 4 * g, vs4);
+    for (int dt = 0; dt < DT; ++dt) {
+      const int d = dt * 16 + 4 * g;
+      if (!OUT && ct < coltiles) *reinterpret_cast<f32x4*>(cst + ((ct * DT + dt) * 64 + lane) * 4) = S[e][dt];
+      if (OUT && col < Dv && d < D) *reinterpret_cast<f32x4*>(Sb + (long)col * D + d) = S[e][dt];
     }
   }
 }
@@ -517,8 +584,14 @@ VDA_EXPORT int vda_linear_attention(
   if (H <= 0 || D < 1 || Dv < 1 || D > 1024 || rot < 0 || rot > D || (rot & 1) || (rot > 0 && (!cos_sin || !positions)) ||
       (!z && !log_decay) || seq0 < 0 || seq0 > S)
     return -1;
-  // chunk-parallel for key widths of up to 256: sequences of more than 16 new tokens, from seq0 on
-  const bool chunked = D <= 256 && max_q > 16 && scratch && seq0 < S && C >= 16 && C % 16 == 0;
+  // chunk-parallel for key widths of up to 256: sequences of more than 16 new tokens, from seq0 on,
+  // and only for rows that can be read four values at a time
+  const int es = dtype == VDA_F32 ? 16 : 8;
+  auto ok4 = [&](const void* p, long stride) { return !p || (((uintptr_t)p % es) == 0 && stride % 4 == 0); };
+  const bool vec = D % 4 == 0 && ok4(q, q_stride) && ok4(k, k_stride) && ok4(z, z_stride);
+  const bool vec_v = Dv % 4 == 0 && ok4(v, v_stride) && ok4(gate, g_stride) && ok4(out, o_stride) && !((uintptr_t)norm_w % 16);
+  const bool chunked = D <= 256 && max_q > 16 && scratch && seq0 < S && C >= 16 && C % 16 == 0 && vec && vec_v &&
+                       rot % 8 == 0 && (!z || rot == 0) && !((uintptr_t)z_bias % 16) && !((uintptr_t)cos_sin % 16);
   const int DT = lin_dt(D);
   const int ET = (DT <= 8 && Dv > 64) ? 2 : 1;
   LinArgs a;
@@ -532,10 +605,7 @@ VDA_EXPORT int vda_linear_attention(
   a.col_groups = (Dv + 64 * ET - 1) / (64 * ET);
   a.o_raw = a.col_groups > 1 ? o_raw : nullptr;
   if (chunked && a.col_groups > 1 && !o_raw) return -1;
-  const int es = dtype == VDA_F32 ? 16 : 8;
-  auto ok4 = [&](const void* p, long stride) { return !p || (((uintptr_t)p % es) == 0 && stride % 4 == 0); };
-  a.vec = D % 4 == 0 && ok4(q, q_stride) && ok4(k, k_stride) && ok4(z, z_stride);
-  a.vec_v = Dv % 4 == 0 && ok4(v, v_stride);
+  a.vec = vec;
   const long chunks = chunked ? (long)T / C + (S - seq0) + 1 : 0;
   a.chunk_state = scratch;
   a.chunk_decay = scratch ? scratch + chunks * H * ((long)((Dv + 15) / 16) * DT * 256) : nullptr;
@@ -574,7 +644,8 @@ VDA_EXPORT int vda_linear_attention(
   const int DP = DT * 16, QP = DP + 4;
   const dim3 grid(nch, S - seq0, H * a.col_groups);
   auto chunk_lds = [&](bool outp) {
-    return ((size_t)16 * QP * (1 + (outp ? 1 : 0) + (z ? 1 : 0)) + (size_t)DP * 20 + (size_t)64 * ET * 20 + (z ? DP : 0) + 64) * 4;
+    return ((size_t)16 * QP * (1 + (outp ? 1 : 0) + (z ? 1 : 0)) + (size_t)DP * 20 + (size_t)64 * ET * 20 +
+            (outp ? (size_t)16 * (64 * ET + 4) : 0) + (z ? DP : 0)) * 4;
   };
 #define CK(TT, DD, EE, CC, OO)                                                                                         \
   do {                                                                                                                 \

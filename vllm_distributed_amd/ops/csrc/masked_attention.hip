@@ -42,14 +42,21 @@ struct QkExtras {
   int whole;               // one norm over all queries, one over all keys; q_w, k_w as long as the projections
 };
 
-// 1 / rms of all query values and of all key values of a token (q | k side by side in `row`), every thread of the block
-template <typename T>
+// 1 / rms of all query values and of all key values of a token (q | k side by side in `row`), every thread of the block;
+// VEC values per load (q_len and k_len multiples of it)
+template <typename T, int VEC>
 __device__ __forceinline__ void whole_row_norms(const T* row, int q_len, int k_len, float eps, float& rq, float& rk) {
+  using V = T __attribute__((ext_vector_type(VEC)));
   __shared__ float red[2][4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   float sq = 0.f, sk = 0.f;
-  for (int e = tid; e < q_len; e += 256) { const float v = (float)row[e]; sq += v * v; }
-  for (int e = tid; e < k_len; e += 256) { const float v = (float)row[q_len + e]; sk += v * v; }
+  for (int e = tid * VEC; e < q_len + k_len; e += 256 * VEC) {
+    const V v = *reinterpret_cast<const V*>(row + e);
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) ss += (float)v[i] * (float)v[i];
+    if (e < q_len) sq += ss; else sk += ss;
+  }
   sq = wave_sum(sq);
   sk = wave_sum(sk);
   if (lane == 0) { red[0][wave] = sq; red[1][wave] = sk; }
@@ -87,7 +94,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_cache_kernel(
   const float qt = query_temperature(x, positions[t]);
   const int nq = H * maps, nk = G * maps;
   float rq = 1.f, rk = 1.f;
-  if (x.whole) whole_row_norms<T>(row, nq * D, nk * D, eps, rq, rk);
+  if (x.whole) whole_row_norms<T, 1>(row, nq * D, nk * D, eps, rq, rk);
   // one wave per D-wide unit: the query maps first, then the key maps
   for (int u = wave; u < nq + nk; u += 4) {
     const bool is_q = u < nq;
@@ -158,7 +165,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_cache_vec_kernel(
   const float qt = query_temperature(xo, positions[t]);
   const int nq = H * maps, nk = G * maps, total = nq + nk;
   float rq = 1.f, rk = 1.f;
-  if (xo.whole) whole_row_norms<T>(row, nq * D, nk * D, eps, rq, rk);
+  if (xo.whole) whole_row_norms<T, 8>(row, nq * D, nk * D, eps, rq, rk);
   for (int u0 = 0; u0 < total; u0 += UPB) {
     const int u = u0 + tid / LPU;
     const bool live = u < total;
@@ -565,11 +572,41 @@ __global__ __launch_bounds__(256) void map_combine_kernel(T* __restrict__ out, c
   }
 }
 
+// one map and one gate per head: out = a * sigmoid(gate[t, h]), eight values per thread
+template <typename T>
+__global__ __launch_bounds__(256) void head_gate_kernel(T* __restrict__ out, const T* __restrict__ a,
+                                                        const T* __restrict__ gate, long gate_stride, long n8, int H,
+                                                        int per) {
+  using V8 = typename Vec<T>::v8;
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;          // per = Dv / 8 vectors of a head
+  if (i >= n8) return;
+  const long row = i / per;
+  const float g = 1.f / (1.f + expf(-(float)gate[row / H * gate_stride + row % H]));
+  const V8 v = ld16<V8>(a + i * 8);
+  V8 o;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) o[j] = (T)((float)v[j] * g);
+  st16<V8>(out + i * 8, o);
+}
+
 VDA_EXPORT int vda_map_combine(void* out, const void* a, const float* lam, const void* gate, long gate_stride,
                                int gate_heads, int T, int H, int G, int Dv, int maps, float eps, float out_scale, int dtype, hipStream_t st) {
   if (T <= 0) return 0;
   if (H % G || maps < 1 || maps > 2 || (maps == 2 && !lam)) return -1;
   const long rows = (long)T * H;
+  if (maps == 1 && gate && gate_heads && Dv % 8 == 0 && (uintptr_t)a % 32 == 0 && (uintptr_t)out % 32 == 0) {
+    const long n8 = rows * (Dv / 8);
+    const dim3 gg((unsigned)((n8 + 255) / 256));
+#define LG(TT) hipLaunchKernelGGL((head_gate_kernel<TT>), gg, dim3(256), 0, st, (TT*)out, (const TT*)a,                \
+                                  (const TT*)gate, gate_stride, n8, H, Dv / 8)
+    if (dtype == VDA_BF16) LG(bf16_t);
+    else if (dtype == VDA_F16) LG(f16_t);
+    else if (dtype == VDA_F32) LG(float);
+    else return -3;
+#undef LG
+    VDA_CHECK_LAUNCH();
+    return 0;
+  }
 #define L(TT) hipLaunchKernelGGL((map_combine_kernel<TT>), dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, st,         \
                                  (TT*)out, (const TT*)a, lam, (const TT*)gate, gate_stride, gate_heads, rows, H, G, Dv, maps, eps, \
                                  out_scale)

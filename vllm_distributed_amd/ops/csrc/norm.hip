@@ -754,7 +754,7 @@ VDA_EXPORT int vda_fp32_rows_dot(float* out, const void* x, long x_stride, const
 //     x += extra (a row in the activation type) + step (one fp32 row for all tokens)
 //     h  = tanh(alpha * x) * nw + nb                                                 the next sub-layer's input
 // Branches with a weight are divided by their root mean square over the row first (two parallel mixers whose outputs are
-// normed before they are summed); their rows are read once for the sums and, from cache, once more for the update.
+// normed before they are summed).
 struct SquashArgs {
   float* x;
   const void* y[2];
@@ -784,32 +784,59 @@ __device__ __forceinline__ float squash_tanh(float z) {
   return copysignf(1.f - 2.f / (e + 1.f), z);
 }
 
-template <typename T, int VEC, int BLOCK>
+// TRIPS > 0: TRIPS * BLOCK * VEC values cover the row, which is read once and kept in registers; 0: any width, branches
+// with a weight are read a second time
+template <typename T, int VEC, int BLOCK, int TRIPS>
 __global__ __launch_bounds__(BLOCK) void residual_squash_norm_kernel(const SquashArgs a) {
   using V = T __attribute__((ext_vector_type(VEC)));
   using F = float __attribute__((ext_vector_type(VEC)));
+  constexpr int NT = TRIPS > 0 ? TRIPS : 1;
   __shared__ float red[2][BLOCK / 64];
   const long t = blockIdx.x;
   const int tid = threadIdx.x, W = a.W;
+  float* xr = a.x + t * W;
+  V yk[2][NT];
+  F xk[NT];
+  if (TRIPS > 0) {
+#pragma unroll
+    for (int k = 0; k < NT; ++k) {
+      const int c = (k * BLOCK + tid) * VEC;
+      if (c < W) {
+        xk[k] = *reinterpret_cast<const F*>(xr + c);
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+          if (b < a.nbranch) yk[b][k] = *reinterpret_cast<const V*>((const T*)a.y[b] + t * a.y_stride[b] + c);
+      }
+    }
+  }
   float rs[2] = {1.f, 1.f};
-  bool any = false;
-  for (int b = 0; b < a.nbranch; ++b) any |= a.w[b] != nullptr;
-  if (any) {
-    for (int b = 0; b < a.nbranch; ++b) {
-      if (!a.w[b]) continue;
+  if ((a.nbranch > 0 && a.w[0]) || (a.nbranch > 1 && a.w[1])) {
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      if (b >= a.nbranch || !a.w[b]) continue;
       const T* yr = (const T*)a.y[b] + t * a.y_stride[b];
       float ss = 0.f;
-      for (int c = tid * VEC; c < W; c += BLOCK * VEC) {
-        const V v = *reinterpret_cast<const V*>(yr + c);
+      if (TRIPS > 0) {
 #pragma unroll
-        for (int i = 0; i < VEC; ++i) ss += (float)v[i] * (float)v[i];
+        for (int k = 0; k < NT; ++k)
+          if ((k * BLOCK + tid) * VEC < W) {
+#pragma unroll
+            for (int i = 0; i < VEC; ++i) ss += (float)yk[b][k][i] * (float)yk[b][k][i];
+          }
+      } else {
+        for (int c = tid * VEC; c < W; c += BLOCK * VEC) {
+          const V v = *reinterpret_cast<const V*>(yr + c);
+#pragma unroll
+          for (int i = 0; i < VEC; ++i) ss += (float)v[i] * (float)v[i];
+        }
       }
       ss = wave_sum(ss);
       if ((tid & 63) == 0) red[b][tid >> 6] = ss;
     }
     __syncthreads();
-    for (int b = 0; b < a.nbranch; ++b) {
-      if (!a.w[b]) continue;
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      if (b >= a.nbranch || !a.w[b]) continue;
       float ss = 0.f;
 #pragma unroll
       for (int k = 0; k < BLOCK / 64; ++k) ss += red[b][k];
@@ -817,14 +844,14 @@ __global__ __launch_bounds__(BLOCK) void residual_squash_norm_kernel(const Squas
     }
   }
   const float al = a.h ? *a.alpha : 0.f;
-  float* xr = a.x + t * W;
-  for (int c = tid * VEC; c < W; c += BLOCK * VEC) {
-    F x = *reinterpret_cast<const F*>(xr + c);
+  auto update = [&](int c, F x, V y0, V y1) {
     F add;
 #pragma unroll
     for (int i = 0; i < VEC; ++i) add[i] = 0.f;
-    for (int b = 0; b < a.nbranch; ++b) {
-      const V y = *reinterpret_cast<const V*>((const T*)a.y[b] + t * a.y_stride[b] + c);
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      if (b >= a.nbranch) continue;
+      const V& y = b ? y1 : y0;
       if (a.w[b]) {
         const F w = *reinterpret_cast<const F*>(a.w[b] + c);
 #pragma unroll
@@ -854,6 +881,20 @@ __global__ __launch_bounds__(BLOCK) void residual_squash_norm_kernel(const Squas
       for (int i = 0; i < VEC; ++i) o[i] = (T)(squash_tanh(al * x[i]) * w[i] + bb[i]);
       *reinterpret_cast<V*>((T*)a.h + t * a.h_stride + c) = o;
     }
+  };
+  if (TRIPS > 0) {
+#pragma unroll
+    for (int k = 0; k < NT; ++k) {
+      const int c = (k * BLOCK + tid) * VEC;
+      if (c < W) update(c, xk[k], yk[0][k], yk[1][k]);
+    }
+  } else {
+    for (int c = tid * VEC; c < W; c += BLOCK * VEC) {
+      V y0, y1;
+      if (a.nbranch > 0) y0 = *reinterpret_cast<const V*>((const T*)a.y[0] + t * a.y_stride[0] + c);
+      if (a.nbranch > 1) y1 = *reinterpret_cast<const V*>((const T*)a.y[1] + t * a.y_stride[1] + c);
+      update(c, *reinterpret_cast<const F*>(xr + c), y0, y1);
+    }
   }
 }
 
@@ -872,12 +913,15 @@ VDA_EXPORT int vda_residual_squash_norm(float* x, int nbranch, const void* y0, l
                    h_stride % 4 == 0 && !((uintptr_t)y0 % al) && !((uintptr_t)y1 % al) && !((uintptr_t)extra % al) &&
                    !((uintptr_t)h % al) && !((uintptr_t)x % 16) && !((uintptr_t)w0 % 16) && !((uintptr_t)w1 % 16) &&
                    !((uintptr_t)step % 16) && !((uintptr_t)nw % 16) && !((uintptr_t)nb % 16);
-#define L3(TT, VV, BB) hipLaunchKernelGGL((residual_squash_norm_kernel<TT, VV, BB>), dim3(T), dim3(BB), 0, st, a)
+#define L3(TT, VV, BB, KK) hipLaunchKernelGGL((residual_squash_norm_kernel<TT, VV, BB, KK>), dim3(T), dim3(BB), 0, st, a)
 #define L(TT)                                                          \
   do {                                                                 \
-    if (vec && W <= 512) L3(TT, 4, 128);                               \
-    else if (vec) L3(TT, 4, 256);                                      \
-    else L3(TT, 1, 256);                                               \
+    if (vec && W <= 512) L3(TT, 4, 128, 1);                            \
+    else if (vec && W <= 1024) L3(TT, 4, 256, 1);                      \
+    else if (vec && W <= 2048) L3(TT, 4, 256, 2);                      \
+    else if (vec && W <= 4096) L3(TT, 4, 256, 4);                      \
+    else if (vec) L3(TT, 4, 256, 0);                                   \
+    else L3(TT, 1, 256, 0);                                            \
   } while (0)
   if (dtype == VDA_BF16) L(bf16_t);
   else if (dtype == VDA_F16) L(f16_t);

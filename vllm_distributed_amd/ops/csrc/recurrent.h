@@ -21,6 +21,15 @@ __device__ __forceinline__ f32x4 mfma_f32_k16(f32x4 a, f32x4 b, f32x4 c) {
   return c;
 }
 
+// two such products in turn: neither waits for the step right before it
+__device__ __forceinline__ void mfma_f32_k16_two(f32x4 a0, f32x4 b0, f32x4& c0, f32x4 a1, f32x4 b1, f32x4& c1) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    c0 = mfma_f32(a0[r], b0[r], c0);
+    c1 = mfma_f32(a1[r], b1[r], c1);
+  }
+}
+
 // sum over the 16 lanes of a DPP row, result in every lane
 __device__ __forceinline__ float row16_sum(float v) {
   v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));
