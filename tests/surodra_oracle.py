@@ -171,36 +171,140 @@ def run_list(n, loop):
         [(i, t, i == a) for t in range(loop["times"]) for i in range(a, b)] + [(i, 0, False) for i in range(b, n)]
 
 
-def model_logits(tokens, weights, config, dtype=torch.float32, trail=None):
-    """tokens: list of ids.  Returns logits [L, vocab]; ``trail`` collects the residual after every layer run."""
+def sub(weights, prefix):
+    return {n[len(prefix):]: t for n, t in weights.items() if n.startswith(prefix)}
+
+
+def forward(cfg, weights, tokens, dtype=torch.float32, want_layers=False):
+    """tokens: list of ids.  Logits [L, vocab]; with ``want_layers`` also the residual after every layer run."""
     W = {n: t.to(dtype) for n, t in weights.items()}
-    eps, mult = config["norm"]["eps"], config.get("residual_mult", 1.0)
+    eps, mult = cfg["norm"]["eps"], cfg["residual_mult"]
 
     def norm(x, name):
         return squash_norm(x, W[name + ".alpha"], W[name], W[name + ".b"])
-
-    def sub(prefix):
-        return {n[len(prefix):]: t for n, t in W.items() if n.startswith(prefix)}
     e = W["embed"][torch.tensor(tokens)]
-    x = e
-    for i, t, first in run_list(len(config["layers"]), config.get("loop")):
-        spec = config["layers"][i]
+    x, trail = e, []
+    for i, t, first in run_list(len(cfg["layers"]), cfg.get("loop")):
+        spec = cfg["layers"][i]
         if first:
             if t > 0:
                 x = x + e
             x = x + W["loop.step"][t]
-        x = x + mult * MIXERS[spec["type"]](norm(x, f"l{i}.norm1"), sub(f"l{i}.mix."), spec["mixer"], eps)
+        x = x + mult * MIXERS[spec["type"]](norm(x, f"l{i}.norm1"), sub(W, f"l{i}.mix."), spec["mixer"], eps)
         if spec.get("mlp"):
-            x = x + mult * feed_forward(norm(x, f"l{i}.norm2"), sub(f"l{i}.mlp."))
-        if trail is not None:
-            trail.append(x.clone())
-    y = norm(x, "final.norm") @ W["head"].T * config.get("logit_scale", 1.0)
-    cap = config.get("logit_softcap")
-    return cap * torch.tanh(y / cap) if cap else y
+            x = x + mult * feed_forward(norm(x, f"l{i}.norm2"), sub(W, f"l{i}.mlp."))
+        trail.append(x)
+    y = norm(x, "final.norm") @ W["head"].T * cfg["logit_scale"]
+    y = cfg["logit_softcap"] * torch.tanh(y / cfg["logit_softcap"])
+    return (y, torch.stack(trail)) if want_layers else y
 
 
-def load_folder(folder):
-    from safetensors.torch import load_file
-    with open(os.path.join(folder, "config.json")) as f:
-        config = json.load(f)
-    return config, load_file(os.path.join(folder, "model.safetensors"))
+# ---- small random models ---------------------------------------------------------------------------------------------
+def _mlp(ff):
+    return None if ff is None else {"kind": "dense", "ff": ff}
+
+
+def _rot(dims, base, factor=None):
+    if not dims:
+        return {}
+    return {"rot": {"base": base, "dims": dims, **({"scaling": {"factor": factor}} if factor else {})}}
+
+
+def delta_layer(heads=4, kv_heads=2, dim=12, vdim=20, conv=4, ff=40):
+    return {"type": "delta", "mlp": _mlp(ff),
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def parallel_layer(heads=4, kv_heads=2, dim=12, vdim=20, rot_dims=8, base=300.0, factor=3.0, scale=0.3, right_heads=3,
+                   right_dim=8, right_vdim=12, tau=5.0, rank=7, ff=40):
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, **_rot(rot_dims, base, factor)}
+    layer = {"type": "parallel", "mlp": _mlp(ff),
+             "mixer": {"left": left, "right": {"heads": right_heads, "dim": right_dim, "vdim": right_vdim, "tau": tau}}}
+    return layer, rank
+
+
+def retention_layer(heads=3, dim=12, vdim=20, decay=(0.9, 0.97, 0.995), rot_dims=12, base=500.0, ff=None):
+    return {"type": "retention", "mlp": _mlp(ff),
+            "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": list(decay), **_rot(rot_dims, base)}}
+
+
+def make_config(layers, vocab=96, width=48, eps=1e-5, loop=None, mult=0.4, logit_scale=0.7, cap=9.0):
+    """(config, ranks of the decay projections by layer); ``layers`` may hold (layer, rank) pairs."""
+    ranks = {i: l[1] for i, l in enumerate(layers) if isinstance(l, tuple)}
+    cfg = {"architecture": "Surodra", "vocab": vocab, "width": width, "norm": {"eps": eps}, "residual_mult": mult,
+           "logit_scale": logit_scale, "logit_softcap": cap,
+           "layers": [l[0] if isinstance(l, tuple) else l for l in layers]}
+    if loop:
+        cfg["loop"] = {"start": loop[0], "stop": loop[1], "times": loop[2]}
+    return cfg, ranks
+
+
+def make_weights(cfg, ranks, seed=0):
+    g = torch.Generator().manual_seed(seed)
+    Wd, V = cfg["width"], cfg["vocab"]
+
+    def rnd(*shape, s=1.0):
+        return torch.randn(*shape, generator=g) * s
+
+    def lin(o, i, s=1.0):
+        return rnd(o, i, s=s / math.sqrt(i))
+
+    def near1(*shape):
+        return 1.0 + rnd(*shape, s=0.15)
+    W = {"embed": rnd(V, Wd), "head": lin(V, Wd, 6.0)}
+
+    def norm(name):
+        W.update({name: near1(Wd), name + ".b": rnd(Wd, s=0.2), name + ".alpha": 0.5 + 0.3 * torch.rand((), generator=g)})
+    norm("final.norm")
+    if cfg.get("loop"):
+        W["loop.step"] = rnd(cfg["loop"]["times"], Wd, s=0.6)
+    for i, L in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", L["mixer"]
+        norm(p + "norm1")
+        if L["type"] == "delta":
+            H, G, D, E = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            W.update({p + "mix.q": lin(G * D, Wd, 2.0), p + "mix.k": lin(G * D, Wd, 2.0), p + "mix.v": lin(H * E, Wd, 3.0),
+                      p + "mix.b": lin(H, Wd, 2.0), p + "mix.a": lin(H, Wd, 2.0), p + "mix.g": lin(H * E, Wd, 2.0),
+                      p + "mix.o": lin(Wd, H * E, 3.0), p + "mix.A_log": rnd(H, s=0.5) - 1.0, p + "mix.dt_bias": rnd(H) - 2.0,
+                      p + "mix.norm": near1(E)})
+            for n, c in (("q", G * D), ("k", G * D), ("v", H * E)):
+                W[p + f"mix.{n}.conv"] = rnd(c, m["conv"], s=0.8)
+        elif L["type"] == "retention":
+            H, D, E = m["heads"], m["dim"], m["vdim"]
+            W.update({p + "mix.q": lin(H * D, Wd, 2.0), p + "mix.k": lin(H * D, Wd, 2.0), p + "mix.v": lin(H * E, Wd, 2.0),
+                      p + "mix.g": lin(H * E, Wd, 2.0), p + "mix.o": lin(Wd, H * E, 3.0)})
+        else:
+            a, b, R = m["left"], m["right"], ranks[i]
+            H, G, D, E = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            W.update({p + "mix.left.q": lin(H * D, Wd, 2.0), p + "mix.left.k": lin(G * D, Wd, 2.0),
+                      p + "mix.left.v": lin(G * E, Wd, 2.0), p + "mix.left.q.norm": 1.5 * near1(H * D),
+                      p + "mix.left.k.norm": 1.5 * near1(G * D), p + "mix.left.sink": rnd(H) + 1.0,
+                      p + "mix.left.g": lin(H, Wd, 2.0), p + "mix.left.o": lin(Wd, H * E), p + "mix.left.out": 2.0 * near1(Wd)})
+            H, D, E = b["heads"], b["dim"], b["vdim"]
+            W.update({p + "mix.right.q": lin(H * D, Wd, 2.0), p + "mix.right.k": lin(H * D, Wd, 2.0),
+                      p + "mix.right.v": lin(H * E, Wd, 2.0), p + "mix.right.g": lin(H * E, Wd, 2.0),
+                      p + "mix.right.o": lin(Wd, H * E), p + "mix.right.norm": near1(E), p + "mix.right.a1": lin(R, Wd, 2.0),
+                      p + "mix.right.a2": lin(H * D, R, 2.0), p + "mix.right.a2.b": rnd(H * D) + 1.0,
+                      p + "mix.right.out": 2.0 * near1(Wd)})
+        if L.get("mlp"):
+            norm(p + "norm2")
+            ff = L["mlp"]["ff"]
+            W.update({p + "mlp.gate": lin(ff, Wd, 2.5), p + "mlp.up": lin(ff, Wd, 2.5), p + "mlp.down": lin(Wd, ff, 2.0)})
+    # the checkpoint holds bfloat16: round once, so that oracle and engine read the same numbers
+    return {k: v.to(torch.bfloat16) for k, v in W.items()}
+
+
+def save_checkpoint(folder, cfg, W):
+    from safetensors.torch import save_file
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    save_file({k: v.contiguous() for k, v in W.items()}, os.path.join(folder, "model.safetensors"))
+    return folder
+
+
+def logit_error(got, want):
+    """Root mean square difference over the vocabulary with the mean taken off, relative to the logits' own spread."""
+    d = torch.as_tensor(got).float() - torch.as_tensor(want).float()
+    d = d - d.mean(-1, keepdim=True)
+    return (d.pow(2).mean(-1).sqrt() / torch.as_tensor(want).float().std(-1).clamp_min(1e-6)).max().item()
