@@ -170,9 +170,10 @@ def main() -> None:
         argv = (["--models", "rapovik,jamba-moe"] if a.compare_rapovik else
                 ["--models", "sevazen,mixtral-swa"] if a.compare_sevazen else
                 ["--models", "lefolorn,sevazen,mixtral-swa"] if a.compare_lefolorn else
-                ["--models", "surodra,nositar,jamba"] if a.compare_surodra else []) + ["--sizes", a.sizes, "--batch", str(32 if a.batch == 256 else a.batch),
-                "--input-len", str(2048 if a.input_len == 1024 else a.input_len),
-                "--output-len", str(64 if a.output_len == 128 else a.output_len)]
+                ["--models", "surodra,nositar,jamba"] if a.compare_surodra else [])
+        argv += ["--sizes", a.sizes, "--batch", str(32 if a.batch == 256 else a.batch),
+                 "--input-len", str(2048 if a.input_len == 1024 else a.input_len),
+                 "--output-len", str(64 if a.output_len == 128 else a.output_len)]
         hybrid_compare.main(argv + (["--enforce-eager"] if a.enforce_eager else []))
         return
     if a.pp < 1 or a.gpus % a.pp:

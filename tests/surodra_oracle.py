@@ -228,7 +228,7 @@ def retention_layer(heads=3, dim=12, vdim=20, decay=(0.9, 0.97, 0.995), rot_dims
             "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": list(decay), **_rot(rot_dims, base)}}
 
 
-def make_config(layers, vocab=96, width=48, eps=1e-5, loop=None, mult=0.4, logit_scale=0.7, cap=9.0):
+def make_config(layers, vocab=96, width=48, eps=1e-2, loop=None, mult=0.3, logit_scale=0.7, cap=9.0):
     """(config, ranks of the decay projections by layer); ``layers`` may hold (layer, rank) pairs."""
     ranks = {i: l[1] for i, l in enumerate(layers) if isinstance(l, tuple)}
     cfg = {"architecture": "Surodra", "vocab": vocab, "width": width, "norm": {"eps": eps}, "residual_mult": mult,
@@ -263,23 +263,24 @@ def make_weights(cfg, ranks, seed=0):
         norm(p + "norm1")
         if L["type"] == "delta":
             H, G, D, E = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-            W.update({p + "mix.q": lin(G * D, Wd, 2.0), p + "mix.k": lin(G * D, Wd, 2.0), p + "mix.v": lin(H * E, Wd, 3.0),
+            W.update({p + "mix.q": lin(G * D, Wd, 2.0), p + "mix.k": lin(G * D, Wd, 2.0), p + "mix.v": lin(H * E, Wd, 2.0),
                       p + "mix.b": lin(H, Wd, 2.0), p + "mix.a": lin(H, Wd, 2.0), p + "mix.g": lin(H * E, Wd, 2.0),
-                      p + "mix.o": lin(Wd, H * E, 3.0), p + "mix.A_log": rnd(H, s=0.5) - 1.0, p + "mix.dt_bias": rnd(H) - 2.0,
+                      p + "mix.o": lin(Wd, H * E, 1.5), p + "mix.A_log": rnd(H, s=0.5) - 1.0, p + "mix.dt_bias": rnd(H) - 2.0,
                       p + "mix.norm": near1(E)})
             for n, c in (("q", G * D), ("k", G * D), ("v", H * E)):
                 W[p + f"mix.{n}.conv"] = rnd(c, m["conv"], s=0.8)
         elif L["type"] == "retention":
             H, D, E = m["heads"], m["dim"], m["vdim"]
             W.update({p + "mix.q": lin(H * D, Wd, 2.0), p + "mix.k": lin(H * D, Wd, 2.0), p + "mix.v": lin(H * E, Wd, 2.0),
-                      p + "mix.g": lin(H * E, Wd, 2.0), p + "mix.o": lin(Wd, H * E, 3.0)})
+                      p + "mix.g": lin(H * E, Wd, 2.0), p + "mix.o": lin(Wd, H * E, 1.5)})
         else:
             a, b, R = m["left"], m["right"], ranks[i]
             H, G, D, E = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
             W.update({p + "mix.left.q": lin(H * D, Wd, 2.0), p + "mix.left.k": lin(G * D, Wd, 2.0),
                       p + "mix.left.v": lin(G * E, Wd, 2.0), p + "mix.left.q.norm": 1.5 * near1(H * D),
                       p + "mix.left.k.norm": 1.5 * near1(G * D), p + "mix.left.sink": rnd(H) + 1.0,
-                      p + "mix.left.g": lin(H, Wd, 2.0), p + "mix.left.o": lin(Wd, H * E), p + "mix.left.out": 2.0 * near1(Wd)})
+                      p + "mix.left.g": lin(H, Wd, 2.0), p + "mix.left.o": lin(Wd, H * E),
+                      p + "mix.left.out": 2.0 * near1(Wd)})
             H, D, E = b["heads"], b["dim"], b["vdim"]
             W.update({p + "mix.right.q": lin(H * D, Wd, 2.0), p + "mix.right.k": lin(H * D, Wd, 2.0),
                       p + "mix.right.v": lin(H * E, Wd, 2.0), p + "mix.right.g": lin(H * E, Wd, 2.0),

@@ -16,7 +16,7 @@ CASES = [("cpu", "float32"), pytest.param("cuda", "float32", marks=pytest.mark.g
 OP_CASES = [("cpu", torch.float32), pytest.param("cuda", torch.float32, marks=pytest.mark.gpu),
             pytest.param("cuda", torch.bfloat16, marks=pytest.mark.gpu)]
 # 16-bit: models this narrow (48 values per row) average little rounding away; the crafted cases move by more
-TOL = {"float32": 3e-4, "bfloat16": 0.15}
+TOL = {"float32": 3e-4, "bfloat16": 0.12}
 OP_TOL = {torch.float32: 3e-5, torch.bfloat16: 2.5e-2}
 
 
@@ -180,7 +180,7 @@ def test_linearly_scaled_frequencies():
 
 # (heads, key heads, D, Dv, rotated, page size): any-size kernel and, in 16 bits, the matrix-core forms
 ATTN = [(4, 2, 12, 20, 8, 16), (3, 1, 20, 8, 0, 32), (1, 1, 5, 7, 4, 16), (8, 2, 64, 64, 16, 16), (4, 4, 128, 128, 128, 32),
-        (2, 1, 72, 40, 6, 16)]
+        (2, 1, 72, 40, 6, 16), (16, 1, 64, 64, 12, 16), (4, 2, 96, 96, 32, 32), (2, 2, 256, 256, 48, 16)]
 
 
 @pytest.mark.parametrize("dev,dt", OP_CASES)
@@ -326,8 +326,8 @@ def test_gated_linear_attention(dev, dt, H, D, E, tau, bias):
 
     def launch(x, qsl, lens, tbl, longest, few, pos):
         return ops.linear_attention(x[:, :nk], x[:, nk: 2 * nk], x[:, 2 * nk: 2 * nk + nv],
-                                    x[:, 2 * nk + nv: 2 * nk + 2 * nv], P["norm"].to(dev), state, qsl, lens, tbl, H, D, E, eps,
-                                    longest, z=x[:, 2 * nk + 2 * nv:], z_bias=P["a2.b"].to(dev), tau=tau,
+                                    x[:, 2 * nk + nv: 2 * nk + 2 * nv], P["norm"].to(dev), state, qsl, lens, tbl, H, D, E,
+                                    eps, longest, z=x[:, 2 * nk + 2 * nv:], z_bias=P["a2.b"].to(dev), tau=tau,
                                     q_scale=D ** -0.5, first_long_seq=few)
     got = in_portions(xs, dev, dt, launch)
     for g, w in zip(got, want):
@@ -402,7 +402,7 @@ VARIANTS = {
                                O.delta_layer(heads=6, kv_heads=3, dim=16, vdim=4, conv=5)], loop=(1, 2, 2), mult=1.0),
     "parallel_only": dict(layers=[O.parallel_layer(heads=1, kv_heads=1, dim=4, vdim=6, rot_dims=2, factor=None, ff=None),
                                   O.parallel_layer(heads=6, kv_heads=2, dim=10, vdim=4, rot_dims=10, right_heads=2,
-                                                   right_dim=4, right_vdim=40, tau=12.0, rank=20)], cap=2.0),
+                                                   right_dim=4, right_vdim=40, tau=12.0, rank=20)], cap=2.0, eps=1e-6),
     "retention_only": dict(layers=[O.retention_layer(heads=1, dim=40, vdim=8, decay=(0.99,), rot_dims=0),
                                    O.retention_layer(heads=2, dim=6, vdim=36, decay=(0.7, 0.9999), rot_dims=4, ff=17)],
                            loop=(0, 1, 4), logit_scale=1.0),
@@ -425,8 +425,8 @@ def test_whole_prompt(tmp_path, dev, dtype, name):
 
 
 def test_the_loops_additions_matter():
-    """The oracle itself: the step rows of every pass, the embedding output between passes, the sinks and the soft cap
-    change the logits by far more than the tests' tolerance."""
+    """The oracle itself: the step rows of every pass, the sinks and the soft cap change the logits by far more than the
+    fp32 tolerance of the comparisons above and below."""
     cfg, ranks = O.make_config(mixed_layers(), loop=(1, 4, 2))
     W = O.make_weights(cfg, ranks, 3)
     p = tokens(12, cfg["vocab"], 1)
@@ -437,7 +437,7 @@ def test_the_loops_additions_matter():
             t[:] = -60.0
         else:
             t[row] = 0
-        assert O.logit_error(O.forward(cfg, dict(W, **{k: t}), p), full) > 0.1, (k, row)
+        assert O.logit_error(O.forward(cfg, dict(W, **{k: t}), p), full) > 0.05, (k, row)
     assert O.logit_error(O.forward(dict(cfg, logit_softcap=1e6), W, p), full) > 0.02
 
 
@@ -562,7 +562,8 @@ def test_far_token_decides(tmp_path, dev, dtype, kind):
     cfg, W = needle_model(kind)
     folder = O.save_checkpoint(str(tmp_path / "m"), cfg, W)
     body = [t % 63 + 1 for t in tokens(460, 64, 12)]
-    prompts = {"first": [0] + body[:99], "page_end": body[:15] + [0] + body[15:60], "page_start": body[:16] + [0] + body[16:60],
+    prompts = {"first": [0] + body[:99], "page_end": body[:15] + [0] + body[15:60],
+               "page_start": body[:16] + [0] + body[16:60],
                "far": body[:3] + [0] + body[3:440]}
     sched = [[("first", 1), ("page_end", 16)], [("first", 60), ("page_end", 2)], [("first", 1), ("page_end", 30)],
              [("first", 38), ("page_end", 13)], [("page_start", 17), ("far", 150)], [("page_start", 1), ("far", 200)],

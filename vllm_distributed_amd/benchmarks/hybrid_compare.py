@@ -1,5 +1,5 @@
-"""Prefill and decode throughput of a Nositar, Rapovik, Sevazen, Lefolorn or Surodra stack beside the closest existing models of
-equal size, random weights.
+"""Prefill and decode throughput of a Nositar, Rapovik, Sevazen, Lefolorn or Surodra stack beside the closest existing
+models of equal size, random weights.
 
     python bench.py --compare-nositar [--sizes small,medium] [--batch 32] [--input-len 2048] [--output-len 64]
     python bench.py --compare-rapovik [...]        (rapovik beside jamba-moe)
@@ -178,8 +178,9 @@ def surodra_config(s: dict) -> dict:
             "layers": [(delta, par, ret)[i % 3] for i in range(s["layers"])]}
 
 
-MODELS = {"surodra": surodra_config, "lefolorn": lefolorn_config, "sevazen": sevazen_config, "mixtral-swa": mixtral_swa_config, "nositar": nositar_config, "llama-swa": llama_config, "jamba": jamba_config, "jamba-moe": jamba_moe_config,
-          "rapovik": rapovik_config}
+MODELS = {"surodra": surodra_config, "lefolorn": lefolorn_config, "sevazen": sevazen_config,
+          "mixtral-swa": mixtral_swa_config, "nositar": nositar_config, "llama-swa": llama_config, "jamba": jamba_config,
+          "jamba-moe": jamba_moe_config, "rapovik": rapovik_config}
 
 
 def run_one(kind: str, size: str, batch: int, input_len: int, output_len: int, eager: bool) -> dict:

@@ -346,8 +346,8 @@ class ModelConfig:
                          # encoder-decoder: the cross-attention cache is per-request state of the same kind
                          "WhisperForConditionalGeneration", "BartForConditionalGeneration", "BartModel",
                          "MllamaForConditionalGeneration", "Zamba2ForCausalLM", "Plamo2ForCausalLM",
-                         "Florence2ForConditionalGeneration", "NositarForCausalLM", "RapovikForCausalLM", "SevazenForCausalLM",
-                         "SurodraForCausalLM")
+                         "Florence2ForConditionalGeneration", "NositarForCausalLM", "RapovikForCausalLM",
+                         "SevazenForCausalLM", "SurodraForCausalLM")
                    for a in self.architectures)
 
     @property

@@ -12,7 +12,8 @@ head and key channel or one per head.
 
 The state (S and the convolution's last taps - 1 inputs) lives in the runner's per-request state slots, the
 mechanism of the other recurrent mixers; everything the recurrence consumes besides the projections is fp32.
-Kernels: ops/csrc/delta_rule.hip (the recurrence, norms, decays, gates, output norm), ops/csrc/mamba.hip (the convolution, shared with the state-space mixers).
+Kernels: ops/csrc/delta_rule.hip (the recurrence, norms, decays, gates, output norm), ops/csrc/mamba.hip (the
+convolution, shared with the state-space mixers).
 """
 from __future__ import annotations
 

@@ -63,9 +63,9 @@ _HALF_SPLIT_TABLES: dict = {}
 
 def half_split_cos_sin(max_len: int, rot_dim: int, base: float, scaling: Optional[dict], device) -> torch.Tensor:
     """fp32 [max_len, rot_dim] for kernels that rotate in fp32: cos(p f_i) for i < rot_dim / 2, then sin(p f_i), with
-    f_i = base^(-2i / rot_dim) rescaled by ``scaling``: None, {"kind": "linear", factor} (every f_i divided by it), {"kind": "llama3", factor, low, high, original} or
-    {"kind": "yarn", factor, original, fast, slow, magnitude} (cos and sin times ``magnitude``).  Angles are formed in
-    fp64 and rounded once."""
+    f_i = base^(-2i / rot_dim) rescaled by ``scaling``: None, {"kind": "linear", factor} (every f_i
+    divided by it), {"kind": "llama3", factor, low, high, original} or {"kind": "yarn", factor, original, fast, slow,
+    magnitude} (cos and sin times ``magnitude``).  Angles are formed in fp64 and rounded once."""
     sc = dict(scaling or {})
     key = (int(max_len), int(rot_dim), float(base), tuple(sorted(sc.items())), str(device))
     t = _HALF_SPLIT_TABLES.get(key)

@@ -1984,7 +1984,8 @@ def masked_softmax_attention(qn: torch.Tensor, k_cache: torch.Tensor, v_cache: t
     N.call("vda_masked_softmax_attention", out.data_ptr(), qn.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
            block_table.data_ptr(), block_table.stride(0), seq_lens.data_ptr(), query_start_loc.data_ptr(),
            N.ptr(sink), N.ptr(lam), N.ptr(gate), gate.stride(0) if gate is not None else 0,
-           int(gate is not None and gate.shape[1] != H * Dv), float(scale), int(window), int(chunk), int(maps), float(eps), float(out_scale), seq_lens.shape[0], H, G, MD // maps, Dv, bs,
+           int(gate is not None and gate.shape[1] != H * Dv), float(scale), int(window),
+           int(chunk), int(maps), float(eps), float(out_scale), seq_lens.shape[0], H, G, MD // maps, Dv, bs,
            max(int(max_query_len), 1), float(softcap), N.ptr(dist_bias),
            dist_bias.shape[0] - 1 if dist_bias is not None else 0, N.dt(out_dtype), N.stream())
     return out

@@ -32,9 +32,6 @@
 // sequence was cut.
 #include "recurrent.h"
 
-__device__ __forceinline__ float dr_softplus(float v) { return v > 20.f ? v : log1pf(expf(v)); }
-__device__ __forceinline__ float dr_sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
-
 // grid: tokens; one wave per (token, vector): G query vectors, G key vectors (with their dot products), H decays
 template <typename T>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(
@@ -69,7 +66,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
       dot = wave_sum(dot);
       // per head: [beta, q^ . k^]
       for (int h = v * rep + lane; h < (v + 1) * rep; h += 64) {
-        sc[(t * H + h) * 2] = dr_sigmoid((float)b_raw[t * b_stride + h]);
+        sc[(t * H + h) * 2] = rec_sigmoid((float)b_raw[t * b_stride + h]);
         sc[(t * H + h) * 2 + 1] = dot;
       }
     } else {
@@ -77,7 +74,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
       const float a_scale = expf(a_log[h]);
       for (int d = lane; d < Dp; d += 64)
         dec[(t * H + h) * Dp + d] =
-            d < D ? expf(-a_scale * dr_softplus((float)a_raw[t * a_stride + (long)h * D + d] + dt_bias[(long)h * D + d]))
+            d < D ? expf(-a_scale * rec_softplus((float)a_raw[t * a_stride + (long)h * D + d] + dt_bias[(long)h * D + d]))
                   : 0.f;
     }
   }
@@ -219,7 +216,7 @@ __global__ __launch_bounds__(256) void delta_out_norm_gate_kernel(T* __restrict_
   ss = wave_sum(ss);
   const float rs = 1.f / sqrtf(ss / (float)Dv + eps);
   for (int j = lane; j < Dv; j += 64) {
-    const float gt = dr_sigmoid((float)gate_raw[t * g_stride + (long)h * Dv + j]);
+    const float gt = rec_sigmoid((float)gate_raw[t * g_stride + (long)h * Dv + j]);
     out[t * o_stride + (long)h * Dv + j] = (T)(o[j] * rs * norm_w[j] * gt);
   }
 }
@@ -533,8 +530,8 @@ __global__ __launch_bounds__(256) void delta_block_prepare_kernel(const DeltaHea
 
 // grid (H, sequences, groups of 64 columns): walks the blocks of its sequence, S of sixteen columns per wave in
 // accumulators.  A block's operands (read by all four waves) sit in one of two LDS buffers while those of the next two
-// blocks are on their way from memory; one barrier per block.  The column group is the slowest grid index, so that workgroups that
-// read the same blocks tend to share an L2.
+// blocks are on their way from memory; one barrier per block.  The column group is the slowest grid index, so that
+// workgroups that read the same blocks tend to share an L2.
 template <typename T, int DT>
 __global__ __launch_bounds__(256) void delta_block_walk_kernel(const DeltaHeadArgs a) {
   constexpr int DP = DT * 16, NV = 48 * DP, BUF = NV + DELTA_MAT;

@@ -11,7 +11,8 @@
 // Sequences with few new tokens (decoding, short portions):
 //   step   one workgroup per (sequence, head), token by token, everything in one launch: the state is read and written
 //          once, norm and gate included.
-// Longer ones (when the rows allow 4-value accesses; otherwise `step` walks them too), chunk-parallel (fp32 matrix instructions, see recurrent.h): a sequence is cut into chunks of C tokens,
+// Longer ones (when the rows allow 4-value accesses; otherwise `step` walks them too), chunk-parallel on the fp32 matrix
+// instruction (recurrent.h), a sequence cut into chunks of C tokens:
 //   chunk<OUT = false>   per (chunk, head): the state the chunk alone would build, and its total decay
 //   carry                per (sequence, head): the state at every chunk's start, one after the other (elementwise)
 //   chunk<OUT = true>    per (chunk, head): from that state, sixteen tokens at a time:
@@ -376,7 +377,10 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
     if (OUT && !a.o_raw) {                             // this block's gates; used when its output leaves
       const long t = min(tb + tt, L - 1);
 #pragma unroll
-      for (int m = 0; m < NVI; ++m) rg[m] = *reinterpret_cast<const V4*>(gp + t * a.g_stride + (d0 + 64 * m < Dv ? d0 + 64 * m : 0));
+      for (int m = 0; m < NVI; ++m) {
+        const int cc = d0 + 64 * m;
+        rg[m] = *reinterpret_cast<const V4*>(gp + t * a.g_stride + (cc < Dv ? cc : 0));
+      }
     }
     if (tb + 16 < end) fetch(tb + 16);
     __syncthreads();
@@ -414,7 +418,8 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
       for (int m = 0; m < NI; ++m) {
         const int d = d0 + 64 * m;
         if (DP < 64 && d >= DP) continue;
-        const f32x4 b = *reinterpret_cast<const f32x4*>(bc + tt * QP + d), bn = *reinterpret_cast<const f32x4*>(bc + 15 * QP + d);
+        const f32x4 b = *reinterpret_cast<const f32x4*>(bc + tt * QP + d);
+        const f32x4 bn = *reinterpret_cast<const f32x4*>(bc + 15 * QP + d);
         f32x4 k = *reinterpret_cast<const f32x4*>(ks + tt * QP + d);
 #pragma unroll
         for (int i = 0; i < 4; ++i) kT[(d + i) * TP + tt] = k[i] * expf(bn[i] - b[i]);
@@ -589,7 +594,8 @@ VDA_EXPORT int vda_linear_attention(
   const int es = dtype == VDA_F32 ? 16 : 8;
   auto ok4 = [&](const void* p, long stride) { return !p || (((uintptr_t)p % es) == 0 && stride % 4 == 0); };
   const bool vec = D % 4 == 0 && ok4(q, q_stride) && ok4(k, k_stride) && ok4(z, z_stride);
-  const bool vec_v = Dv % 4 == 0 && ok4(v, v_stride) && ok4(gate, g_stride) && ok4(out, o_stride) && !((uintptr_t)norm_w % 16);
+  const bool vec_v = Dv % 4 == 0 && ok4(v, v_stride) && ok4(gate, g_stride) && ok4(out, o_stride) &&
+                     !((uintptr_t)norm_w % 16);
   const bool chunked = D <= 256 && max_q > 16 && scratch && seq0 < S && C >= 16 && C % 16 == 0 && vec && vec_v &&
                        rot % 8 == 0 && (!z || rot == 0) && !((uintptr_t)z_bias % 16) && !((uintptr_t)cos_sin % 16);
   const int DT = lin_dt(D);

@@ -476,7 +476,8 @@ VDA_EXPORT int vda_masked_softmax_attention(void* out, const void* qn, const voi
                                             const int* block_table, long bt_stride, const int* seq_lens,
                                             const int* qsl, const float* sink, const float* lam, const void* gate,
                                             long gate_stride, int gate_heads, float scale, int window, int chunk,
-                                            int maps, float eps, float out_scale, int S, int H, int G, int D, int Dv, int bs, int max_q,
+                                            int maps, float eps, float out_scale, int S, int H, int G, int D,
+                                            int Dv, int bs, int max_q,
                                             float softcap, const float* dist_bias, int far, int dtype,
                                             hipStream_t st) {
   if (S <= 0 || max_q <= 0) return 0;
@@ -512,7 +513,8 @@ VDA_EXPORT int vda_masked_softmax_attention(void* out, const void* qn, const voi
   MaskedAttnArgs a;
   a.out = out; a.qn = qn; a.k_cache = k_cache; a.v_cache = v_cache; a.block_table = block_table;
   a.bt_stride = bt_stride; a.seq_lens = seq_lens; a.qsl = qsl; a.sink = sink; a.lam = lam; a.gate = gate;
-  a.gate_stride = gate_stride; a.gate_heads = gate_heads; a.scale = scale; a.eps = eps; a.out_scale = out_scale; a.window = window;
+  a.gate_stride = gate_stride; a.gate_heads = gate_heads;
+  a.scale = scale; a.eps = eps; a.out_scale = out_scale; a.window = window;
   a.chunk = chunk; a.maps = maps; a.H = H; a.G = G; a.D = D; a.Dv = Dv; a.bs = bs; a.HG = HG; a.BQ = BQ; a.BK = BK;
   a.softcap = softcap; a.dist_bias = dist_bias; a.far = far;
   dim3 grid((max_q + BQ - 1) / BQ, S, G * ((R + HG - 1) / HG)), block(256);
@@ -590,7 +592,8 @@ __global__ __launch_bounds__(256) void head_gate_kernel(T* __restrict__ out, con
 }
 
 VDA_EXPORT int vda_map_combine(void* out, const void* a, const float* lam, const void* gate, long gate_stride,
-                               int gate_heads, int T, int H, int G, int Dv, int maps, float eps, float out_scale, int dtype, hipStream_t st) {
+                               int gate_heads, int T, int H, int G, int Dv, int maps, float eps, float out_scale,
+                               int dtype, hipStream_t st) {
   if (T <= 0) return 0;
   if (H % G || maps < 1 || maps > 2 || (maps == 2 && !lam)) return -1;
   const long rows = (long)T * H;
@@ -608,7 +611,8 @@ VDA_EXPORT int vda_map_combine(void* out, const void* a, const float* lam, const
     return 0;
   }
 #define L(TT) hipLaunchKernelGGL((map_combine_kernel<TT>), dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, st,         \
-                                 (TT*)out, (const TT*)a, lam, (const TT*)gate, gate_stride, gate_heads, rows, H, G, Dv, maps, eps, \
+                                 (TT*)out, (const TT*)a, lam, (const TT*)gate, gate_stride, gate_heads, rows, H, G,    \
+                                 Dv, maps, eps,                                                                       \
                                  out_scale)
   if (dtype == VDA_BF16) L(bf16_t);
   else if (dtype == VDA_F16) L(f16_t);
