@@ -228,7 +228,7 @@ def retention_layer(heads=3, dim=12, vdim=20, decay=(0.9, 0.97, 0.995), rot_dims
             "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": list(decay), **_rot(rot_dims, base)}}
 
 
-def make_config(layers, vocab=96, width=48, eps=1e-2, loop=None, mult=0.3, logit_scale=0.7, cap=9.0):
+def make_config(layers, vocab=96, width=48, eps=1e-2, loop=None, mult=0.35, logit_scale=0.7, cap=9.0):
     """(config, ranks of the decay projections by layer); ``layers`` may hold (layer, rank) pairs."""
     ranks = {i: l[1] for i, l in enumerate(layers) if isinstance(l, tuple)}
     cfg = {"architecture": "Surodra", "vocab": vocab, "width": width, "norm": {"eps": eps}, "residual_mult": mult,

@@ -306,7 +306,7 @@ def test_delta_rule_with_a_decay_per_head(dev, dt, H, G, D, E, taps):
 
 # (heads, D, Dv, tau, decays of the channels): ordinary ones, ones that vanish within a few tokens (their running products
 # underflow inside a block), and a mixture
-GLA = [(3, 12, 20, 5.0, 1.0), (2, 64, 128, 16.0, 0.0), (1, 5, 70, 1.0, 1.0), (2, 128, 64, 0.3, -3.0), (1, 33, 8, 1.0, -6.0),
+GLA = [(3, 12, 20, 5.0, 1.0), (2, 64, 128, 12.0, 0.0), (1, 5, 70, 1.0, 1.0), (2, 128, 64, 0.3, -3.0), (1, 33, 8, 1.0, -6.0),
        (2, 160, 36, 8.0, 1.0), (1, 32, 300, 2.0, -2.0)]
 
 
@@ -514,9 +514,9 @@ def test_unequal_requests_share_steps_and_reuse_pages_and_slots(tmp_path, dev, d
 NEEDLES = {
     "delta": O.delta_layer(heads=2, kv_heads=1, dim=8, vdim=8, conv=2, ff=None),
     "left": O.parallel_layer(heads=2, kv_heads=1, dim=8, vdim=8, rot_dims=0, scale=0.3, right_heads=2, right_dim=8,
-                             right_vdim=8, tau=16.0, ff=None),
+                             right_vdim=8, tau=14.0, ff=None),
     "right": O.parallel_layer(heads=2, kv_heads=1, dim=8, vdim=8, rot_dims=0, scale=0.3, right_heads=2, right_dim=8,
-                              right_vdim=8, tau=16.0, ff=None),
+                              right_vdim=8, tau=14.0, ff=None),
     "retention": O.retention_layer(heads=2, dim=8, vdim=8, decay=(0.9999, 0.9998), rot_dims=0),
 }
 

@@ -168,13 +168,13 @@ def surodra_config(s: dict) -> dict:
     delta = {"type": "delta", "mlp": mlp, "mixer": {"heads": hh, "kv_heads": hh, "dim": 128, "vdim": 128, "conv": 4}}
     par = {"type": "parallel", "mlp": mlp,
            "mixer": {"left": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5,
-                              "rot": {"base": 500000.0, "dims": d // 4, "scaling": {"factor": 8.0}}},
-                     "right": {"heads": hh, "dim": 64, "vdim": 128, "tau": 16.0, "decay_rank": 16}}}
+                              "rot": {"base": 100000.0, "dims": d // 4, "scaling": {"factor": 4.0}}},
+                     "right": {"heads": hh, "dim": 64, "vdim": 128, "tau": 8.0, "decay_rank": 24}}}
     ret = {"type": "retention", "mlp": mlp,
            "mixer": {"heads": hh, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-5 - 5 * i / hh) for i in range(hh)],
                      "rot": {"base": 10000.0, "dims": 128}}}
-    return {"architecture": "Surodra", "vocab": s["vocab"], "width": w, "norm": {"eps": 1e-6}, "residual_mult": 0.3,
-            "logit_scale": 0.5, "logit_softcap": 15.0, "loop": {"start": 0, "stop": s["layers"], "times": 1},
+    return {"architecture": "Surodra", "vocab": s["vocab"], "width": w, "norm": {"eps": 1e-6}, "residual_mult": 0.4,
+            "logit_scale": 0.25, "logit_softcap": 20.0, "loop": {"start": 0, "stop": s["layers"], "times": 1},
             "layers": [(delta, par, ret)[i % 3] for i in range(s["layers"])]}
 
 
