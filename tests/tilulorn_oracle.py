@@ -1,0 +1,201 @@
+"""A slow, whole-sequence implementation of the Tilulorn design, one function per mechanism, written from its equations
+and sharing no code with the package: the oracle of tests/test_tilulorn.py.  Everything runs in fp32 (or fp64) on the CPU
+over one whole sequence at a time; there is no cache, no batching and no portioning here.
+
+Notation: x residual [L, W]; N(y) = y / rms(y) * w; a layer computes x <- x + mixer(N1 x), then x <- x + ff(N2 x).
+"""
+import json
+import math
+import os
+
+import torch
+
+
+# ---- norms ---------------------------------------------------------------------------------------------------------
+def unit_rms(y, eps):
+    return y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps)
+
+
+def rms_norm(y, w, eps):
+    return unit_rms(y, eps) * w
+
+
+def silu(z):
+    return z * torch.sigmoid(z)
+
+
+# ---- rotation --------------------------------------------------------------------------------------------------------
+def plain_frequencies(dims, base):
+    return [base ** (-2.0 * i / dims) for i in range(dims // 2)]
+
+
+def yarn_frequencies(dims, base, factor, original, fast, slow):
+    def turn_dim(turns):
+        return dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(base))
+    lo, hi = max(math.floor(turn_dim(fast)), 0), min(math.ceil(turn_dim(slow)), dims - 1)
+    out = []
+    for i, f in enumerate(plain_frequencies(dims, base)):
+        r = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        out.append(f / factor * r + f * (1 - r))
+    return out
+
+
+def turn(x, freqs, pairs, size=1.0):
+    """x [L, heads, D]; pair i of ``pairs`` (two index lists) turns by position * freqs[i]; cos and sin times ``size``."""
+    L = x.shape[0]
+    ang = torch.arange(L, dtype=torch.float64)[:, None] * torch.tensor(freqs, dtype=torch.float64)[None, :]
+    c, s = (size * torch.cos(ang)).to(x.dtype)[:, None, :], (size * torch.sin(ang)).to(x.dtype)[:, None, :]
+    first, second = pairs
+    a, b = x[..., first], x[..., second]
+    y = x.clone()
+    y[..., first] = a * c - b * s
+    y[..., second] = b * c + a * s
+    return y
+
+
+def rotate_neighbours(x, rot):
+    """Values 2i and 2i + 1 form a pair; every frequency divided by the factor."""
+    dims = int((rot or {}).get("dims", 0) or 0)
+    if dims == 0:
+        return x
+    factor = rot["scaling"]["factor"] if rot.get("scaling") else 1.0
+    f = [v / factor for v in plain_frequencies(dims, rot["base"])]
+    return turn(x, f, (list(range(0, dims, 2)), list(range(1, dims, 2))))
+
+
+def rotate_halves_yarn(x, rot):
+    """Values i and i + dims / 2 form a pair; frequencies of long wavelengths divided by the factor."""
+    dims = int((rot or {}).get("dims", 0) or 0)
+    if dims == 0:
+        return x
+    f, size = plain_frequencies(dims, rot["base"]), 1.0
+    sc = rot.get("scaling")
+    if sc:
+        f = yarn_frequencies(dims, rot["base"], sc["factor"], sc["original"], sc["fast"], sc["slow"])
+        size = 0.1 * math.log(sc["factor"]) + 1.0
+    return turn(x, f, (list(range(dims // 2)), list(range(dims // 2, dims))), size)
+
+
+# ---- mixers ------------------------------------------------------------------------------------------------------------
+def latent_mixer(h, w, m, eps):
+    """Keys and values come out of one normed latent per token; one rotated key part serves every head."""
+    L = h.shape[0]
+    H, D, P, E, R = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+    q = (rms_norm(h @ w["dq"].T, w["dq.norm"], eps) @ w["uq"].T).view(L, H, D + P)
+    down = h @ w["dkv"].T
+    c = rms_norm(down[:, :R], w["dkv.norm"], eps)
+    k = (c @ w["uk"].T).view(L, H, D)
+    v = (c @ w["uv"].T).view(L, H, E)
+    k_rot = rotate_halves_yarn(down[:, None, R:], m.get("rot"))[:, 0]
+    q_rot = rotate_halves_yarn(q[..., D:], m.get("rot"))
+    unseen = torch.arange(L)[None, :] > torch.arange(L)[:, None]
+    gate = torch.sigmoid(h @ w["g"].T)
+    out = []
+    for n in range(H):
+        s = (q[:, n, :D] @ k[:, n].T + q_rot[:, n] @ k_rot.T) * m["scale"]
+        p = torch.softmax(s.masked_fill(unseen, float("-inf")), -1)
+        out.append((p @ v[:, n]) * gate[:, n: n + 1])
+    return torch.cat(out, -1) @ w["o"].T
+
+
+def window_mixer(h, w, m, eps):
+    """Sliding-window attention whose values are its keys before norm and rotation; a sink in every denominator."""
+    L = h.shape[0]
+    H, G, D = m["heads"], m["kv_heads"], m["dim"]
+    k_raw = h @ w["k"].T
+    q = rms_norm(h @ w["q"].T, w["q.norm"], eps)             # over the whole projection, not per head
+    k = rms_norm(k_raw, w["k.norm"], eps)
+    v = k_raw.view(L, G, D)
+    q, k = rotate_neighbours(q.view(L, H, D), m.get("rot")), rotate_neighbours(k.view(L, G, D), m.get("rot"))
+    back = torch.arange(L)[:, None] - torch.arange(L)[None, :]
+    seen = back >= 0
+    if m.get("mask"):
+        seen = seen & (back < m["mask"]["size"])
+    gate = torch.sigmoid(h @ w["g"].T)
+    out = []
+    for n in range(H):
+        g = n // (H // G)
+        s = ((q[:, n] @ k[:, g].T) * m["scale"]).masked_fill(~seen, float("-inf"))
+        top = torch.maximum(s.max(-1, keepdim=True).values, w["sink"][n])
+        e = torch.exp(s - top)
+        p = e / (e.sum(-1, keepdim=True) + torch.exp(w["sink"][n] - top))
+        out.append((p @ v[:, g]) * gate[:, n: n + 1])
+    return torch.cat(out, -1) @ w["o"].T
+
+
+def shifted_mix(h, mu):
+    """h + (h' - h) mu, h' the row of the token before (zeros before the first)."""
+    before = torch.cat([torch.zeros_like(h[:1]), h[:-1]])
+    return h + (before - h) * mu
+
+
+def bonus_memory(r, k, v, decay, u):
+    """r, k, decay [L, H, D], v [L, H, E], u [H, D]: read the old memory plus the own token through the bonus, then fade
+    and write:  o_t = (S + diag(u) k_t v_t^T)^T r_t,  S <- diag(decay_t) S + k_t v_t^T."""
+    L, H, D = r.shape
+    S = torch.zeros(H, D, v.shape[-1], dtype=r.dtype)
+    out = []
+    for t in range(L):
+        kv = k[t][:, :, None] * v[t][:, None, :]
+        out.append(((S + u[:, :, None] * kv) * r[t][:, :, None]).sum(1))
+        S = decay[t][:, :, None] * S + kv
+    return torch.stack(out)
+
+
+def wkv_mixer(h, w, m, eps):
+    L = h.shape[0]
+    H, D = m["heads"], m["dim"]
+    mix = {s: shifted_mix(h, w["mu." + s]) for s in "rkvgw"}
+    r, k, v = ((mix[s] @ w[s].T).view(L, H, D) for s in "rkv")
+    z = torch.tanh(mix["w"] @ w["w1"].T) @ w["w2"].T + w["w0"]
+    decay = torch.exp(-torch.exp(z)).view(L, H, D)
+    o = unit_rms(bonus_memory(r, k, v, decay, w["u"]), eps).reshape(L, H * D) * w["norm"]
+    return (o * silu(mix["g"] @ w["g"].T)) @ w["o"].T
+
+
+MIXERS = {"latent_attention": latent_mixer, "attention": window_mixer, "wkv": wkv_mixer}
+
+
+# ---- feed-forward ------------------------------------------------------------------------------------------------------
+def table_experts(h, w, tokens):
+    """The token id alone picks the experts; each counts 1 / (how many a token has)."""
+    out = torch.zeros_like(h)
+    for t, tok in enumerate(tokens):
+        row = w["table"][tok].tolist()
+        for e in row:
+            e = int(e)
+            a = silu(w[f"e{e}.gate"] @ h[t]) * (w[f"e{e}.up"] @ h[t])
+            out[t] += (w[f"e{e}.down"] @ a) / len(row)
+    return out
+
+
+# ---- the stack -----------------------------------------------------------------------------------------------------------
+def run_list(n, loop):
+    """(layer, pass, is this the first layer of a pass?) in running order."""
+    if not loop:
+        return [(i, 0, False) for i in range(n)]
+    a, b = loop["start"], loop["stop"]
+    return [(i, 0, False) for i in range(a)] + \
+        [(i, t, i == a) for t in range(loop["times"]) for i in range(a, b)] + [(i, 0, False) for i in range(b, n)]
+
+
+def sub(weights, prefix):
+    return {n[len(prefix):]: t for n, t in weights.items() if n.startswith(prefix)}
+
+
+def forward(cfg, weights, tokens, dtype=torch.float32, want_layers=False):
+    """tokens: list of ids.  Logits [L, vocab]; with ``want_layers`` also the residual after every layer run."""
+    W = {n: t.to(dtype) if t.is_floating_point() else t for n, t in weights.items()}
+    eps = cfg["norm"]["eps"]
+    e = W["embed"][torch.tensor(tokens)]
+    x, trail = e, []
+    for i, t, first in run_list(len(cfg["layers"]), cfg.get("loop")):
+        spec = cfg["layers"][i]
+        if first:
+            x = torch.cat([x, e], -1) @ W["loop.in"].T + W["loop.step"][t]
+        x = x + MIXERS[spec["type"]](rms_norm(x, W[f"l{i}.norm1"], eps), sub(W, f"l{i}.mix."), spec["mixer"], eps)
+        if spec.get("mlp"):
+            x = x + table_experts(rms_norm(x, W[f"l{i}.norm2"], eps), sub(W, f"l{i}.mlp."), tokens)
+        trail.append(x)
+    y = rms_norm(x, W["final.norm"], eps) @ W["head"].T
+    return (y, torch.stack(trail)) if want_layers else y

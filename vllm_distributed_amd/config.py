@@ -179,6 +179,9 @@ def load_hf_config(model: str, overrides: Optional[dict] = None) -> HFConfig:
     if d.get("architecture") == "Surodra":         # a looped layer list of recurrent mixers, some beside attention
         from .models.surodra import normalise_config as surodra_config
         d = surodra_config(d, model if os.path.isdir(model) else None)
+    if d.get("architecture") == "Tilulorn":        # a looped layer list of latent, window and recurrent mixers
+        from .models.tilulorn import normalise_config as tilulorn_config
+        d = tilulorn_config(d, model if os.path.isdir(model) else None)
     if d.get("model_type") in ("exaone", "telechat", "qwen", "chatglm"):
         from .models.renamed_decoders import normalise_config
         d = normalise_config(d)
@@ -347,7 +350,7 @@ class ModelConfig:
                          "WhisperForConditionalGeneration", "BartForConditionalGeneration", "BartModel",
                          "MllamaForConditionalGeneration", "Zamba2ForCausalLM", "Plamo2ForCausalLM",
                          "Florence2ForConditionalGeneration", "NositarForCausalLM", "RapovikForCausalLM",
-                         "SevazenForCausalLM", "SurodraForCausalLM")
+                         "SevazenForCausalLM", "SurodraForCausalLM", "TilulornForCausalLM")
                    for a in self.architectures)
 
     @property

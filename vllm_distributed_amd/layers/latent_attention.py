@@ -7,10 +7,12 @@ plus a rotated key part that all heads share; only the latent and that part are 
     k_h = W_uk_h c,  v_h = W_uv_h c
     score(i, j, h) = scale * (q_plain . k_h + q_rot . k_rot),   j <= i and i - j < window,   softmax over j
                                    (``sink``: a learned number per head whose exponential joins the denominator)
-    out = W_o [sum_j p v_h]_h
+    out = W_o [sum_j p v_h]_h      (``gate`` "head": head h's part times sigmoid(W_g x)[h])
 
 The rotation turns the pairs (2i, 2i + 1), i < rot_dims / 2, of the P rotated values by position * base^(-2i / rot_dims)
-(angles, cosines and sines in fp32; values past rot_dims pass unchanged).  The key up-projection is folded into the
+(angles, cosines and sines in fp32; values past rot_dims pass unchanged); with ``rot_pairing`` "halves" the pairs are
+(i, i + rot_dims / 2), and ``rot_scaling`` rescales the frequencies (the kinds of ``rotary.half_split_cos_sin``).  Without
+``window`` every earlier key is visible.  The key up-projection is folded into the
 query (q_abs = W_uk_h^T q_plain, so the score is q_abs . c + q_rot . k_rot) and the value up-projection is applied
 after the attention, which then runs over the cached rows [c | k_rot] for all heads alike: the cache holds R + P
 values per token (``MLAAttention``; the MFMA kernel keeps a transposed copy of c beside them).  A mixer whose weights serve several passes of a looped
@@ -30,7 +32,8 @@ from ..forward_context import get_forward_context
 from ..parallel.state import get_tensor_model_parallel_world_size
 from .attention import MLAAttention
 from .hyper_connections import _fp32_param
-from .linear import MergedColumnParallelLinear, ReplicatedLinear, RowParallelLinear
+from .linear import MergedColumnParallelLinear, ReplicatedLinear, RowParallelLinear, row_padding, zero_tail_rows
+from .rotary import half_split_cos_sin
 
 _TABLES: dict = {}
 
@@ -53,7 +56,8 @@ def interleaved_cos_sin(max_len: int, dims: int, base: float, device) -> torch.T
 class WindowedLatentAttention(nn.Module):
     def __init__(self, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, v_head_dim: int, kv_rank: int,
                  scale: float, window: Optional[int], rot_base: Optional[float], rot_dims: int, eps: float,
-                 passes: int = 1, quant_config=None, prefix: str = "", q_rank: int = 0, sink: bool = False):
+                 passes: int = 1, quant_config=None, prefix: str = "", q_rank: int = 0, sink: bool = False,
+                 gate: Optional[str] = None, rot_pairing: str = "neighbours", rot_scaling: Optional[dict] = None):
         super().__init__()
         if get_tensor_model_parallel_world_size() > 1:
             raise NotImplementedError("windowed latent attention runs with tensor_parallel_size=1")
@@ -63,11 +67,21 @@ class WindowedLatentAttention(nn.Module):
         self.rot_dims = int(rot_dims) if rot_base else 0
         if self.rot_dims > P or self.rot_dims % 2:
             raise ValueError(f"{prefix}: {self.rot_dims} rotated dimensions do not fit an even part of {P}")
+        if rot_pairing not in ("halves", "neighbours"):
+            raise ValueError(f"{prefix}: rotation pairing {rot_pairing!r} ('halves' or 'neighbours')")
+        self.rot_pairing, self.rot_scaling = rot_pairing, rot_scaling
         self.q_rank = int(q_rank or 0)
+        if gate not in (None, "head") or (gate and not self.q_rank):
+            raise ValueError(f"{prefix}: gate {gate!r} (None, or 'head' beside a query latent)")
+        self.has_gate = gate is not None
         if self.q_rank:
-            # one GEMM for both down-projections: [query latent | key / value latent + rotated key part]
-            self.down_proj = MergedColumnParallelLinear(hidden_size, [self.q_rank, R + P], bias=False,
+            # one GEMM for both down-projections: [query latent | key / value latent + rotated key part], and the gate's
+            # rows behind them
+            sizes = [self.q_rank, R + P] + ([H] if self.has_gate else [])
+            pad = row_padding(sum(sizes)) if self.has_gate else 0
+            self.down_proj = MergedColumnParallelLinear(hidden_size, sizes + ([pad] if pad else []), bias=False,
                                                         quant_config=quant_config, prefix=f"{prefix}.down_proj")
+            zero_tail_rows(self.down_proj, pad)
             self.q_norm = _fp32_param((self.q_rank,))
             self.uq_proj = ReplicatedLinear(self.q_rank, H * (D + P), bias=False, quant_config=quant_config,
                                             prefix=f"{prefix}.uq_proj")
@@ -98,7 +112,11 @@ class WindowedLatentAttention(nn.Module):
 
     def _tables(self, device) -> torch.Tensor:
         if self._cos_sin is None or self._cos_sin.device != device:
-            self._cos_sin = interleaved_cos_sin(self.max_len, self.rot_dims, self.rot_base or 1.0, device)
+            if self.rot_pairing == "halves" or self.rot_scaling:
+                self._cos_sin = half_split_cos_sin(self.max_len, self.rot_dims, self.rot_base or 1.0, self.rot_scaling,
+                                                   device)
+            else:
+                self._cos_sin = interleaved_cos_sin(self.max_len, self.rot_dims, self.rot_base or 1.0, device)
         return self._cos_sin
 
     def _folded_weights(self):
@@ -118,7 +136,7 @@ class WindowedLatentAttention(nn.Module):
         if self.q_rank:
             both = self.down_proj(x)
             q = self.uq_proj(ops.group_rms_norm(both[:, : self.q_rank], self.q_norm, self.eps, 1))
-            down = both[:, self.q_rank:]
+            down = both[:, self.q_rank: self.q_rank + R + P]
         else:
             q = self.q_proj(x)
             down = self.dkv_proj(x)
@@ -136,7 +154,10 @@ class WindowedLatentAttention(nn.Module):
                 qf[n:, :, R:].zero_()
             ops.latent_norm_rope_cache(q[:n], down[:n], self.c_norm, self._tables(q.device), positions[:n], qf[:n],
                                        attn.k_cache, md.slot_mapping[:n], H, D, P, R, self.rot_dims, self.eps,
-                                       attn.v_cache if self.use_mfma else None)
+                                       attn.v_cache if self.use_mfma else None, self.rot_pairing)
             o_lat = attn.forward_cached(qf, self.sink)
         o = torch.bmm(o_lat.transpose(0, 1), w_uv_t).transpose(0, 1)
+        if self.has_gate:
+            g0 = self.q_rank + R + P
+            return self.o_proj(ops.head_gate_rows(o, both[:, g0: g0 + H]))
         return self.o_proj(o.reshape(T, H * Dv))

@@ -12,6 +12,7 @@ on the projections, several score maps per head, window / chunk masks, sinks and
     q       <- q * (1 + coef * ln(floor((p + 1) / every) + 1)) at position p (``q_temp`` = (coef, every))
     v       <- (1 - lam) v + lam v_first (``v_mix``): v_first are the values that the first such layer of the stack
                made of the same token; the layers of one forward pass hand them on through a dictionary
+    v        = the projected keys before norm and rotation instead (``key_values``: no value projection, Dv = D)
     score   = scale * q . k;  score <- cap * tanh(score / cap) (``softcap``);  score += rel[bucket(i - j), h]
                (``dist_bias`` = (rows, far): distances below rows / 2 have a row each, the others share the rest in
                logarithmic steps up to ``far``)
@@ -108,7 +109,7 @@ class MaskedSoftmaxAttention(nn.Module):
                  rot_base: float = 10000.0, rot_scaling: Optional[dict] = None, users: int = 1, quant_config=None,
                  prefix: str = "", rot_pairing: str = "halves", q_temp: Optional[tuple] = None, softcap: float = 0.0,
                  dist_bias: Optional[tuple] = None, sink_fixed: Optional[float] = None, v_mix: bool = False,
-                 norm_over: str = "head"):
+                 norm_over: str = "head", key_values: bool = False):
         super().__init__()
         if get_tensor_model_parallel_world_size() > 1:
             raise NotImplementedError("this attention layer runs with tensor_parallel_size=1")
@@ -124,8 +125,11 @@ class MaskedSoftmaxAttention(nn.Module):
         self.window, self.chunk, self.maps, self.diff = int(window or 0), int(chunk or 0), int(maps), float(diff)
         self.taps = int(conv_taps or 0)
         self.rot_dims, self.rot_base, self.rot_scaling = int(rot_dims), float(rot_base), rot_scaling
-        if rot_pairing not in ("halves", "neighbours") or (rot_pairing == "neighbours" and rot_scaling):
-            raise ValueError(f"{prefix}: rotation pairing {rot_pairing!r} (with frequency scaling: halves only)")
+        if rot_pairing not in ("halves", "neighbours"):
+            raise ValueError(f"{prefix}: rotation pairing {rot_pairing!r} ('halves' or 'neighbours')")
+        self.key_values = bool(key_values)
+        if self.key_values and (D != Dv or maps != 1 or conv_taps or v_mix):
+            raise ValueError(f"{prefix}: keys as values need one width ({D}, {Dv}), one map, no convolution, no mixing")
         if sink and sink_fixed is not None:
             raise ValueError(f"{prefix}: a learned sink and a fixed one exclude each other")
         self.rot_pairing = rot_pairing
@@ -134,14 +138,14 @@ class MaskedSoftmaxAttention(nn.Module):
             raise ValueError(f"{prefix}: the query temperature grows every {self.q_temp[1]} positions")
         self.softcap = float(softcap or 0.0)
         self.layer_name = prefix
-        nq, nk, nv = H * maps * D, G * maps * D, G * Dv
+        nq, nk, nv = H * maps * D, G * maps * D, 0 if self.key_values else G * Dv
         self.qkv_width = nq + nk + nv
         if gate not in (False, True, "head"):
             raise ValueError(f"{prefix}: gate {gate!r} (False, True or 'head')")
         self.gate_width = (H if gate == "head" else H * Dv) if gate else 0
         pad = row_padding(self.qkv_width + self.gate_width) if gate == "head" else 0
-        sizes = [nq, nk, nv] + ([self.gate_width] if gate else []) + ([pad] if pad else [])
-        # one GEMM for everything that reads x: q | k | v (| gate); the gate's part of the bias stays zero
+        sizes = [nq, nk] + ([nv] if nv else []) + ([self.gate_width] if gate else []) + ([pad] if pad else [])
+        # one GEMM for everything that reads x: q | k (| v) (| gate); the gate's part of the bias stays zero
         self.in_proj = MergedColumnParallelLinear(hidden_size, sizes, bias=bias, quant_config=quant_config,
                                                   prefix=f"{prefix}.in_proj")
         zero_tail_rows(self.in_proj, pad)
@@ -200,7 +204,7 @@ class MaskedSoftmaxAttention(nn.Module):
         if self.rot_dims == 0:
             return None
         if self._cos_sin is None or self._cos_sin.device != device:
-            if self.rot_pairing == "neighbours":
+            if self.rot_pairing == "neighbours" and not self.rot_scaling:
                 from .latent_attention import interleaved_cos_sin
                 self._cos_sin = interleaved_cos_sin(self.max_len, self.rot_dims, self.rot_base, device)
             else:
@@ -256,7 +260,8 @@ class MaskedSoftmaxAttention(nn.Module):
         elif self.taps == 1:
             qkv = (p[:n, :W].float() * self.conv_weight.float().view(1, -1)).to(p.dtype)
         g_rows = gate[:n] if gate is not None else None
-        extras = dict(pairing=self.rot_pairing, q_temp=self.q_temp, whole_norm=self.whole_norm)
+        extras = dict(pairing=self.rot_pairing, q_temp=self.q_temp, whole_norm=self.whole_norm,
+                      key_values=self.key_values)
         if self.vmix is not None:
             if lent is None:
                 raise ValueError(f"{self.layer_name}: value mixing needs the forward pass's dictionary")

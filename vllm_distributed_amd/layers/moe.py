@@ -85,6 +85,47 @@ def grouped_topk_with_identity(logits: torch.Tensor, bias: Optional[torch.Tensor
     return w, ids, idw
 
 
+class TokenExpertTables(nn.Module):
+    """Routing without a router: per routed layer a table [vocab, top] gives every token id its experts (int32).  The tables of
+    a stack lie in one tensor, so that one lookup per forward pass serves all of its layers; a token's experts count
+    1 / top each."""
+
+    def __init__(self, vocab: int, tops: list, num_experts: list):
+        super().__init__()
+        self.tops, self.num_experts = [int(t) for t in tops], [int(e) for e in num_experts]
+        for t, e in zip(self.tops, self.num_experts):
+            if not 1 <= t <= e:
+                raise ValueError(f"{t} experts per token out of {e}")
+        widest = max(self.tops)
+        # until a checkpoint fills them: neighbouring token ids and places take neighbouring experts
+        first = torch.arange(vocab, dtype=torch.int32)[:, None] + torch.arange(widest, dtype=torch.int32)
+        self.table = nn.Parameter(torch.stack([first % e for e in self.num_experts]), requires_grad=False)
+        set_weight_attrs(self.table, {"weight_loader": self._load})
+        rows = int(get_current_vllm_config().scheduler_config.max_num_batched_tokens) + 64
+        for t in sorted(set(self.tops)):
+            self.register_buffer(f"share_{t}", torch.full((rows, t), 1.0 / t, dtype=torch.float32), persistent=False)
+
+    def _load(self, param: nn.Parameter, t: torch.Tensor, index: int) -> None:
+        E = self.num_experts[index]
+        if t.is_floating_point() or t.shape != (param.shape[1], self.tops[index]):
+            raise ValueError(f"expert table {index}: {t.dtype} {tuple(t.shape)}, expected integers "
+                             f"{(param.shape[1], self.tops[index])}")
+        if t.numel() and (int(t.min()) < 0 or int(t.max()) >= E):
+            raise ValueError(f"expert table {index} names experts outside 0 .. {E - 1}")
+        param.data[index, :, : t.shape[1]].copy_(t)
+
+    def forward(self, input_ids: torch.Tensor) -> list:
+        """Per routed layer (weights fp32 [T, top], ids int32 [T, top])."""
+        T = input_ids.shape[0]
+        ids = torch.index_select(self.table, 1, input_ids)
+        out = []
+        for i, t in enumerate(self.tops):
+            share = getattr(self, f"share_{t}")
+            w = share[:T] if T <= share.shape[0] else torch.full((T, t), 1.0 / t, dtype=torch.float32, device=ids.device)
+            out.append((w, ids[i, :, :t].contiguous()))
+        return out
+
+
 class UnquantizedMoEMethod:
     def create_weights(self, layer: "FusedMoE", E: int, H: int, I: int, dtype: torch.dtype) -> None:
         w13 = nn.Parameter(torch.empty(E, (2 if getattr(layer, "gated", True) else 1) * I, H, dtype=dtype),

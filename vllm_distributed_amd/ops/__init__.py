@@ -681,6 +681,18 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None
     return torch.nn.functional.linear(x, w, bias)
 
 
+def grouped_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """y[g] = x[g] @ w[g].T for x [G, M, K], w [G, N, K]: products of one size over inputs of their own."""
+    return torch.stack([linear(x[g], w[g]) for g in range(x.shape[0])])
+
+
+def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x @ w.T with fp32 sums that stay fp32 (16-bit operands of a product that becomes the fp32 residual)."""
+    if x.is_cuda and x.dtype != torch.float32:
+        return torch.mm(x, w.t(), out_dtype=torch.float32)
+    return torch.nn.functional.linear(x.float(), w.float())
+
+
 def gate_up_silu_mul(x: torch.Tensor, w: torch.Tensor) -> Optional[torch.Tensor]:
     """silu(x @ gate.T) * (x @ up.T) for w = [gate rows; up rows] in ONE kernel (the activation runs in the GEMM
     epilogue, the [M, 2 I] intermediate never exists), or None when this batch does not take the in-tree GEMM."""
@@ -1596,22 +1608,27 @@ def linear_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: to
                      max_query_len: int, *, log_decay: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None,
                      z_bias: Optional[torch.Tensor] = None, tau: float = 1.0, cos_sin: Optional[torch.Tensor] = None,
                      positions: Optional[torch.Tensor] = None, rot: int = 0, q_scale: float = 1.0,
-                     k_scale: float = 1.0, first_long_seq: int = 0) -> torch.Tensor:
+                     k_scale: float = 1.0, first_long_seq: int = 0, decay_exp: bool = False,
+                     bonus: Optional[torch.Tensor] = None) -> torch.Tensor:
     """S <- diag(decay) S + k v^T, o = S^T q per head over a ragged batch, then o / rms(o) * norm_w * silu(gate) (see
     ops/csrc/linear_attention.hip).  q, k [T, H*D], v, gate [T, H*Dv] in the activation type (row strides arbitrary);
     the first ``rot`` values of every q / k head are rotated (halves; cos_sin fp32 [positions, rot]), q times q_scale, k
     times k_scale, all in fp32.  Decay: exp(log_decay[h]) (fp32 [H]) or sigmoid(z + z_bias)^(1 / tau) per key channel
-    (z [T, H*D], z_bias fp32 [H*D] or None).  norm_w fp32 [Dv] or None.  state fp32 [slots, H, Dv, D] (transposed),
+    (z [T, H*D], z_bias fp32 [H*D] or None), or exp(-exp(z + z_bias)) with ``decay_exp``.  ``bonus`` fp32 [H*D] (with z):
+    the memory is read before the token is written, o = (S + diag(bonus) k v^T)^T q.  norm_w fp32 [Dv] (one row for all
+    heads), [H*Dv] or None.  state fp32 [slots, H, Dv, D] (transposed),
     updated in place; sequence s uses slot ``slot_table[s, 0]`` and starts from zero when all its tokens are in this
     batch.  ``first_long_seq``: sequences before it bring at most ``RECURRENT_STEP_TOKENS`` tokens each."""
     if not _dev(q) or D > 1024:
         return R.linear_attention(q, k, v, gate, norm_w, state, query_start_loc, seq_lens, slot_table, H, D, Dv, eps,
-                                  log_decay, z, z_bias, tau, cos_sin, positions, rot, q_scale, k_scale)
+                                  log_decay, z, z_bias, tau, cos_sin, positions, rot, q_scale, k_scale, decay_exp, bonus)
     T, S = q.shape[0], seq_lens.shape[0]
+    assert bonus is None or z is not None
+    norm_head = Dv if norm_w is not None and norm_w.numel() == H * Dv and H > 1 else 0
     assert (log_decay is None) != (z is None)
     for t, n in ((q, H * D), (k, H * D), (v, H * Dv), (gate, H * Dv), (z, H * D)):
         assert t is None or (t.stride(1) == 1 and t.dtype == q.dtype and t.shape == (T, n))
-    for t, n in ((norm_w, Dv), (log_decay, H), (z_bias, H * D)):
+    for t, n in ((norm_w, H * Dv if norm_head else Dv), (log_decay, H), (z_bias, H * D), (bonus, H * D)):
         assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n)
     assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, Dv, D)
     assert rot == 0 or (cos_sin.dtype == torch.float32 and cos_sin.is_contiguous() and cos_sin.shape[1] == rot
@@ -1629,10 +1646,29 @@ def linear_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: to
                               dtype=torch.float32, device=q.device)
     N.call("vda_linear_attention", out.data_ptr(), out.stride(0), N.ptr(o_raw), N.ptr(scratch), q.data_ptr(), q.stride(0),
            k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), N.ptr(z), z.stride(0) if z is not None else 0,
-           N.ptr(z_bias), 1.0 / float(tau), N.ptr(log_decay), gate.data_ptr(), gate.stride(0), N.ptr(cos_sin),
-           N.ptr(positions), int(rot), float(q_scale), float(k_scale), N.ptr(norm_w), float(eps), state.data_ptr(),
+           N.ptr(z_bias), 1.0 / float(tau), int(decay_exp), N.ptr(bonus), N.ptr(log_decay), gate.data_ptr(), gate.stride(0), N.ptr(cos_sin),
+           N.ptr(positions), int(rot), float(q_scale), float(k_scale), N.ptr(norm_w), norm_head, float(eps), state.data_ptr(),
            query_start_loc.data_ptr(), seq_lens.data_ptr(), slot_table.data_ptr(), slot_table.stride(0), T, S,
            int(first_long_seq), H, D, Dv, max(int(max_query_len), 1), C, N.dt(q.dtype), N.stream())
+    return out
+
+
+def token_shift_mix(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, query_start_loc: torch.Tensor,
+                    seq_lens: torch.Tensor, slot_table: torch.Tensor, max_query_len: int) -> torch.Tensor:
+    """h [T, W] (row stride arbitrary), mu fp32 [M, W], state [slots, W] in h's type.  Returns [M, T, W]: row m of a token is
+    h + (h' - h) * mu[m] with h' the row of the token before it in its sequence: the row above, for the first new token
+    of a sequence the one in its slot ``slot_table[s, 0]``, zeros when the sequence starts here.  The last new row of
+    every sequence replaces the slot's."""
+    T, W = h.shape
+    M, S = mu.shape[0], seq_lens.shape[0]
+    if not _dev(h):
+        return R.token_shift_mix(h, mu, state, query_start_loc, seq_lens, slot_table)
+    assert h.stride(1) == 1 and mu.dtype == torch.float32 and mu.is_contiguous() and mu.shape == (M, W) and 1 <= M <= 8
+    assert state.dtype == h.dtype and state.is_contiguous() and state.shape[-1] == W and state.numel() % W == 0
+    out = torch.empty((M, T, W), dtype=h.dtype, device=h.device)
+    N.call("vda_token_shift_mix", out.data_ptr(), out.stride(0), h.data_ptr(), h.stride(0), mu.data_ptr(), state.data_ptr(),
+           query_start_loc.data_ptr(), seq_lens.data_ptr(), slot_table.data_ptr(), slot_table.stride(0), T, S, M, W,
+           max(int(max_query_len), 1), N.dt(h.dtype), N.stream())
     return out
 
 
@@ -1700,17 +1736,22 @@ def residual_norms(x: torch.Tensor, y: Optional[torch.Tensor] = None, w_post: Op
 
 # ---- fp32 residual with parallel gated sub-layers and a norm in groups ------------------------------------------
 def gated_residual_group_norm(x: torch.Tensor, subs: list, w_next: Optional[torch.Tensor], groups: int, eps: float,
-                              out_dtype: torch.dtype) -> Optional[torch.Tensor]:
+                              out_dtype: torch.dtype, step: Optional[torch.Tensor] = None,
+                              cast_to: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """One pass over the fp32 residual ``x`` [T, W]: x += sum over ``subs`` of (y + extra_w[:, None] * extra) * scale *
     sigmoid(gate), in place -- one tuple (y, scale, gate, extra, extra_w) per sub-layer (at most three; y [T, W] in the
     activation type, scale fp32 [W] or None, gate [T, W] pre-activations or None, extra [T, W] with extra_w fp32 [T] or
     None) -- and, with ``w_next`` (fp32 [W]), returns the updated row normalised in ``groups`` equal consecutive parts,
-    each divided by its own root mean square, times w_next, in ``out_dtype``."""
+    each divided by its own root mean square, times w_next, in ``out_dtype``.  ``step`` (fp32 [W]) joins every row of x
+    behind the sub-layers.  Without ``w_next``, ``cast_to`` ([T, W], unit column stride) receives the updated rows."""
     T, W = x.shape
     if not _dev(x) or (W + groups) * 4 > 60 * 1024 or len(subs) > 3:
-        return R.gated_residual_group_norm(x, subs, w_next, groups, eps, out_dtype)
+        return R.gated_residual_group_norm(x, subs, w_next, groups, eps, out_dtype, step, cast_to)
     assert x.dtype == torch.float32 and x.is_contiguous() and W % groups == 0
-    h = torch.empty((T, W), dtype=out_dtype, device=x.device) if w_next is not None else None
+    assert step is None or (step.dtype == torch.float32 and step.is_contiguous() and step.numel() == W)
+    assert cast_to is None or (w_next is None and cast_to.shape == (T, W) and cast_to.stride(1) == 1
+                               and cast_to.dtype == out_dtype)
+    h = torch.empty((T, W), dtype=out_dtype, device=x.device) if w_next is not None else cast_to
     assert w_next is None or (w_next.dtype == torch.float32 and w_next.is_contiguous())
     args = []
     dt = out_dtype
@@ -1725,7 +1766,7 @@ def gated_residual_group_norm(x: torch.Tensor, subs: list, w_next: Optional[torc
                  N.ptr(extra), extra.stride(0) if extra is not None else 0, N.ptr(extra_w)]
     args += [None, 0, None, None, 0, None, 0, None] * (3 - len(subs))
     assert h is None or not subs or h.dtype == dt
-    N.call("vda_gated_residual_group_norm", x.data_ptr(), len(subs), *args, N.ptr(w_next), N.ptr(h),
+    N.call("vda_gated_residual_group_norm", x.data_ptr(), len(subs), *args, N.ptr(step), N.ptr(w_next), N.ptr(h),
            h.stride(0) if h is not None else 0, float(eps), int(groups), T, W, N.dt(dt), N.stream())
     return h
 
@@ -1734,15 +1775,17 @@ def gated_residual_group_norm(x: torch.Tensor, subs: list, w_next: Optional[torc
 def latent_norm_rope_cache(q: torch.Tensor, down: torch.Tensor, c_weight: torch.Tensor, cos_sin: torch.Tensor,
                            positions: torch.Tensor, qf: torch.Tensor, kc: Optional[torch.Tensor],
                            slot_mapping: torch.Tensor, H: int, D: int, P: int, rank: int, rot_dims: int,
-                           eps: float, vt: Optional[torch.Tensor] = None) -> None:
+                           eps: float, vt: Optional[torch.Tensor] = None, pairing: str = "neighbours") -> None:
     """Per token: the cache row [down[:rank] / rms * c_weight | down[rank:] with its first ``rot_dims`` values rotated] goes
     to ``kc`` [blocks, bs, rank + P] at ``slot_mapping``; the last P values of every query head (q [T, H * (D + P)]),
     rotated alike, go to qf[:, h, rank:] (qf [T, H, rank + P]).  Pairs (2i, 2i + 1) turn by the angle whose cosine and sine
-    are cos_sin[position, i] and cos_sin[position, rot_dims / 2 + i] (fp32).  ``vt`` [blocks, rank, bs]: a transposed
+    are cos_sin[position, i] and cos_sin[position, rot_dims / 2 + i] (fp32); with ``pairing`` "halves" the pairs are
+    (i, i + rot_dims / 2).  ``vt`` [blocks, rank, bs]: a transposed
     copy of the rows' first ``rank`` values, for the kernel that wants one."""
     if not _dev(q):
         return R.latent_norm_rope_cache(q, down, c_weight, cos_sin, positions, qf, kc, slot_mapping, H, D, P, rank,
-                                        rot_dims, eps, vt)
+                                        rot_dims, eps, vt, pairing)
+    assert pairing in ("neighbours", "halves")
     T = q.shape[0]
     assert q.stride(1) == 1 and down.stride(1) == 1 and qf.is_contiguous() and kc.is_contiguous()
     assert q.dtype == down.dtype == qf.dtype == kc.dtype and kc.shape[2] == rank + P and qf.shape == (T, H, rank + P)
@@ -1750,7 +1793,22 @@ def latent_norm_rope_cache(q: torch.Tensor, down: torch.Tensor, c_weight: torch.
     assert positions.dtype == torch.int64 and slot_mapping.dtype == torch.int64 and c_weight.dtype == torch.float32
     N.call("vda_latent_norm_rope_cache", q.data_ptr(), q.stride(0), down.data_ptr(), down.stride(0),
            c_weight.data_ptr(), cos_sin.data_ptr(), positions.data_ptr(), qf.data_ptr(), kc.data_ptr(),
-           vt.data_ptr() if vt is not None and vt.numel() else None, slot_mapping.data_ptr(), T, H, D, P, rank, rot_dims, kc.shape[1], float(eps), N.dt(q.dtype), N.stream())
+           vt.data_ptr() if vt is not None and vt.numel() else None, slot_mapping.data_ptr(), T, H, D, P, rank,
+           rot_dims, kc.shape[1], float(eps), int(pairing == "halves"), N.dt(q.dtype), N.stream())
+
+
+def head_gate_rows(a: torch.Tensor, gate: Optional[torch.Tensor]) -> torch.Tensor:
+    """a [T, H, Dv] (any token and head strides, unit value stride), gate [T, H] pre-activations (row stride arbitrary) or
+    None -> [T, H * Dv] = a * sigmoid(gate[t, h]), contiguous."""
+    T, H, Dv = a.shape
+    if not _dev(a):
+        o = a.float() * torch.sigmoid(gate.float()).unsqueeze(-1) if gate is not None else a
+        return o.to(a.dtype).reshape(T, H * Dv)
+    assert a.stride(2) == 1 and (gate is None or (gate.shape == (T, H) and gate.stride(1) == 1 and gate.dtype == a.dtype))
+    out = torch.empty((T, H * Dv), dtype=a.dtype, device=a.device)
+    N.call("vda_head_gate_rows", out.data_ptr(), a.data_ptr(), a.stride(0), a.stride(1), N.ptr(gate),
+           gate.stride(0) if gate is not None else 0, T, H, Dv, N.dt(a.dtype), N.stream())
+    return out
 
 
 def latent_window_attention(q: torch.Tensor, kc: torch.Tensor, block_table: torch.Tensor, seq_lens: torch.Tensor,
@@ -1849,7 +1907,8 @@ def qk_norm_rope_cache(qkv: torch.Tensor, H: int, G: int, D: int, Dv: int, maps:
                        eps: float, k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor],
                        slot_mapping: torch.Tensor, by_map: bool = False, pairing: str = "halves",
                        q_temp: Optional[tuple] = None, v_first: Optional[torch.Tensor] = None,
-                       v_lam: Optional[torch.Tensor] = None, whole_norm: bool = False) -> torch.Tensor:
+                       v_lam: Optional[torch.Tensor] = None, whole_norm: bool = False,
+                       key_values: bool = False) -> torch.Tensor:
     """qkv [T, >= H*maps*D + G*maps*D + G*Dv] (queries, keys, values side by side; further columns are ignored).  Every
     D-wide map of every query / key head is divided by its root mean square, multiplied by q_weight / k_weight (fp32
     [D]), and its first ``rot`` values are rotated in the half-split layout (value i pairs with i + rot / 2; cos_sin fp32
@@ -1862,12 +1921,15 @@ def qk_norm_rope_cache(qkv: torch.Tensor, H: int, G: int, D: int, Dv: int, maps:
     the queries at position p are multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  ``v_first`` [T, G * Dv] (row
     stride arbitrary) with ``v_lam`` (fp32, one element): the cached values are (1 - lam) v + lam v_first.
     ``whole_norm``: all query values of a token are divided by ONE root mean square (and all key values by one), the
-    weights have a value of their own per projection row (q_weight fp32 [H*maps*D], k_weight fp32 [G*maps*D])."""
-    used = (H + G) * maps * D + G * Dv
+    weights have a value of their own per projection row (q_weight fp32 [H*maps*D], k_weight fp32 [G*maps*D]).
+    ``key_values``: the values are the projected keys before norm and rotation (maps 1, Dv = D; no value columns)."""
+    assert not key_values or (maps == 1 and D == Dv)
+    used = (H + G) * maps * D + (0 if key_values else G * Dv)
     if not _dev(qkv):
         assert not by_map
         return R.qk_norm_rope_cache(qkv[:, :used], H, G, D, Dv, maps, q_weight, k_weight, cos_sin, positions, rot, eps,
-                                    k_cache, v_cache, slot_mapping, pairing, q_temp, v_first, v_lam, whole_norm)
+                                    k_cache, v_cache, slot_mapping, pairing, q_temp, v_first, v_lam, whole_norm,
+                                    key_values)
     assert q_weight.numel() == (H * maps * D if whole_norm else D)
     assert k_weight.numel() == (G * maps * D if whole_norm else D)
     assert pairing in ("halves", "neighbours")
@@ -1888,7 +1950,7 @@ def qk_norm_rope_cache(qkv: torch.Tensor, H: int, G: int, D: int, Dv: int, maps:
            slot_mapping.data_ptr(), T, H, G, D, Dv, maps, rot, bs, float(eps), int(by_map),
            int(pairing == "neighbours"), float(q_temp[0]) if q_temp else 0.0, int(q_temp[1]) if q_temp else 0,
            N.ptr(v_first), v_first.stride(0) if v_first is not None else 0, N.ptr(v_lam), int(whole_norm),
-           N.dt(qkv.dtype), N.stream())
+           int(key_values), N.dt(qkv.dtype), N.stream())
     return qn
 
 

@@ -4,7 +4,7 @@
 
 enum Act { ACT_SILU = 0, ACT_GELU = 1, ACT_GELU_TANH = 2, ACT_RELU = 3, ACT_GELU_NEW = 4,
            ACT_GELU_FAST = 5, ACT_GELU_QUICK = 6, ACT_FATRELU = 7, ACT_RELU2 = 8,
-           ACT_CLAMPED_SWIGLU = 9 /* gated pairs only: see gated_pair, the threshold is its clamp */ };
+           ACT_CLAMPED_SWIGLU = 9 /* gated pairs only: see gated_pair, the threshold is its clamp */, ACT_TANH = 10 };
 
 template <int A> __device__ __forceinline__ float act(float x, float thr) {
   if (A == ACT_SILU) return x / (1.f + __expf(-x));
@@ -18,6 +18,7 @@ template <int A> __device__ __forceinline__ float act(float x, float thr) {
   if (A == ACT_GELU_QUICK) return x / (1.f + __expf(-1.702f * x));
   if (A == ACT_FATRELU) return x > thr ? x : 0.f;
   if (A == ACT_RELU2) { const float r = fmaxf(x, 0.f); return r * r; }
+  if (A == ACT_TANH) return tanhf(x);
   return x;
 }
 
@@ -128,6 +129,7 @@ static int launch_plain(void* out, const void* in, long n, int a, float thr, hip
     case ACT_GELU_FAST: L(ACT_GELU_FAST); break;
     case ACT_GELU_QUICK: L(ACT_GELU_QUICK); break;
     case ACT_RELU2: L(ACT_RELU2); break;
+    case ACT_TANH: L(ACT_TANH); break;
     default: return -2;
   }
 #undef L

@@ -730,7 +730,7 @@ VDA_EXPORT int vda_gated_delta_rule_head(void* out, long o_stride, float* o_raw,
   VDA_CHECK_LAUNCH();
   const dim3 ge((unsigned)(((long)max_q * H + 3) / 4), S - seq0);
 #define EP(TT) hipLaunchKernelGGL((head_norm_silu_kernel<TT>), ge, dim3(256), 0, st, (TT*)out, o_stride, o_raw,        \
-                                  (const TT*)gate, g_stride, norm_w, qsl, seq_lens, seq0, a.limit, H, Dv, eps)
+                                  (const TT*)gate, g_stride, norm_w, 0, qsl, seq_lens, seq0, a.limit, H, Dv, eps)
   if (dtype == VDA_BF16) EP(bf16_t);
   else if (dtype == VDA_F16) EP(f16_t);
   else EP(float);

@@ -6,9 +6,11 @@
 // latent space (sum of weights * c) for the caller's value up-projection.
 //
 //   vda_latent_norm_rope_cache   per token: c = down[:R] / rms * weight, rotate down[R:] and every query head's last
-//                                P values (interleaved pairs, angles from an fp32 cos | sin table), write the cache
-//                                row (and, for the MFMA kernel of mla.hip, the transposed copy of c) and
+//                                P values (interleaved or half-split pairs, angles from an fp32 cos | sin table), write
+//                                the cache row (and, for the MFMA kernel of mla.hip, the transposed copy of c) and
 //                                qf[:, :, R:] in one launch
+//   vda_head_gate_rows           out[t, h, :] = a[h, t, :] * sigmoid(gate[t, h]): the heads' outputs, in the order the value
+//                                up-projection leaves them, gated and laid out token by token
 //   vda_latent_window_attention  softmax(scale * qf . row) over the keys j <= i, i - j < window (with `sink`, exp(sink[h])
 //                                joins head h's denominator without key or value); scores, softmax and
 //                                the weighted sum in fp32.  One workgroup per (sequence, tile of query tokens) walks
@@ -22,13 +24,21 @@ __global__ __launch_bounds__(256) void latent_norm_rope_cache_kernel(
     const T* __restrict__ q, long q_stride, const T* __restrict__ down, long down_stride,
     const float* __restrict__ c_weight, const float* __restrict__ cos_sin, const long* __restrict__ positions,
     T* __restrict__ qf, T* __restrict__ kc, T* __restrict__ vt, const long* __restrict__ slot_mapping, int H, int D,
-    int P, int R, int rot, int bs, float eps) {
+    int P, int R, int rot, int bs, float eps, int halves) {
   __shared__ float red[16];
   const long t = blockIdx.x;
   const int tid = threadIdx.x;
   const int DK = R + P, half = rot / 2;
   const T* dr = down + t * down_stride;
   const float* cs = cos_sin + positions[t] * (long)rot;
+  // value i < rot of a rotated part: pairs (2i, 2i + 1), or (i, i + rot / 2) with `halves`
+  auto turned = [&](const T* p, int i) {
+    const bool first = halves ? i < half : !(i & 1);
+    const int pr = halves ? (first ? i : i - half) : i >> 1;
+    const float co = cs[pr], si = cs[half + pr];
+    const float own = (float)p[i], other = (float)p[halves ? (first ? i + half : i - half) : i ^ 1];
+    return first ? own * co - other * si : own * co + other * si;
+  };
   float ss = 0.f;
   for (int c = tid; c < R; c += 256) {
     const float v = (float)dr[c];
@@ -46,49 +56,70 @@ __global__ __launch_bounds__(256) void latent_norm_rope_cache_kernel(
       if (col) col[(long)c * bs] = v;
     }
     for (int i = tid; i < P; i += 256) {
-      float v;
-      if (i < rot) {
-        const int pr = i >> 1;
-        const float co = cs[pr], si = cs[half + pr];
-        const float u = (float)dr[R + (i & ~1)], w = (float)dr[R + (i | 1)];
-        v = (i & 1) ? w * co + u * si : u * co - w * si;
-      } else {
-        v = (float)dr[R + i];
-      }
-      row[R + i] = (T)v;
+      row[R + i] = (T)(i < rot ? turned(dr + R, i) : (float)dr[R + i]);
     }
   }
   // the query heads' rotated parts
   for (int e = tid; e < H * P; e += 256) {
     const int h = e / P, i = e % P;
     const T* qp = q + t * q_stride + (long)h * (D + P) + D;
-    float v;
-    if (i < rot) {
-      const int pr = i >> 1;
-      const float co = cs[pr], si = cs[half + pr];
-      const float u = (float)qp[i & ~1], w = (float)qp[i | 1];
-      v = (i & 1) ? w * co + u * si : u * co - w * si;
-    } else {
-      v = (float)qp[i];
-    }
-    qf[(t * H + h) * DK + R + i] = (T)v;
+    qf[(t * H + h) * DK + R + i] = (T)(i < rot ? turned(qp, i) : (float)qp[i]);
   }
 }
 
 VDA_EXPORT int vda_latent_norm_rope_cache(const void* q, long q_stride, const void* down, long down_stride,
                                           const float* c_weight, const float* cos_sin, const long* positions,
                                           void* qf, void* kc, void* vt, const long* slot_mapping, int T, int H, int D,
-                                          int P, int R, int rot, int bs, float eps, int dtype, hipStream_t st) {
+                                          int P, int R, int rot, int bs, float eps, int halves, int dtype,
+                                          hipStream_t st) {
   if (T <= 0) return 0;
   if (rot < 0 || rot > P || (rot & 1)) return -1;
 #define L(TT) hipLaunchKernelGGL((latent_norm_rope_cache_kernel<TT>), dim3(T), dim3(256), 0, st, (const TT*)q,      \
                                  q_stride, (const TT*)down, down_stride, c_weight, cos_sin, positions, (TT*)qf,      \
-                                 (TT*)kc, (TT*)vt, slot_mapping, H, D, P, R, rot, bs, eps)
+                                 (TT*)kc, (TT*)vt, slot_mapping, H, D, P, R, rot, bs, eps, halves)
   if (dtype == VDA_BF16) L(bf16_t);
   else if (dtype == VDA_F16) L(f16_t);
   else if (dtype == VDA_F32) L(float);
   else return -3;
 #undef L
+  VDA_CHECK_LAUNCH();
+  return 0;
+}
+
+// one value per thread and step; V consecutive values of a head at a time
+template <typename T, int V>
+__global__ __launch_bounds__(256) void head_gate_rows_kernel(T* __restrict__ out, const T* __restrict__ a, long a_t,
+                                                             long a_h, const T* __restrict__ gate, long gate_stride,
+                                                             long n, int H, int per) {
+  using VV = T __attribute__((ext_vector_type(V)));
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;          // per = Dv / V vectors of a head
+  if (i >= n) return;
+  const long row = i / per, t = row / H;
+  const int h = (int)(row - t * H), c = (int)(i - row * per) * V;
+  const float g = gate ? 1.f / (1.f + expf(-(float)gate[t * gate_stride + h])) : 1.f;
+  const VV v = *reinterpret_cast<const VV*>(a + t * a_t + h * a_h + c);
+  VV o;
+#pragma unroll
+  for (int j = 0; j < V; ++j) o[j] = (T)((float)v[j] * g);
+  *reinterpret_cast<VV*>(out + i * V) = o;
+}
+
+VDA_EXPORT int vda_head_gate_rows(void* out, const void* a, long a_t, long a_h, const void* gate, long gate_stride, int T,
+                                  int H, int Dv, int dtype, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (H < 1 || Dv < 1) return -1;
+  const int V = Dv % 8 == 0 && a_t % 8 == 0 && a_h % 8 == 0 && (uintptr_t)a % 32 == 0 && (uintptr_t)out % 32 == 0 ? 8 : 1;
+  const long n = (long)T * H * (Dv / V);
+  const dim3 grid((unsigned)((n + 255) / 256));
+#define L2(TT, VV) hipLaunchKernelGGL((head_gate_rows_kernel<TT, VV>), grid, dim3(256), 0, st, (TT*)out, (const TT*)a, a_t,  \
+                                      a_h, (const TT*)gate, gate_stride, n, H, Dv / VV)
+#define L(TT) do { if (V == 8) L2(TT, 8); else L2(TT, 1); } while (0)
+  if (dtype == VDA_BF16) L(bf16_t);
+  else if (dtype == VDA_F16) L(f16_t);
+  else if (dtype == VDA_F32) L(float);
+  else return -3;
+#undef L
+#undef L2
   VDA_CHECK_LAUNCH();
   return 0;
 }

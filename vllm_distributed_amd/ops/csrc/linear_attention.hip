@@ -1,10 +1,13 @@
 // Linear attention with decay over a ragged batch with per-request fp32 state.  Per token and head
 //     S <- diag(decay) S + k v^T,   o = S^T q                       (S: [D, Dv], stored transposed, [Dv, D])
 //     out = o / rms(o) * norm_w * silu(gate)                        (norm_w optional)
+// or, with a bonus u per head and key channel (the RWKV form: the own token enters the read-out through the bonus, not the
+// memory),   o = (S + diag(u) k v^T)^T q,   S <- diag(decay) S + k v^T,
 // with q and k scaled and, on the first `rot` values of a head, rotated (value i paired with i + rot / 2, fp32 angles from
 // a table) before they enter, and a decay that is either
 //     one number per head (retention):              decay[h], given as its logarithm, or
-//     one number per token, head and key channel:   sigmoid(z + bias)^(1 / tau) (gated linear attention).
+//     one number per token, head and key channel:   sigmoid(z + bias)^(1 / tau) (gated linear attention), or
+//                                                   exp(-exp(z + bias)) (`decay_exp`).
 // The batch description is the one of the other recurrent kernels (qsl, seq_lens, slot in column 0 of the table; a
 // sequence carries state in when seq_len - new_tokens > 0).
 //
@@ -17,6 +20,7 @@
 //   carry                per (sequence, head): the state at every chunk's start, one after the other (elementwise)
 //   chunk<OUT = true>    per (chunk, head): from that state, sixteen tokens at a time:
 //                            o_i = (q_i e^b_i)^T S + sum over j <= i of (sum_d q_id k_jd e^(b_id - b_jd)) v_j
+//                            with a bonus: b_(i-1) in the place of b_i, j < i, and (sum_d q_id u_d k_id) v_i on top
 //                            S  <- diag(e^b_n) S + sum_j (k_j e^(b_n - b_j)) v_j^T        b: running sum of log decays
 //                        norm and gate in the same launch when one workgroup holds all of a head's columns.
 // Every exponent that is formed is <= 0 but one: e^-b_j, used only while the sixteen tokens' b stays above -40; stronger
@@ -28,12 +32,15 @@ struct LinArgs {
   long q_stride, k_stride, v_stride, z_stride, g_stride;
   const float* z_bias;          // [H * D] or null
   float inv_tau;
+  int decay_exp;                // decay exp(-exp(z + bias)) instead of sigmoid(z + bias)^inv_tau
+  const float* bonus;           // [H * D] or null (with z only)
   const float* log_decay;       // [H] (no z)
   const float* cos_sin;         // [positions, rot]
   const long* positions;
   int rot;
   float q_scale, k_scale;
-  const float* norm_w;          // [Dv] or null
+  const float* norm_w;          // [Dv], [H * Dv] (norm_head = Dv) or null
+  int norm_head;                // values between two heads' norm weights
   float eps;
   float* state;                 // [slots, H, Dv, D]
   void* out;
@@ -81,6 +88,12 @@ __device__ __forceinline__ f32x4 lin_row4(const LinArgs& a, const T* row, int d,
   return x;
 }
 
+// log decay of a channel whose pre-activation is z.  exp(-exp(z)) is zero in fp32 long before the bound, which keeps
+// differences of running sums finite and exact.
+__device__ __forceinline__ float lin_log_decay(const LinArgs& a, float z) {
+  return a.decay_exp ? fmaxf(-expf(z), -200.f) : rec_logsigmoid(z) * a.inv_tau;
+}
+
 // log decays of channels d .. d + 3 at token t (0 beyond D)
 template <typename T>
 __device__ __forceinline__ f32x4 lin_log_decay4(const LinArgs& a, long t, int h, int d) {
@@ -90,13 +103,13 @@ __device__ __forceinline__ f32x4 lin_log_decay4(const LinArgs& a, long t, int h,
   const f32x4 z = load4<T>((const T*)a.z + t * a.z_stride + (long)h * a.D + d, n, a.vec);
 #pragma unroll
   for (int i = 0; i < 4; ++i)
-    if (i < n) o[i] = rec_logsigmoid(z[i] + (a.z_bias ? a.z_bias[(long)h * a.D + d + i] : 0.f)) * a.inv_tau;
+    if (i < n) o[i] = lin_log_decay(a, z[i] + (a.z_bias ? a.z_bias[(long)h * a.D + d + i] : 0.f));
   return o;
 }
 
 // ---- few new tokens ------------------------------------------------------------------------------------------------
 // grid (H, S); 16 columns x 16 lanes at a time, NCG such column groups in registers together
-template <typename T, int NR, bool CHAN>
+template <typename T, int NR, bool CHAN, bool BONUS>
 __global__ __launch_bounds__(256) void lin_step_kernel(const LinArgs a, const int tile) {
   constexpr int NCG = NR <= 8 ? 4 : NR <= 16 ? 2 : 1;
   constexpr int DP = 16 * NR;
@@ -117,7 +130,14 @@ __global__ __launch_bounds__(256) void lin_step_kernel(const LinArgs a, const in
   const bool vs4 = (D & 3) == 0;
   float* Sb = a.state + ((long)a.slot_table[s * a.st_stride] * a.H + h) * (long)Dv * D;
   const float gh = CHAN ? 0.f : expf(a.log_decay[h]);
-  float S[NCG][NR];
+  float S[NCG][NR], ur[NR];
+  if (BONUS) {
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      const int d = rec_lane_value<NR>(part, i);
+      ur[i] = d < D ? a.bonus[(long)h * D + d] : 0.f;
+    }
+  }
   auto load_group = [&](int c0, bool live) {
 #pragma unroll
     for (int n = 0; n < NCG; ++n) {
@@ -162,8 +182,10 @@ __global__ __launch_bounds__(256) void lin_step_kernel(const LinArgs a, const in
           float p = 0.f;
 #pragma unroll
           for (int i = 0; i < NR; ++i) {
-            S[n][i] = S[n][i] * (CHAN ? gr[i] : gh) + kr[i] * v;
-            p += S[n][i] * qr[i];
+            const float kv = kr[i] * v;
+            if (BONUS) p += (S[n][i] + ur[i] * kv) * qr[i];
+            S[n][i] = S[n][i] * (CHAN ? gr[i] : gh) + kv;
+            if (!BONUS) p += S[n][i] * qr[i];
           }
           p = row16_sum(p);
           if (part == 0 && col < Dv) os[tt * Dv + col] = p;
@@ -187,7 +209,7 @@ __global__ __launch_bounds__(256) void lin_step_kernel(const LinArgs a, const in
       for (int c = lane; c < Dv; c += 64) {
         const float zg = (float)((const T*)a.gate)[t * a.g_stride + (long)h * Dv + c];
         ((T*)a.out)[t * a.o_stride + (long)h * Dv + c] =
-            (T)(o[c] * rs * (a.norm_w ? a.norm_w[c] : 1.f) * zg * rec_sigmoid(zg));
+            (T)(o[c] * rs * (a.norm_w ? a.norm_w[(long)h * a.norm_head + c] : 1.f) * zg * rec_sigmoid(zg));
       }
     }
   }
@@ -200,7 +222,7 @@ __global__ __launch_bounds__(256) void lin_step_kernel(const LinArgs a, const in
 // Staging layout: thread -> token tid / 16, values d0 + 64 m with d0 = 4 * (tid % 16).  The next sixteen tokens' rows are
 // on their way from memory, unconverted, while these are computed; a block's output leaves LDS in the staging phase of
 // the next one, so two barriers (four with channel decays) separate everything.
-template <typename T, int DT, int ET, bool CHAN, bool OUT>
+template <typename T, int DT, int ET, bool CHAN, bool OUT, bool BONUS>
 __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_kernel(const LinArgs a) {
   constexpr int DP = DT * 16, QP = DP + 4, TP = 20, CW = 64 * ET, OP = CW + 4;
   constexpr int NI = (DP + 63) / 64, NVI = ET;
@@ -213,6 +235,7 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
   float* os = qs + (OUT ? 16 * QP : 0);                // [16][OP]   (OUT)
   float* bc = os + (OUT ? 16 * OP : 0);                // [16][QP]   (CHAN) running sums of log decays
   float* dec = bc + (CHAN ? 16 * QP : 0);              // [DP]       (CHAN) e^b_n
+  float* bon = dec + (CHAN ? DP : 0);                  // [16]       (BONUS) sum_d q u k of each token
   const int srel = blockIdx.y, s = a.seq0 + srel, tid = threadIdx.x;
   const int sl = a.seq_lens[s];
   if (sl <= 0) return;
@@ -258,6 +281,12 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
   const T* zp = CHAN ? (const T*)a.z + (long)h * D + t0 * a.z_stride : nullptr;
   const T* gp = (const T*)a.gate + (long)h * Dv + t0 * a.g_stride;
   V4 rk[NI], rk2[NI], rq[NI], rq2[NI], rz[NI], rv[NVI], rg[NVI];
+  f32x4 ru[NI];
+  if (BONUS && OUT) {
+#pragma unroll
+    for (int m = 0; m < NI; ++m)
+      ru[m] = *reinterpret_cast<const f32x4*>(a.bonus + (long)h * D + (d0 + 64 * m < D ? d0 + 64 * m : 0));
+  }
   int pos = 0;
   auto fetch = [&](int tb) {
     const long t = min(tb + tt, L - 1);
@@ -306,7 +335,7 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
       const int cc = d0 + 64 * m;
       if (cc >= Dv) continue;
       f32x4 w = {1.f, 1.f, 1.f, 1.f};
-      if (a.norm_w) w = *reinterpret_cast<const f32x4*>(a.norm_w + cc);
+      if (a.norm_w) w = *reinterpret_cast<const f32x4*>(a.norm_w + (long)h * a.norm_head + cc);
       V4 y;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -334,6 +363,7 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
     __syncthreads();
     if (OUT && tb > first) emit(tb - 16);
     const float f = CHAN ? 0.f : expf(ld * (float)max(n - 1 - tt, 0));
+    float quk = 0.f;
 #pragma unroll
     for (int m = 0; m < NI; ++m) {
       const int d = d0 + 64 * m;
@@ -354,18 +384,23 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
       }
       *reinterpret_cast<f32x4*>(ks + tt * QP + d) = k;
       if (OUT) *reinterpret_cast<f32x4*>(qs + tt * QP + d) = q;
+      if (BONUS && OUT) quk += q[0] * k[0] * ru[m][0] + q[1] * k[1] * ru[m][1] + q[2] * k[2] * ru[m][2] + q[3] * k[3] * ru[m][3];
       if (CHAN) {
         if (live) {
           f32x4 zb = {0.f, 0.f, 0.f, 0.f};
           if (a.z_bias) zb = *reinterpret_cast<const f32x4*>(a.z_bias + (long)h * D + d);
 #pragma unroll
-          for (int i = 0; i < 4; ++i) b[i] = rec_logsigmoid((float)rz[m][i] + zb[i]) * a.inv_tau;
+          for (int i = 0; i < 4; ++i) b[i] = lin_log_decay(a, (float)rz[m][i] + zb[i]);
         }
         *reinterpret_cast<f32x4*>(bc + tt * QP + d) = b;
       } else {
 #pragma unroll
         for (int i = 0; i < 4; ++i) kT[(d + i) * TP + tt] = k[i] * f;
       }
+    }
+    if (BONUS && OUT) {                                // a token's values sit in sixteen neighbouring lanes
+      quk = row16_sum(quk);
+      if ((tid & 15) == 0) bon[tt] = quk;
     }
 #pragma unroll
     for (int m = 0; m < NVI; ++m) {
@@ -404,11 +439,11 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
         // element by element, all exponents <= 0
         if (busy) {
           for (int d = 0; d < D; ++d) {
-            const float qi = qs[lo * QP + d], bi = bc[lo * QP + d];
+            const float qi = qs[lo * QP + d], bi = BONUS ? (lo ? bc[(lo - 1) * QP + d] : 0.f) : bc[lo * QP + d];
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int j = 4 * g + r;
-              pt[r] += j <= lo ? qi * ks[j * QP + d] * expf(bi - bc[j * QP + d]) : 0.f;
+              pt[r] += j <= lo - (BONUS ? 1 : 0) ? qi * ks[j * QP + d] * expf(bi - bc[j * QP + d]) : 0.f;
             }
           }
         }
@@ -425,9 +460,11 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
         for (int i = 0; i < 4; ++i) kT[(d + i) * TP + tt] = k[i] * expf(bn[i] - b[i]);
         if (OUT) {
           f32x4 q = *reinterpret_cast<const f32x4*>(qs + tt * QP + d);
+          f32x4 bq = b;                                // the decays between the state's time and the read-out
+          if (BONUS) bq = tt ? *reinterpret_cast<const f32x4*>(bc + (tt - 1) * QP + d) : f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            q[i] *= expf(b[i]);
+            q[i] *= expf(bq[i]);
             if (!strong) k[i] *= expf(-b[i]);
           }
           *reinterpret_cast<f32x4*>(qs + tt * QP + d) = q;
@@ -451,6 +488,11 @@ __global__ __launch_bounds__(256, DT <= 4 ? 3 : DT == 8 ? 2 : 1) void lin_chunk_
         pt += pt2;
 #pragma unroll
         for (int r = 0; r < 4; ++r) pt[r] = CHAN ? (4 * g + r <= lo ? pt[r] : 0.f) : pt[r] * pf[r];
+      }
+      if (BONUS) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (4 * g + r == lo) pt[r] = bon[lo];
       }
       f32x4 O[ET], o2[ET];
 #pragma unroll
@@ -580,14 +622,14 @@ VDA_EXPORT int vda_linear_attention_fused(int D, int Dv) {           // can one 
 
 VDA_EXPORT int vda_linear_attention(
     void* out, long o_stride, float* o_raw, float* scratch, const void* q, long q_stride, const void* k, long k_stride,
-    const void* v, long v_stride, const void* z, long z_stride, const float* z_bias, float inv_tau,
-    const float* log_decay, const void* gate, long g_stride, const float* cos_sin, const long* positions, int rot,
-    float q_scale, float k_scale, const float* norm_w, float eps, float* state, const int* qsl, const int* seq_lens,
+    const void* v, long v_stride, const void* z, long z_stride, const float* z_bias, float inv_tau, int decay_exp,
+    const float* bonus, const float* log_decay, const void* gate, long g_stride, const float* cos_sin, const long* positions, int rot,
+    float q_scale, float k_scale, const float* norm_w, int norm_head, float eps, float* state, const int* qsl, const int* seq_lens,
     const int* slot_table, long st_stride, int T, int S, int seq0, int H, int D, int Dv, int max_q, int C,
     int dtype, hipStream_t st) {
   if (S <= 0 || T <= 0) return 0;
   if (H <= 0 || D < 1 || Dv < 1 || D > 1024 || rot < 0 || rot > D || (rot & 1) || (rot > 0 && (!cos_sin || !positions)) ||
-      (!z && !log_decay) || seq0 < 0 || seq0 > S)
+      (!z && !log_decay) || seq0 < 0 || seq0 > S || (bonus && !z) || (norm_head != 0 && norm_head != Dv))
     return -1;
   // chunk-parallel for key widths of up to 256: sequences of more than 16 new tokens, from seq0 on,
   // and only for rows that can be read four values at a time
@@ -597,13 +639,14 @@ VDA_EXPORT int vda_linear_attention(
   const bool vec_v = Dv % 4 == 0 && ok4(v, v_stride) && ok4(gate, g_stride) && ok4(out, o_stride) &&
                      !((uintptr_t)norm_w % 16);
   const bool chunked = D <= 256 && max_q > 16 && scratch && seq0 < S && C >= 16 && C % 16 == 0 && vec && vec_v &&
-                       rot % 8 == 0 && (!z || rot == 0) && !((uintptr_t)z_bias % 16) && !((uintptr_t)cos_sin % 16);
+                       rot % 8 == 0 && (!z || rot == 0) && !((uintptr_t)z_bias % 16) && !((uintptr_t)bonus % 16) &&
+                       !((uintptr_t)cos_sin % 16);
   const int DT = lin_dt(D);
   const int ET = (DT <= 8 && Dv > 64) ? 2 : 1;
   LinArgs a;
   a.q = q; a.k = k; a.v = v; a.z = z; a.gate = gate;
   a.q_stride = q_stride; a.k_stride = k_stride; a.v_stride = v_stride; a.z_stride = z_stride; a.g_stride = g_stride;
-  a.z_bias = z_bias; a.inv_tau = inv_tau; a.log_decay = log_decay; a.cos_sin = cos_sin; a.positions = positions;
+  a.z_bias = z_bias; a.inv_tau = inv_tau; a.decay_exp = decay_exp; a.bonus = bonus; a.norm_head = norm_head; a.log_decay = log_decay; a.cos_sin = cos_sin; a.positions = positions;
   a.rot = rot; a.q_scale = q_scale; a.k_scale = k_scale; a.norm_w = norm_w; a.eps = eps; a.state = state; a.out = out;
   a.o_stride = o_stride; a.qsl = qsl; a.seq_lens = seq_lens; a.slot_table = slot_table; a.st_stride = st_stride;
   a.H = H; a.D = D; a.Dv = Dv; a.seq0 = seq0; a.C = C;
@@ -625,8 +668,9 @@ VDA_EXPORT int vda_linear_attention(
   const size_t slds = step_lds(tile);
 #define STEP(TT, NN)                                                                                                   \
   do {                                                                                                                 \
-    if (z) hipLaunchKernelGGL((lin_step_kernel<TT, NN, true>), dim3(H, S), dim3(256), slds, st, a, tile);              \
-    else hipLaunchKernelGGL((lin_step_kernel<TT, NN, false>), dim3(H, S), dim3(256), slds, st, a, tile);               \
+    if (bonus) hipLaunchKernelGGL((lin_step_kernel<TT, NN, true, true>), dim3(H, S), dim3(256), slds, st, a, tile);    \
+    else if (z) hipLaunchKernelGGL((lin_step_kernel<TT, NN, true, false>), dim3(H, S), dim3(256), slds, st, a, tile);  \
+    else hipLaunchKernelGGL((lin_step_kernel<TT, NN, false, false>), dim3(H, S), dim3(256), slds, st, a, tile);        \
   } while (0)
 #define STEPS(TT)                                                                                                      \
   switch (NR) {                                                                                                        \
@@ -651,19 +695,24 @@ VDA_EXPORT int vda_linear_attention(
   const dim3 grid(nch, S - seq0, H * a.col_groups);
   auto chunk_lds = [&](bool outp) {
     return ((size_t)16 * QP * (1 + (outp ? 1 : 0) + (z ? 1 : 0)) + (size_t)DP * 20 + (size_t)64 * ET * 20 +
-            (outp ? (size_t)16 * (64 * ET + 4) : 0) + (z ? DP : 0)) * 4;
+            (outp ? (size_t)16 * (64 * ET + 4) : 0) + (z ? DP : 0) + (bonus ? 16 : 0)) * 4;
   };
-#define CK(TT, DD, EE, CC, OO)                                                                                         \
+#define CK(TT, DD, EE, CC, OO, BB)                                                                                       \
   do {                                                                                                                 \
     const size_t lb = chunk_lds(OO);                                                                                   \
     if (lb > 48 * 1024) {                                                                                              \
-      hipError_t e_ = hipFuncSetAttribute((const void*)lin_chunk_kernel<TT, DD, EE, CC, OO>,                           \
+      hipError_t e_ = hipFuncSetAttribute((const void*)lin_chunk_kernel<TT, DD, EE, CC, OO, BB>,                       \
                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)lb);                        \
       if (e_ != hipSuccess) return (int)e_;                                                                            \
     }                                                                                                                  \
-    hipLaunchKernelGGL((lin_chunk_kernel<TT, DD, EE, CC, OO>), grid, dim3(256), lb, st, a);                            \
+    hipLaunchKernelGGL((lin_chunk_kernel<TT, DD, EE, CC, OO, BB>), grid, dim3(256), lb, st, a);                        \
   } while (0)
-#define CB(TT, DD, EE, OO) do { if (z) CK(TT, DD, EE, true, OO); else CK(TT, DD, EE, false, OO); } while (0)
+#define CB(TT, DD, EE, OO)                                                                                             \
+  do {                                                                                                                 \
+    if (OO && bonus) CK(TT, DD, EE, true, OO, OO); /* the bonus concerns the outputs only */                           \
+    else if (z) CK(TT, DD, EE, true, OO, false);                                                                       \
+    else CK(TT, DD, EE, false, OO, false);                                                                             \
+  } while (0)
 #define CA(TT, OO)                                                                                                     \
   do {                                                                                                                 \
     if (DT == 2 && ET == 1) CB(TT, 2, 1, OO); else if (DT == 2) CB(TT, 2, 2, OO);                                      \
@@ -689,7 +738,7 @@ VDA_EXPORT int vda_linear_attention(
   if (a.o_raw) {
     const dim3 ge((unsigned)(((long)max_q * H + 3) / 4), S - seq0);
 #define EP(TT) hipLaunchKernelGGL((head_norm_silu_kernel<TT>), ge, dim3(256), 0, st, (TT*)out, o_stride, o_raw,        \
-                                  (const TT*)gate, g_stride, norm_w, qsl, seq_lens, seq0, a.limit, H, Dv, eps)
+                                  (const TT*)gate, g_stride, norm_w, norm_head, qsl, seq_lens, seq0, a.limit, H, Dv, eps)
     if (dtype == VDA_BF16) EP(bf16_t);
     else if (dtype == VDA_F16) EP(f16_t);
     else EP(float);

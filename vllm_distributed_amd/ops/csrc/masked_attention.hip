@@ -4,6 +4,7 @@
 //     fp32 cos | sin table; or ONE norm over all query heads of a token and one over all key heads (`whole`), with
 //     weights as long as the projections;
 //   * a query temperature: queries at position p times 1 + coef * ln(floor((p + 1) / every) + 1);
+//   * values that are the projected keys themselves, before norm and rotation (`key_values`);
 //   * value mixing: v <- (1 - lam) v + lam v_first with the values another layer made of the same token, before the
 //     cache write;
 //   * scores squashed by cap * tanh(score / cap); a learned bias per (query - key distance, head) from a table whose
@@ -40,6 +41,7 @@ struct QkExtras {
   long v_first_stride;
   const float* v_lam;      // one value: v <- (1 - lam) v + lam v_first
   int whole;               // one norm over all queries, one over all keys; q_w, k_w as long as the projections
+  int key_values;          // the values are the projected keys (before norm and rotation); maps == 1, D == Dv
 };
 
 // 1 / rms of all query values and of all key values of a token (q | k side by side in `row`), every thread of the block;
@@ -139,7 +141,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_cache_kernel(
     }
   }
   if (slot >= 0) {
-    const T* vsrc = row + (long)(nq + nk) * D;
+    const T* vsrc = row + (long)(x.key_values ? nq : nq + nk) * D;
     T* vdst = v_cache + (slot / bs) * (long)G * Dv * bs + slot % bs;      // [blocks, G, Dv, bs]
     for (int e = tid; e < G * Dv; e += 256) vdst[(long)e * bs] = mixed_value<T>(x, vsrc[e], t, e);
   }
@@ -228,7 +230,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_cache_vec_kernel(
     st16<V8>(dst + d0, o8);
   }
   if (slot >= 0) {
-    const T* vsrc = row + (long)total * D;
+    const T* vsrc = row + (long)(xo.key_values ? nq : total) * D;
     T* vdst = v_cache + (slot / bs) * (long)G * Dv * bs + slot % bs;      // [blocks, G, Dv, bs]
     for (int e = tid; e < G * Dv; e += 256) vdst[(long)e * bs] = mixed_value<T>(xo, vsrc[e], t, e);
   }
@@ -239,10 +241,12 @@ VDA_EXPORT int vda_qk_norm_rope_cache(void* qn, const void* qkv, long qkv_stride
                                       const long* slot_mapping, int T, int H, int G, int D, int Dv, int maps, int rot,
                                       int bs, float eps, int by_map, int neighbours, float q_coef, int q_every,
                                       const void* v_first, long v_first_stride, const float* v_lam, int whole,
-                                      int dtype, hipStream_t st) {
+                                      int key_values, int dtype, hipStream_t st) {
   if (T <= 0) return 0;
-  if (rot < 0 || rot > D || (rot & 1) || maps < 1 || (rot > 0 && !cos_sin) || (v_first && !v_lam)) return -1;
-  const QkExtras xo{neighbours, q_coef, q_every, v_first, v_first_stride, v_lam, whole};
+  if (rot < 0 || rot > D || (rot & 1) || maps < 1 || (rot > 0 && !cos_sin) || (v_first && !v_lam) ||
+      (key_values && (maps != 1 || D != Dv)))
+    return -1;
+  const QkExtras xo{neighbours, q_coef, q_every, v_first, v_first_stride, v_lam, whole, key_values};
   // half-split pairs: the partner sits rot / 16 lanes away; neighbours: inside the lane's own eight values
   const bool vec = (D == 32 || D == 64 || D == 128 || D == 256) && (neighbours ? rot % 8 == 0 : (rot / 2) % 8 == 0) &&
                    qkv_stride % 8 == 0 &&

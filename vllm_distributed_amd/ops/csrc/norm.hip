@@ -298,7 +298,8 @@ VDA_EXPORT int vda_group_rms_norm(void* out, long o_stride, const void* x, long 
 //   h[t]  = x[t] / rms_g(x[t]) * w_next    with rms_g the root mean square of the value's own part, the row being
 //           split into `groups` equal consecutive parts
 // Every piece is optional: no sub-layer at all is the stack's first or last norm, no h is the last residual update; up to
-// three sub-layer outputs join in one pass (a shared expert beside the routed ones takes the third place).
+// three sub-layer outputs join in one pass (a shared expert beside the routed ones takes the third place).  A row `step`
+// [W], the same for every token, joins behind them; h without w_next is the updated row itself in the activation type.
 // One workgroup per token; the updated row waits in LDS for its parts' sums.
 struct GatedSub {
   const void* y;        // [T, W] the sub-layer's output
@@ -314,6 +315,7 @@ struct GatedResidualArgs {
   float* x;
   GatedSub sub[3];
   int nsub;
+  const float* step;    // [W] or null
   const float* w_next;
   void* h;
   long h_stride;
@@ -354,7 +356,11 @@ __global__ __launch_bounds__(256) void gated_residual_group_norm_kernel(const Ga
         add[i] += f;
       }
     }
-    if (a.nsub > 0) {
+    if (a.step) {
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) add[i] += a.step[c + i];
+    }
+    if (a.nsub > 0 || a.step) {
 #pragma unroll
       for (int i = 0; i < VEC; ++i) v[i] += add[i];
       if (VEC == 4) *reinterpret_cast<f32x4*>(xr + c) = f32x4{v[0], v[1 % VEC], v[2 % VEC], v[3 % VEC]};
@@ -364,6 +370,14 @@ __global__ __launch_bounds__(256) void gated_residual_group_norm_kernel(const Ga
     for (int i = 0; i < VEC; ++i) row[c + i] = v[i];
   }
   if (!a.h) return;
+  if (!a.w_next) {                        // every thread casts the values it holds
+    T* hr = (T*)a.h + t * a.h_stride;
+    for (int c = tid * VEC; c < W; c += 256 * VEC) {
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) hr[c + i] = (T)row[c + i];
+    }
+    return;
+  }
   __syncthreads();
   const int part = W / a.groups;
   for (int g = wave; g < a.groups; g += 4) {
@@ -428,7 +442,12 @@ __global__ __launch_bounds__(256) void gated_residual_group_norm_reg_kernel(cons
 #pragma unroll
         for (int i = 0; i < 4; ++i) add[i] += f[i];
       }
-      if (a.nsub > 0) {
+      if (a.step) {
+        const f32x4 s4 = *reinterpret_cast<const f32x4*>(a.step + c);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) add[i] += s4[i];
+      }
+      if (a.nsub > 0 || a.step) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) v[k][i] += add[i];
         *reinterpret_cast<f32x4*>(xr + c) = f32x4{v[k][0], v[k][1], v[k][2], v[k][3]};
@@ -437,7 +456,7 @@ __global__ __launch_bounds__(256) void gated_residual_group_norm_reg_kernel(cons
 #pragma unroll
       for (int i = 0; i < 4; ++i) v[k][i] = 0.f;
     }
-    if (a.h) {
+    if (a.h && a.w_next) {
       float ss = v[k][0] * v[k][0] + v[k][1] * v[k][1] + v[k][2] * v[k][2] + v[k][3] * v[k][3];
       if (seg) {                                      // a part is `seg` neighbouring lanes: its sum stays in the wave
         for (int o = seg >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
@@ -449,9 +468,18 @@ __global__ __launch_bounds__(256) void gated_residual_group_norm_reg_kernel(cons
     }
   }
   if (!a.h) return;
+  T* hr = (T*)a.h + t * a.h_stride;
+  if (!a.w_next) {
+    using V4 = typename Vec<T>::v4;
+#pragma unroll
+    for (int k = 0; k < TRIPS; ++k) {
+      const int c = (k * 256 + tid) * 4;
+      if (c < W) *reinterpret_cast<V4*>(hr + c) = V4{(T)v[k][0], (T)v[k][1], (T)v[k][2], (T)v[k][3]};
+    }
+    return;
+  }
   if (!seg) __syncthreads();
   const int part = W / a.groups;
-  T* hr = (T*)a.h + t * a.h_stride;
 #pragma unroll
   for (int k = 0; k < TRIPS; ++k) {
     const int c = (k * 256 + tid) * 4;
@@ -478,16 +506,16 @@ VDA_EXPORT int vda_gated_residual_group_norm(
     float* x, int nsub, const void* y0, long y0_stride, const float* s0, const void* g0, long g0_stride,
     const void* e0, long e0_stride, const float* ew0, const void* y1, long y1_stride, const float* s1, const void* g1,
     long g1_stride, const void* e1, long e1_stride, const float* ew1, const void* y2, long y2_stride, const float* s2,
-    const void* g2, long g2_stride, const void* e2, long e2_stride, const float* ew2, const float* w_next, void* h,
-    long h_stride, float eps, int groups, int T, int W, int dtype, hipStream_t st) {
-  if (T <= 0 || (nsub == 0 && !h)) return 0;
-  if (nsub < 0 || nsub > 3 || (nsub > 0 && !y0) || (nsub > 1 && !y1) || (nsub > 2 && !y2) || (h && !w_next) ||
+    const void* g2, long g2_stride, const void* e2, long e2_stride, const float* ew2, const float* step,
+    const float* w_next, void* h, long h_stride, float eps, int groups, int T, int W, int dtype, hipStream_t st) {
+  if (T <= 0 || (nsub == 0 && !h && !step)) return 0;
+  if (nsub < 0 || nsub > 3 || (nsub > 0 && !y0) || (nsub > 1 && !y1) || (nsub > 2 && !y2) ||
       groups < 1 || W % groups || (e0 && !ew0) || (e1 && !ew1) || (e2 && !ew2))
     return -1;
   const size_t lds = ((size_t)W + groups) * 4;
   if (lds > 60 * 1024) return -2;
   GatedResidualArgs a;
-  a.x = x; a.nsub = nsub; a.w_next = w_next; a.h = h; a.h_stride = h_stride; a.eps = eps; a.W = W; a.groups = groups;
+  a.x = x; a.nsub = nsub; a.step = step; a.w_next = w_next; a.h = h; a.h_stride = h_stride; a.eps = eps; a.W = W; a.groups = groups;
   a.sub[0] = GatedSub{y0, y0_stride, s0, g0, g0_stride, e0, e0_stride, ew0};
   a.sub[1] = GatedSub{y1, y1_stride, s1, g1, g1_stride, e1, e1_stride, ew1};
   a.sub[2] = GatedSub{y2, y2_stride, s2, g2, g2_stride, e2, e2_stride, ew2};
@@ -501,7 +529,7 @@ VDA_EXPORT int vda_gated_residual_group_norm(
   int seg = 0;                                             // lanes per part when a part is a power of two <= 256
   if (part % 256 != 0 && part >= 4 && part <= 256 && (part & (part - 1)) == 0) seg = part / 4;
   const bool reg = vec && trips <= 4 && (part % 256 == 0 || seg) && ((uintptr_t)x % 16 == 0) &&
-                   (!w_next || (uintptr_t)w_next % 16 == 0) && (!h || (uintptr_t)h % al == 0) && [&] {
+                   (uintptr_t)step % 16 == 0 && (!w_next || (uintptr_t)w_next % 16 == 0) && (!h || (uintptr_t)h % al == 0) && [&] {
                      for (int i = 0; i < nsub; ++i) {
                        const GatedSub& u = a.sub[i];
                        if ((uintptr_t)u.y % al || (uintptr_t)u.gate % al || (uintptr_t)u.extra % al ||

@@ -126,12 +126,13 @@ template <int NR> __device__ __forceinline__ void rec_lane_row(float* o, const f
 }
 
 // out[t, h, :] = o / sqrt(mean(o^2) + eps) * norm_w * silu(gate) over a head's Dv values, for the tokens of sequences
-// seq0 + blockIdx.y with more than `limit` new tokens: one wave per (token, head).  norm_w may be null (no weight).
+// seq0 + blockIdx.y with more than `limit` new tokens: one wave per (token, head).  norm_w may be null (no weight); its
+// rows of Dv values lie norm_head apart (0: one row for all heads).
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_silu_kernel(T* __restrict__ out, long o_stride,
                                                              const float* __restrict__ o_raw,
                                                              const T* __restrict__ gate, long g_stride,
-                                                             const float* __restrict__ norm_w,
+                                                             const float* __restrict__ norm_w, int norm_head,
                                                              const int* __restrict__ qsl,
                                                              const int* __restrict__ seq_lens, int seq0, int limit,
                                                              int H, int Dv, float eps) {
@@ -150,6 +151,6 @@ __global__ __launch_bounds__(256) void head_norm_silu_kernel(T* __restrict__ out
   const float rs = 1.f / sqrtf(ss / (float)Dv + eps);
   for (int j = lane; j < Dv; j += 64) {
     const float z = (float)gate[t * g_stride + (long)h * Dv + j];
-    out[t * o_stride + (long)h * Dv + j] = (T)(o[j] * rs * (norm_w ? norm_w[j] : 1.f) * z * rec_sigmoid(z));
+    out[t * o_stride + (long)h * Dv + j] = (T)(o[j] * rs * (norm_w ? norm_w[(long)h * norm_head + j] : 1.f) * z * rec_sigmoid(z));
   }
 }

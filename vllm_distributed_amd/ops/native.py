@@ -23,7 +23,7 @@ BF16, F16, F32, FP8 = 0, 1, 2, 3
 _DT = {torch.bfloat16: BF16, torch.float16: F16, torch.float32: F32, torch.float8_e4m3fn: FP8}
 
 ACT = {"silu": 0, "gelu": 1, "gelu_tanh": 2, "gelu_pytorch_tanh": 2, "relu": 3, "gelu_new": 4,
-       "gelu_fast": 5, "quick_gelu": 6, "gelu_quick": 6, "fatrelu": 7, "relu2": 8, "clamped_swiglu": 9}
+       "gelu_fast": 5, "quick_gelu": 6, "gelu_quick": 6, "fatrelu": 7, "relu2": 8, "clamped_swiglu": 9, "tanh": 10}
 
 P, I, L, F = c_void_p, c_int, c_long, c_float
 _SIGS = {
@@ -60,17 +60,18 @@ _SIGS = {
     "vda_moe_topk_softmax": [P, P, P, I, I, I, I, L, I, P],
     "vda_moe_align": [P, P, P, I, I, P],
     "vda_residual_norms": [P, P, L, P, P, P, L, F, F, I, I, I, P],
-    "vda_latent_norm_rope_cache": [P, L, P, L, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, P],
+    "vda_latent_norm_rope_cache": [P, L, P, L, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P],
+    "vda_head_gate_rows": [P, P, L, L, P, L, I, I, I, I, P],
     "vda_latent_window_attention": [P, P, P, P, L, P, P, F, I, I, I, I, I, I, I, P, I, P],
     "vda_mlstm": [P, L, P, P, L, P, P, P, P, P, P, P, P, L, I, I, I, I, I, I, F, F, I, P],
     "vda_moe_grouped_sigmoid_topk": [P, P, P, P, I, I, I, I, I, I, L, I, P],
     "vda_moe_grouped_topk": [P, P, P, P, P, I, I, I, I, I, I, F, I, I, I, L, I, P],
-    "vda_gated_residual_group_norm": [P, I] + [P, L, P, P, L, P, L, P] * 3 + [P, P, L, F, I, I, I, I, P],
+    "vda_gated_residual_group_norm": [P, I] + [P, L, P, P, L, P, L, P] * 3 + [P, P, P, L, F, I, I, I, I, P],
     "vda_group_rms_norm": [P, L, P, L, P, F, I, I, I, I, I, P],
     "vda_moe_pairs": [P, L, P, P, L, P, P, P, P, I, I, I, I, I, I, F, I, I, P],
     "vda_residual_layer_norm": [P, P, L, P, P, P, L, F, I, I, I, P, L, P, L, P],
     "vda_fp32_rows_dot": [P, P, L, P, P, I, I, I, I, P],
-    "vda_qk_norm_rope_cache": [P, P, L, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, I, F, I, P, L, P, I, I, P],
+    "vda_qk_norm_rope_cache": [P, P, L, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, I, F, I, P, L, P, I, I, I, P],
     "vda_map_combine": [P, P, P, P, L, I, I, I, I, I, I, F, F, I, P],
     "vda_masked_softmax_attention": [P, P, P, P, P, L, P, P, P, P, P, L, I, F, I, I, I, F, F, I, I, I, I, I, I, I, F, P,
                                      I, I, P],
@@ -111,8 +112,9 @@ _SIGS = {
     "vda_gated_delta_rule_head": [P, L, P, P, P, L, P, L, P, L, P, L, P, P, P, P, P, P, P, L, I, I, I, I, I, I, I, I, F,
                                   I, P],
     "vda_delta_head_scratch": [I, I, I, I, I],
-    "vda_linear_attention": [P, L, P, P, P, L, P, L, P, L, P, L, P, F, P, P, L, P, P, I, F, F, P, F, P, P, P, P, L, I, I, I,
-                             I, I, I, I, I, I, P],
+    "vda_linear_attention": [P, L, P, P, P, L, P, L, P, L, P, L, P, F, I, P, P, P, L, P, P, I, F, F, P, I, F, P, P, P, P, L,
+                             I, I, I, I, I, I, I, I, I, P],
+    "vda_token_shift_mix": [P, L, P, L, P, P, P, P, P, L, I, I, I, I, I, I, P],
     "vda_linear_attention_scratch": [I, I, I, I, I, I],
     "vda_linear_attention_fused": [I, I],
     "vda_residual_squash_norm": [P, I, P, L, P, P, L, P, F, F, P, L, P, P, P, P, P, L, I, I, I, P],

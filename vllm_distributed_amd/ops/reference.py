@@ -52,6 +52,8 @@ def _act(kind: str, x: torch.Tensor, threshold: float = 0.0) -> torch.Tensor:
         return torch.where(x > threshold, x, torch.zeros_like(x))
     if kind == "relu2":
         return F.relu(x).square()
+    if kind == "tanh":
+        return torch.tanh(x)
     raise ValueError(f"unknown activation {kind!r}")
 
 
@@ -706,10 +708,12 @@ def gated_delta_rule(qkv, a_raw, b_raw, gate_raw, a_log, dt_bias, norm_w, state,
 
 # ---- linear attention with decay ---------------------------------------------------------------------------------
 def linear_attention(q, k, v, gate, norm_w, state, qsl, seq_lens, slot_table, H: int, D: int, Dv: int, eps: float,
-                     log_decay, z, z_bias, tau: float, cos_sin, positions, rot: int, q_scale: float, k_scale: float):
+                     log_decay, z, z_bias, tau: float, cos_sin, positions, rot: int, q_scale: float, k_scale: float,
+                     decay_exp: bool = False, bonus=None):
     """q, k [T, H*D], v, gate [T, H*Dv]; state fp32 [slots, H, Dv, D] (S transposed), updated in place.  q and k rotated
     (halves) and scaled in fp32; per token and head S <- diag(decay) S + k v^T, o = S^T q with decay =
-    exp(log_decay[h]) or sigmoid(z + z_bias)^(1 / tau) per key channel; out = o / rms(o) * norm_w * silu(gate)."""
+    exp(log_decay[h]) or sigmoid(z + z_bias)^(1 / tau) per key channel, or exp(-exp(z + z_bias)) (``decay_exp``); with
+    ``bonus`` [H*D] o = (S + diag(bonus) k v^T)^T q before S takes the token; out = o / rms(o) * norm_w * silu(gate)."""
     T = q.shape[0]
     qf, kf = q.float().reshape(T, H, D), k.float().reshape(T, H, D)
     vf = v.float().reshape(T, H, Dv)
@@ -720,7 +724,7 @@ def linear_attention(q, k, v, gate, norm_w, state, qsl, seq_lens, slot_table, H:
     qf, kf = qf * q_scale, kf * k_scale
     if z is not None:
         zf = z.float() + (z_bias.float() if z_bias is not None else 0.0)
-        decay = torch.exp(F.logsigmoid(zf) / tau).view(T, H, D)
+        decay = (torch.exp(-torch.exp(zf)) if decay_exp else torch.exp(F.logsigmoid(zf) / tau)).view(T, H, D)
     else:
         decay = torch.exp(log_decay.float()).view(1, H, 1).expand(T, H, D)
     out = torch.zeros((T, H, Dv), dtype=torch.float32, device=q.device)
@@ -733,13 +737,36 @@ def linear_attention(q, k, v, gate, norm_w, state, qsl, seq_lens, slot_table, H:
         S = state[slot].transpose(1, 2).clone() if sl - (t1 - t0) > 0 else \
             torch.zeros((H, D, Dv), dtype=torch.float32, device=q.device)
         for t in range(t0, t1):
-            S = decay[t].unsqueeze(-1) * S + kf[t].unsqueeze(-1) * vf[t].unsqueeze(1)
-            out[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+            kv = kf[t].unsqueeze(-1) * vf[t].unsqueeze(1)
+            if bonus is not None:
+                out[t] = torch.einsum("hdv,hd->hv", S + bonus.float().view(H, D, 1) * kv, qf[t])
+            S = decay[t].unsqueeze(-1) * S + kv
+            if bonus is None:
+                out[t] = torch.einsum("hdv,hd->hv", S, qf[t])
         state[slot] = S.transpose(1, 2)
     o = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps)
     if norm_w is not None:
-        o = o * norm_w.float()
+        o = o * norm_w.float().view(-1, Dv)
     return (o.view(T, H * Dv) * F.silu(gate.float())).to(q.dtype)
+
+
+def token_shift_mix(h, mu, state, qsl, seq_lens, slot_table):
+    """h [T, W], mu fp32 [M, W], state [slots, ..., W]: [M, T, W] = h + (h' - h) * mu[m], h' the row before in the same
+    sequence (from the slot for a portion's first row, zeros at the start); the slot keeps the last new row."""
+    T, W = h.shape
+    rows = state.view(-1, W)
+    out = torch.zeros((mu.shape[0], T, W), dtype=h.dtype, device=h.device)
+    for s in range(seq_lens.shape[0]):
+        sl, t0, t1 = int(seq_lens[s]), int(qsl[s]), int(qsl[s + 1])
+        if sl <= 0 or t1 <= t0:
+            continue
+        slot = int(slot_table[s, 0])
+        first = rows[slot: slot + 1] if sl - (t1 - t0) > 0 else torch.zeros_like(h[:1])
+        x = h[t0:t1].float()
+        before = torch.cat([first, h[t0: t1 - 1]]).float()
+        out[:, t0:t1] = (x + (before - x) * mu.float().unsqueeze(1)).to(h.dtype)
+        rows[slot] = h[t1 - 1]
+    return out
 
 
 # ---- fp32 residual under a squashing norm -----------------------------------------------------------------------
@@ -780,12 +807,13 @@ def residual_norms(x, y, w_post, w_pre, eps: float, out_dtype, gain_offset: floa
     return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * (gain_offset + w_pre.float())).to(out_dtype)
 
 
-def gated_residual_group_norm(x, subs, w_next, groups: int, eps: float, out_dtype):
+def gated_residual_group_norm(x, subs, w_next, groups: int, eps: float, out_dtype, step=None, cast_to=None):
     """x fp32 [T, W], in place: x += sum over ``subs`` of y * scale * sigmoid(gate), one tuple (y, scale, gate, extra,
     extra_w) per sub-layer (scale fp32 [W] or None, gate [T, W] pre-activations or None, extra [T, W] with extra_w fp32
     [T] or None: y + extra_w[:, None] * extra takes y's place); the sub-layers' terms are summed before they join x.
+    ``step`` (fp32 [W]) joins every row.
     With ``w_next`` returns every one of ``groups`` equal parts of the updated row divided by its own root mean square,
-    times w_next, in ``out_dtype``."""
+    times w_next, in ``out_dtype``; without it the updated rows go to ``cast_to``, if given."""
     total = None
     for y, scale, gate, extra, extra_w in subs:
         f = y.float()
@@ -796,10 +824,14 @@ def gated_residual_group_norm(x, subs, w_next, groups: int, eps: float, out_dtyp
         if gate is not None:
             f = f * torch.sigmoid(gate.float())
         total = f if total is None else total + f
+    if step is not None:
+        total = step.float() if total is None else total + step.float()
     if total is not None:
         x += total
     if w_next is None:
-        return None
+        if cast_to is not None:
+            cast_to.copy_(x)
+        return cast_to
     T, W = x.shape
     p = x.view(T, groups, W // groups)
     return ((p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)).view(T, W) * w_next.float()).to(out_dtype)
@@ -813,7 +845,7 @@ def rotate_interleaved(x, cos, sin):
 
 
 def latent_norm_rope_cache(q, down, c_weight, cos_sin, positions, qf, kc, slot_mapping, H: int, D: int, P: int,
-                           R: int, rot_dims: int, eps: float, vt=None):
+                           R: int, rot_dims: int, eps: float, vt=None, pairing: str = "neighbours"):
     """q [T, H * (D + P)], down [T, R + P]; cos_sin fp32 [positions, rot_dims] (cosines then sines).
     Cache row of a token = [rms(down[:R]) * c_weight | rotated down[R:]] -> kc [blocks, bs, R + P] at slot_mapping;
     the rotated last P values of every query head go to qf[:, h, R:] (qf [T, H, R + P])."""
@@ -824,9 +856,12 @@ def latent_norm_rope_cache(q, down, c_weight, cos_sin, positions, qf, kc, slot_m
     c = down[:, :R].float()
     c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * c_weight.float()
     kr = down[:, R:].float().clone()
-    kr[:, :rot_dims] = rotate_interleaved(kr[:, :rot_dims], cos, sin)
     qr = q.view(T, H, D + P)[:, :, D:].float().clone()
-    qr[:, :, :rot_dims] = rotate_interleaved(qr[:, :, :rot_dims], cos[:, None], sin[:, None])
+    if pairing == "halves":
+        kr, qr = rotate_halves(kr, cos, sin, rot_dims), rotate_halves(qr, cos[:, None], sin[:, None], rot_dims)
+    else:
+        kr[:, :rot_dims] = rotate_interleaved(kr[:, :rot_dims], cos, sin)
+        qr[:, :, :rot_dims] = rotate_interleaved(qr[:, :, :rot_dims], cos[:, None], sin[:, None])
     qf[:, :, R:] = qr.to(qf.dtype)
     if kc is not None:
         bs = kc.shape[1]
@@ -944,8 +979,9 @@ def position_temperature(positions, coef: float, every: int):
 
 def qk_norm_rope_cache(qkv, H: int, G: int, D: int, Dv: int, maps: int, q_weight, k_weight, cos_sin, positions,
                        rot: int, eps: float, k_cache, v_cache, slot_mapping, pairing: str = "halves", q_temp=None,
-                       v_first=None, v_lam=None, whole_norm: bool = False):
-    """qkv [T, H*maps*D + G*maps*D + G*Dv].  Every D-wide map of every query / key head is divided by its root mean
+                       v_first=None, v_lam=None, whole_norm: bool = False, key_values: bool = False):
+    """qkv [T, H*maps*D + G*maps*D + G*Dv], or without the last part when the values are the projected keys
+    (``key_values``).  Every D-wide map of every query / key head is divided by its root mean
     square, multiplied by q_weight / k_weight [D] and its first ``rot`` values are rotated (cos_sin fp32 [positions, rot],
     cosines then sines; ``pairing``: value i with i + rot / 2, "halves", or 2i with 2i + 1, "neighbours").  ``q_temp`` =
     (coef, every): queries times ``position_temperature``.  ``v_first`` [T, G * Dv] with ``v_lam`` (one fp32 value):
@@ -955,7 +991,7 @@ def qk_norm_rope_cache(qkv, H: int, G: int, D: int, Dv: int, maps: int, q_weight
     nq, nk = H * maps * D, G * maps * D
     q = qkv[:, :nq].float().view(T, H * maps, D)
     k = qkv[:, nq: nq + nk].float().view(T, G * maps, D)
-    v = qkv[:, nq + nk:].view(T, G, Dv)
+    v = qkv[:, nq: nq + nk].view(T, G, Dv) if key_values else qkv[:, nq + nk:].view(T, G, Dv)
     if v_first is not None:
         lam = v_lam.float().reshape(())
         v = ((1.0 - lam) * v.float() + lam * v_first[:T].float().view(T, G, Dv))
