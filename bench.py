@@ -156,6 +156,9 @@ def main() -> None:
     ap.add_argument("--compare-surodra", action="store_true",
                     help="likewise for Surodra stacks (per-head gated delta rule, softmax attention beside gated linear "
                          "attention, retention, squashing norms) beside a Nositar and a Jamba stack of equal size")
+    ap.add_argument("--compare-tilulorn", action="store_true",
+                    help="likewise for Tilulorn stacks (latent attention, window attention over key values, RWKV-style time "
+                         "mixing, experts chosen by token id) beside a Lefolorn and a Surodra stack of equal size")
     ap.add_argument("--sizes", default="small,medium", help="--compare-...: small, medium, large")
     ap.add_argument("--rehearse-on-one-gpu", action="store_true", help="--disagg: every engine on GPU 0")
     ap.add_argument("--kv-push", action="store_true", help="--disagg: push blocks while prefilling (landing pool)")
@@ -165,12 +168,13 @@ def main() -> None:
     if a.disagg:
         return run_disagg(a)
     if a.compare_nositar or a.compare_rapovik or a.compare_sevazen or a.compare_lefolorn or \
-            a.compare_surodra:
+            a.compare_surodra or a.compare_tilulorn:
         from vllm_distributed_amd.benchmarks import hybrid_compare
         argv = (["--models", "rapovik,jamba-moe"] if a.compare_rapovik else
                 ["--models", "sevazen,mixtral-swa"] if a.compare_sevazen else
                 ["--models", "lefolorn,sevazen,mixtral-swa"] if a.compare_lefolorn else
-                ["--models", "surodra,nositar,jamba"] if a.compare_surodra else [])
+                ["--models", "surodra,nositar,jamba"] if a.compare_surodra else
+                ["--models", "tilulorn,lefolorn,surodra"] if a.compare_tilulorn else [])
         argv += ["--sizes", a.sizes, "--batch", str(32 if a.batch == 256 else a.batch),
                  "--input-len", str(2048 if a.input_len == 1024 else a.input_len),
                  "--output-len", str(64 if a.output_len == 128 else a.output_len)]

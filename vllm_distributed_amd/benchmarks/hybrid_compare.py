@@ -1,11 +1,12 @@
-"""Prefill and decode throughput of a Nositar, Rapovik, Sevazen, Lefolorn or Surodra stack beside the closest existing
-models of equal size, random weights.
+"""Prefill and decode throughput of a Nositar, Rapovik, Sevazen, Lefolorn, Surodra or Tilulorn stack beside the closest
+existing models of equal size, random weights.
 
     python bench.py --compare-nositar [--sizes small,medium] [--batch 32] [--input-len 2048] [--output-len 64]
     python bench.py --compare-rapovik [...]        (rapovik beside jamba-moe)
     python bench.py --compare-sevazen [...]        (sevazen beside mixtral-swa)
     python bench.py --compare-lefolorn [...]       (lefolorn beside sevazen and mixtral-swa)
     python bench.py --compare-surodra [...]        (surodra beside nositar and jamba)
+    python bench.py --compare-tilulorn [...]       (tilulorn beside lefolorn and surodra)
 
 Per size three engines run one after the other, each in a process of its own (``--one`` is the child's entry):
   nositar      alternating sigmoid head-mixing attention (window + kept first tokens) and gated delta-rule layers,
@@ -25,6 +26,9 @@ Per size three engines run one after the other, each in a process of its own (``
                choices per token, from the better of two groups) plus a shared expert
   surodra      delta-rule, attention-beside-gated-linear-attention and retention mixers in turn under squashing norms over an
                fp32 residual; GELU-gated feed-forwards; the whole list is the looped part, run once
+  tilulorn     latent attention, window attention over values that are the keys, and RWKV-style time mixing in turn over an
+               fp32 residual; every layer has 8 routed gated experts (two per token, chosen by token id); the whole list
+               is the looped part, run once
   mixtral-swa  a Mixtral stack of the same width, depth and heads with the same sliding window and 8 routed gated
                experts (two per token) of equal weight count
 Prefill: ``batch`` prompts of ``input-len`` tokens, one generated token.  Decode: the same requests generating
@@ -178,7 +182,28 @@ def surodra_config(s: dict) -> dict:
             "layers": [(delta, par, ret)[i % 3] for i in range(s["layers"])]}
 
 
-MODELS = {"surodra": surodra_config, "lefolorn": lefolorn_config, "sevazen": sevazen_config,
+def tilulorn_config(s: dict) -> dict:
+    """Latent attention (latent and query latent of the Lefolorn stacks, YaRN frequencies, no window), window attention whose
+    values are its keys (whole heads rotated, sinks) and time mixing (heads of 64, as many channels as the width, decay
+    rank 64) in turn; 8 gated experts per layer of the Mixtral stack's width, two per token id."""
+    w, ff, d = s["width"], s["ff"], s["dim"]
+    rank, rot = (128, 32) if d <= 64 else (512, 64)
+    moe = {"kind": "moe", "router": {"experts": 8, "top": 2}, "expert": {"ff": ff}}
+    lat = {"type": "latent_attention",
+           "mixer": {"heads": s["heads"], "dim": d, "rot_dim": rot, "vdim": d, "kv_rank": rank, "q_rank": w // 2,
+                     "scale": (d + rot) ** -0.5,
+                     "rot": {"base": 10000.0, "dims": rot,
+                             "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    win = {"type": "attention",
+           "mixer": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5,
+                     "mask": {"size": s["window"]}, "rot": {"base": 100000.0, "dims": d, "scaling": {"factor": 4.0}}}}
+    mix = {"type": "wkv", "mixer": {"heads": w // 64, "dim": 64, "decay_rank": 64}}
+    return {"architecture": "Tilulorn", "vocab": s["vocab"], "width": w, "norm": {"eps": 1e-6},
+            "loop": {"start": 0, "stop": s["layers"], "times": 1},
+            "layers": [dict((lat, win, mix)[i % 3], mlp=moe) for i in range(s["layers"])]}
+
+
+MODELS = {"tilulorn": tilulorn_config, "surodra": surodra_config, "lefolorn": lefolorn_config, "sevazen": sevazen_config,
           "mixtral-swa": mixtral_swa_config, "nositar": nositar_config, "llama-swa": llama_config, "jamba": jamba_config,
           "jamba-moe": jamba_moe_config, "rapovik": rapovik_config}
 

@@ -578,6 +578,14 @@ def skinny_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
 _DECODE_WS: dict = {}
 
 
+def _gemm_workspace(device) -> torch.Tensor:
+    """Split-K partial sums; one arena per device, reused by every call (stream order)."""
+    ws = _DECODE_WS.get(device)
+    if ws is None:
+        ws = _DECODE_WS[device] = torch.empty(envs.VDA_DECODE_GEMM_WS_MB << 18, dtype=torch.float32, device=device)
+    return ws
+
+
 def decode_gemm_ok(M: int, N_: int, K: int, dtype: torch.dtype) -> bool:
     """Shapes the weight-streaming decode GEMM takes (and is meant for: the rows of a decode batch)."""
     return (envs.VDA_DECODE_GEMM_MIN_M <= M <= min(envs.VDA_DECODE_GEMM_MAX_M, 256) and K % 256 == 0 and N_ % 4 == 0
@@ -600,9 +608,7 @@ def decode_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
         raise ValueError("decode_gemm: x must be [M, K] with unit column stride and w [N, K] contiguous")
     if out is None:
         out = torch.empty((M, N_), dtype=x.dtype, device=x.device)
-    ws = _DECODE_WS.get(x.device)
-    if ws is None:          # split-K partial sums; one arena per device, reused by every call (stream order)
-        ws = _DECODE_WS[x.device] = torch.empty(envs.VDA_DECODE_GEMM_WS_MB << 18, dtype=torch.float32, device=x.device)
+    ws = _gemm_workspace(x.device)
     N.call("vda_decode_gemm", out.data_ptr(), x.data_ptr(), w.data_ptr(), N.ptr(bias), ws.data_ptr(),
            ws.numel() * 4, M, N_, K, x.stride(0), out.stride(0), N.dt(x.dtype), N.stream())
     return out
@@ -644,12 +650,10 @@ def dense_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = 
         raise ValueError("dense_gemm: x must be 16-bit [M, K] (K % 32 == 0), w [N, K] contiguous of the same dtype")
     if out is None:
         out = torch.empty((M, n_out), dtype=x.dtype, device=x.device)
-    ws = _DECODE_WS.get(x.device)
-    if ws is None:          # split-K partial sums; one arena per device, reused by every call (stream order)
-        ws = _DECODE_WS[x.device] = torch.empty(envs.VDA_DECODE_GEMM_WS_MB << 18, dtype=torch.float32, device=x.device)
+    ws = _gemm_workspace(x.device)
     N.call("vda_dense_gemm", out.data_ptr(), x.data_ptr(), w.data_ptr(), N.ptr(bias), N.ptr(residual), ws.data_ptr(),
            ws.numel() * 4, M, n_out, K, x.stride(0), out.stride(0), residual.stride(0) if residual is not None else 0,
-           epi, N.dt(x.dtype), wt, splits, variant, N.stream())
+           epi, N.dt(x.dtype), wt, splits, variant, 1, 0, 0, 0, N.stream())
     return out
 
 
@@ -682,8 +686,20 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None
 
 
 def grouped_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-    """y[g] = x[g] @ w[g].T for x [G, M, K], w [G, N, K]: products of one size over inputs of their own."""
-    return torch.stack([linear(x[g], w[g]) for g in range(x.shape[0])])
+    """y[g] = x[g] @ w[g].T for x [G, M, K], w [G, N, K]: products of one size over inputs of their own.  The rows of a decode
+    batch go through one launch of the in-tree GEMM, more rows through one library product per g."""
+    G, M, K = x.shape
+    n_out = w.shape[1]
+    y = torch.empty((G, M, n_out), dtype=x.dtype, device=x.device)
+    if x.is_cuda and M <= min(envs.VDA_DENSE_GEMM_MAX_M, 256) and n_out % 4 == 0 and x.is_contiguous() and w.is_contiguous() \
+            and dense_gemm_ok(x[0], w[0]) and w.shape == (G, n_out, K):
+        ws = _gemm_workspace(x.device)
+        N.call("vda_dense_gemm", y.data_ptr(), x.data_ptr(), w.data_ptr(), None, None, ws.data_ptr(), ws.numel() * 4, M, n_out,
+               K, K, n_out, 0, 0, N.dt(x.dtype), 0, 0, 0, G, M * K, n_out * K, M * n_out, N.stream())
+        return y
+    for g in range(G):
+        torch.mm(x[g], w[g].t(), out=y[g])
+    return y
 
 
 def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:

@@ -15,7 +15,20 @@ struct DenseGemmArgs {
   int M, N, K;
   int m_tiles, n_tiles, splits, units_per_split;
   long x_stride, out_stride, res_stride;   // elements
+  // several products of one size in a launch: product z's operands lie z times these many elements further on
+  long x_batch, w_batch, out_batch;
 };
+
+// the arguments of product z (no bias, no residual when there are several)
+template <typename T> __device__ __forceinline__ DenseGemmArgs dense_product(DenseGemmArgs a, unsigned z, int w_rows) {
+  if (z) {
+    a.x = reinterpret_cast<const T*>(a.x) + z * a.x_batch;
+    a.w = reinterpret_cast<const T*>(a.w) + z * a.w_batch;
+    a.out = reinterpret_cast<T*>(a.out) + z * a.out_batch;
+    if (a.splits > 1) a.ws += (long)z * a.splits * a.M * w_rows;
+  }
+  return a;
+}
 
 __device__ __forceinline__ int swz64(int r) { return (-(r >> 2)) & 3; }
 
@@ -166,8 +179,9 @@ __device__ __forceinline__ void dense_epilogue(const DenseGemmArgs& a, const f32
 
 // out[m][n] = epilogue(sum over splits of ws[s][m][row(n)]); four columns per thread (N % 4 == 0)
 template <typename T, int EPI>
-__global__ __launch_bounds__(256) void dense_gemm_reduce_kernel(const DenseGemmArgs a) {
+__global__ __launch_bounds__(256) void dense_gemm_reduce_kernel(const DenseGemmArgs args) {
   using V4 = typename Vec<T>::v4;
+  const DenseGemmArgs a = dense_product<T>(args, blockIdx.y, EPI == DG_GATE_UP ? 2 * args.N : args.N);
   const int nq = a.N >> 2;
   const long q = (long)blockIdx.x * 256 + threadIdx.x;
   if (q >= (long)a.M * nq) return;

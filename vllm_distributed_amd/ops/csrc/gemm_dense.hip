@@ -50,7 +50,8 @@ __device__ __forceinline__ unsigned long long dg_stamp() {
 }
 
 template <typename T, int EPI, int WT, int XT, bool STAMP = false>
-__global__ __launch_bounds__(512, 1) void dense_gemm_kernel(const DenseGemmArgs a) {
+__global__ __launch_bounds__(512, 1) void dense_gemm_kernel(const DenseGemmArgs args) {
+  const DenseGemmArgs a = dense_product<T>(args, blockIdx.z, EPI == DG_GATE_UP ? 2 * args.N : args.N);
   unsigned long long rt0 = 0, rt1 = 0, rt2 = 0;
   if (STAMP) rt0 = __builtin_amdgcn_s_memrealtime();
   using V4 = typename Vec<T>::v4;
@@ -351,13 +352,14 @@ __global__ __launch_bounds__(512, 1) void dense_gemm_k64_kernel(const DenseGemmA
 }
 
 template <typename T, int EPI>
-static int launch_dense_gemm(const DenseGemmArgs& a, int wt, int xt, bool k64, hipStream_t st) {
+static int launch_dense_gemm(const DenseGemmArgs& a, int wt, int xt, bool k64, int batch, hipStream_t st) {
   dim3 grid;
   if (a.m_tiles == 1) grid = dim3((unsigned)(a.n_tiles * a.splits));
   else {
     const int pm = (a.m_tiles + 7) / 8, pn = (a.n_tiles + 7) / 8;
     grid = dim3((unsigned)((pm * pn + 7) / 8 * 8 * 64), (unsigned)a.splits);
   }
+  grid.z = (unsigned)batch;
 #define LAUNCH(WT, XT) hipLaunchKernelGGL((dense_gemm_kernel<T, EPI, WT, XT>), grid, dim3(512), 0, st, a)
 #define BY_XT(WT) do { if (xt == 8) LAUNCH(WT, 8); else if (xt == 4) LAUNCH(WT, 4); else if (xt == 2) LAUNCH(WT, 2); \
                        else LAUNCH(WT, 1); } while (0)
@@ -368,7 +370,8 @@ static int launch_dense_gemm(const DenseGemmArgs& a, int wt, int xt, bool k64, h
 #undef LAUNCH
   if (a.splits > 1) {
     const long quads = (long)a.M * (a.N >> 2);
-    hipLaunchKernelGGL((dense_gemm_reduce_kernel<T, EPI>), dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((dense_gemm_reduce_kernel<T, EPI>), dim3((unsigned)((quads + 255) / 256), (unsigned)batch), dim3(256), 0,
+                       st, a);
   }
   return 0;
 }
@@ -376,17 +379,20 @@ static int launch_dense_gemm(const DenseGemmArgs& a, int wt, int xt, bool k64, h
 // x [M, K] (row stride x_stride elements), w [N or 2 N, K] contiguous, out [M, N] (row stride out_stride), optional
 // bias [N] and residual [M, N] (PLAIN only).  K % 32 == 0; strides multiples of 8 elements; the byte size of x and
 // of w below 4 GiB (32-bit offsets in the copy addresses).  wt / splits: 0 = chosen here (wt 2 or 4: 128 or 256
-// weight rows per tile).  ws: fp32 scratch of ws_bytes for split K (may be null: K is then not split).
+// weight rows per tile).  batch > 1 (M <= 256, no bias or residual): so many products of this size, x_batch / w_batch /
+// out_batch elements apart.  ws: fp32 scratch of ws_bytes for split K (may be null: K is then not split).
 // Returns 0, or a negative code for shapes it does not take.
 VDA_EXPORT int vda_dense_gemm(void* out, const void* x, const void* w, const void* bias, const void* residual,
                               float* ws, size_t ws_bytes, int M, int N, int K, long x_stride, long out_stride,
-                              long res_stride, int epi, int dtype, int wt, int splits, int variant, hipStream_t st) {
+                              long res_stride, int epi, int dtype, int wt, int splits, int variant, int batch,
+                              long x_batch, long w_batch, long out_batch, hipStream_t st) {
   if (M < 1) return M == 0 ? 0 : -1;
   if (N < 1 || K < 32 || K % 32) return -1;
   if (x_stride % 8 || (N % 4 && out_stride % 4)) return -1;
   if (epi != DG_PLAIN && epi != DG_GATE_UP) return -4;
   if (epi == DG_GATE_UP && (bias || residual || N % 4)) return -4;
   if (dtype != VDA_BF16 && dtype != VDA_F16) return -3;
+  if (batch < 1 || (batch > 1 && (bias || residual || M > 256 || x_batch % 8 || w_batch % 8 || out_batch % 4))) return -1;
   const long w_rows = epi == DG_GATE_UP ? 2L * N : N;
   if (w_rows * K * 2 >= (1LL << 32) || (long)M * x_stride * 2 >= (1LL << 32)) return -2;
   int xt = M > 128 ? 8 : M > 64 ? 4 : M > 32 ? 2 : 1;
@@ -399,7 +405,7 @@ VDA_EXPORT int vda_dense_gemm(void* out, const void* x, const void* w, const voi
   // launch and its round trip over the fp32 partial sums.  Splits never create a second round of workgroups.
   auto plan = [&](int t, int forced_splits, double* cost) {
     const int ncol = epi == DG_GATE_UP ? 32 * t : 64 * t;
-    const long tiles = (long)m_tiles * ((N + ncol - 1) / ncol);
+    const long tiles = (long)m_tiles * ((N + ncol - 1) / ncol) * batch;
     int sp = forced_splits;
     if (sp < 1) {
       sp = 1;
@@ -408,10 +414,10 @@ VDA_EXPORT int vda_dense_gemm(void* out, const void* x, const void* w, const voi
       sp = min(sp, 16);
     }
     if (!can_split) sp = 1;
-    while (sp > 1 && (size_t)sp * M * w_rows * sizeof(float) > ws_bytes) --sp;
+    while (sp > 1 && (size_t)sp * M * w_rows * batch * sizeof(float) > ws_bytes) --sp;
     const long rounds = (tiles * sp + 255) / 256;
     const double unit_us = 0.17 * t + 0.011 * xt;
-    *cost = rounds * ((nu + sp - 1) / sp) * unit_us + (sp > 1 ? 4.0 + (double)M * w_rows * sp * 8 / 3e6 : 0.0);
+    *cost = rounds * ((nu + sp - 1) / sp) * unit_us + (sp > 1 ? 4.0 + (double)M * w_rows * sp * batch * 8 / 3e6 : 0.0);
     return sp;
   };
   if (wt != 2 && wt != 4) {
@@ -426,6 +432,7 @@ VDA_EXPORT int vda_dense_gemm(void* out, const void* x, const void* w, const voi
   DenseGemmArgs a;
   a.out = out; a.x = x; a.w = w; a.bias = bias; a.residual = residual; a.ws = ws;
   a.M = M; a.N = N; a.K = K; a.x_stride = x_stride; a.out_stride = out_stride; a.res_stride = res_stride;
+  a.x_batch = x_batch; a.w_batch = w_batch; a.out_batch = out_batch;
   a.m_tiles = m_tiles;
   a.n_tiles = (N + ncol - 1) / ncol;
   // variant: 0 = chosen here, 1 = ring of 32-element units, 2 = 64-element units (256 x 256 tiles, K % 64 == 0)
@@ -435,10 +442,10 @@ VDA_EXPORT int vda_dense_gemm(void* out, const void* x, const void* w, const voi
   if (use_k64) a.units_per_split = (a.units_per_split + 1) & ~1;       // whole 64-element units per split
   a.splits = (nu + a.units_per_split - 1) / a.units_per_split;
   int rc;
-  if (dtype == VDA_BF16) rc = epi == DG_GATE_UP ? launch_dense_gemm<bf16_t, DG_GATE_UP>(a, wt, xt, use_k64, st)
-                                                : launch_dense_gemm<bf16_t, DG_PLAIN>(a, wt, xt, use_k64, st);
-  else rc = epi == DG_GATE_UP ? launch_dense_gemm<f16_t, DG_GATE_UP>(a, wt, xt, use_k64, st)
-                              : launch_dense_gemm<f16_t, DG_PLAIN>(a, wt, xt, use_k64, st);
+  if (dtype == VDA_BF16) rc = epi == DG_GATE_UP ? launch_dense_gemm<bf16_t, DG_GATE_UP>(a, wt, xt, use_k64, batch, st)
+                                                : launch_dense_gemm<bf16_t, DG_PLAIN>(a, wt, xt, use_k64, batch, st);
+  else rc = epi == DG_GATE_UP ? launch_dense_gemm<f16_t, DG_GATE_UP>(a, wt, xt, use_k64, batch, st)
+                              : launch_dense_gemm<f16_t, DG_PLAIN>(a, wt, xt, use_k64, batch, st);
   if (rc) return rc;
   VDA_CHECK_LAUNCH();
   return 0;
@@ -452,6 +459,7 @@ VDA_EXPORT int vda_dense_gemm_stamp(void* dbg, const void* x, const void* w, int
   DenseGemmArgs a;
   a.out = nullptr; a.x = x; a.w = w; a.bias = nullptr; a.residual = nullptr; a.ws = reinterpret_cast<float*>(dbg);
   a.M = M; a.N = N; a.K = K; a.x_stride = K; a.out_stride = N; a.res_stride = 0;
+  a.x_batch = a.w_batch = a.out_batch = 0;
   a.m_tiles = (M + 255) / 256; a.n_tiles = (N + 255) / 256; a.splits = 1; a.units_per_split = K >> 5;
   const int pm = (a.m_tiles + 7) / 8, pn = (a.n_tiles + 7) / 8;
   const dim3 grid((unsigned)((pm * pn + 7) / 8 * 8 * 64));

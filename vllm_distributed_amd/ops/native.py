@@ -86,7 +86,7 @@ _SIGS = {
     "vda_decode_gemm": [P, P, P, P, P, L, I, I, I, L, L, I, P],
     "vda_wq_gemm": [P, P, P, P, P, P, L, I, I, I, I, I, L, L, I, I, I, P],
     "vda_dense_gemm_stamp": [P, P, P, I, I, I, I, P],
-    "vda_dense_gemm": [P, P, P, P, P, P, L, I, I, I, L, L, L, I, I, I, I, I, P],
+    "vda_dense_gemm": [P, P, P, P, P, P, L, I, I, I, L, L, L, I, I, I, I, I, I, L, L, L, P],
     "vda_per_group_fp8_quant": [P, P, P, I, I, I, L, L, I, P],
     "vda_w4_skinny_gemm": [P, P, P, P, P, P, I, I, I, I, L, L, I, P],
     "vda_w4_dequant": [P, P, P, P, I, I, I, I, P],
