@@ -199,3 +199,103 @@ def forward(cfg, weights, tokens, dtype=torch.float32, want_layers=False):
         trail.append(x)
     y = rms_norm(x, W["final.norm"], eps) @ W["head"].T
     return (y, torch.stack(trail)) if want_layers else y
+
+
+# ---- small random models ---------------------------------------------------------------------------------------------
+def _mlp(ff, experts, top):
+    return None if ff is None else {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+
+
+def latent_layer(heads=3, dim=12, rot_dim=8, vdim=20, kv_rank=24, q_rank=28, base=300.0, scaling=(3.0, 24, 4.0, 0.5),
+                 scale=0.25, ff=24, experts=5, top=2):
+    rot = {"base": base, "dims": rot_dim}
+    if scaling:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    return {"type": "latent_attention", "mlp": _mlp(ff, experts, top),
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "q_rank": q_rank,
+                      "scale": scale, "rot": rot}}
+
+
+def window_layer(heads=4, kv_heads=2, dim=12, window=21, rot_dims=8, base=200.0, factor=2.5, scale=0.3, ff=20, experts=4,
+                 top=1):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": scale, "mask": {"size": window}}
+    if rot_dims:
+        m["rot"] = {"base": base, "dims": rot_dims, **({"scaling": {"factor": factor}} if factor else {})}
+    return {"type": "attention", "mlp": _mlp(ff, experts, top), "mixer": m}
+
+
+def wkv_layer(heads=3, dim=12, rank=5, ff=16, experts=3, top=3):
+    return {"type": "wkv", "mlp": _mlp(ff, experts, top), "mixer": {"heads": heads, "dim": dim}}, rank
+
+
+def make_config(layers, vocab=96, width=48, eps=1e-2, loop=None):
+    """(config, ranks of the decay projections by layer); ``layers`` may hold (layer, rank) pairs."""
+    ranks = {i: l[1] for i, l in enumerate(layers) if isinstance(l, tuple)}
+    cfg = {"architecture": "Tilulorn", "vocab": vocab, "width": width, "norm": {"eps": eps},
+           "layers": [l[0] if isinstance(l, tuple) else l for l in layers]}
+    if loop:
+        cfg["loop"] = {"start": loop[0], "stop": loop[1], "times": loop[2]}
+    return cfg, ranks
+
+
+def make_weights(cfg, ranks, seed=0):
+    g = torch.Generator().manual_seed(seed)
+    Wd, V = cfg["width"], cfg["vocab"]
+
+    def rnd(*shape, s=1.0):
+        return torch.randn(*shape, generator=g) * s
+
+    def lin(o, i, s=1.0):
+        return rnd(o, i, s=s / math.sqrt(i))
+
+    def near1(*shape):
+        return 1.0 + rnd(*shape, s=0.15)
+    W = {"embed": rnd(V, Wd), "head": lin(V, Wd, 4.0), "final.norm": near1(Wd)}
+    if cfg.get("loop"):
+        W["loop.in"] = torch.cat([0.7 * torch.eye(Wd) + lin(Wd, Wd, 0.4), lin(Wd, Wd, 0.6)], -1)
+        W["loop.step"] = rnd(cfg["loop"]["times"], Wd, s=0.6)
+    for i, L in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", L["mixer"]
+        x = p + "mix."
+        W[p + "norm1"] = near1(Wd)
+        if L["type"] == "wkv":
+            H, D = m["heads"], m["dim"]
+            W.update({x + s: lin(H * D, Wd, 2.0) for s in "rkvg"})
+            W.update({x + "mu." + s: torch.rand(Wd, generator=g) * 0.9 for s in "rkvgw"})
+            W.update({x + "w1": lin(ranks[i], Wd, 1.5), x + "w2": lin(H * D, ranks[i], 1.5), x + "w0": rnd(H * D) - 2.5,
+                      x + "u": 0.5 + rnd(H, D, s=0.5), x + "norm": near1(H * D), x + "o": lin(Wd, H * D)})
+        elif L["type"] == "attention":
+            H, G, D = m["heads"], m["kv_heads"], m["dim"]
+            W.update({x + "q": lin(H * D, Wd, 2.0), x + "k": lin(G * D, Wd, 2.0), x + "q.norm": 1.5 * near1(H * D),
+                      x + "k.norm": 1.5 * near1(G * D), x + "sink": rnd(H) + 1.0, x + "g": lin(H, Wd, 2.0),
+                      x + "o": lin(Wd, H * D)})
+        else:
+            H, D, P, E, R, Q = (m[n] for n in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank"))
+            W.update({x + "dq": lin(Q, Wd, 2.0), x + "dq.norm": near1(Q), x + "uq": lin(H * (D + P), Q, 2.0),
+                      x + "dkv": lin(R + P, Wd, 2.0), x + "dkv.norm": near1(R), x + "uk": lin(H * D, R, 2.0),
+                      x + "uv": lin(H * E, R, 2.0), x + "g": lin(H, Wd, 2.0), x + "o": lin(Wd, H * E, 1.5)})
+        if L.get("mlp"):
+            ff, n, top = L["mlp"]["expert"]["ff"], L["mlp"]["router"]["experts"], L["mlp"]["router"]["top"]
+            W[p + "norm2"] = near1(Wd)
+            for e in range(n):
+                W.update({p + f"mlp.e{e}.gate": lin(ff, Wd, 2.0), p + f"mlp.e{e}.up": lin(ff, Wd, 2.0),
+                          p + f"mlp.e{e}.down": lin(Wd, ff, 1.5)})
+            W[p + "mlp.table"] = torch.stack([torch.randperm(n, generator=g)[:top] for _ in range(V)]).to(torch.int32)
+    # the checkpoint holds bfloat16: round once, so that oracle and engine read the same numbers
+    return {k: v.to(torch.bfloat16) if v.is_floating_point() else v for k, v in W.items()}
+
+
+def save_checkpoint(folder, cfg, W):
+    from safetensors.torch import save_file
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    save_file({k: v.contiguous() for k, v in W.items()}, os.path.join(folder, "model.safetensors"))
+    return folder
+
+
+def logit_error(got, want):
+    """Root mean square difference over the vocabulary with the mean taken off, relative to the logits' own spread."""
+    d = torch.as_tensor(got).float() - torch.as_tensor(want).float()
+    d = d - d.mean(-1, keepdim=True)
+    return (d.pow(2).mean(-1).sqrt() / torch.as_tensor(want).float().std(-1).clamp_min(1e-6)).max().item()

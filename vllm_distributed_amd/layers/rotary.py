@@ -32,9 +32,8 @@ def _yarn_range(low_rot, high_rot, dim, base, max_pos) -> tuple[int, int]:
 
 
 def _ramp(lo: float, hi: float, n: int, dtype: torch.dtype = torch.float32) -> torch.Tensor:
-    if lo == hi:
-        hi += 0.001
-    return ((torch.arange(n, dtype=dtype) - lo) / (hi - lo)).clamp(0, 1)
+    # no length (or less: both ends behind the last dimension) is a step
+    return ((torch.arange(n, dtype=dtype) - lo) / max(hi - lo, 0.001)).clamp(0, 1)
 
 
 def yarn_mscale(scale: float = 1.0, mscale: float = 1.0) -> float:
