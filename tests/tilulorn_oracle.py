@@ -228,7 +228,7 @@ def wkv_layer(heads=3, dim=12, rank=5, ff=16, experts=3, top=3):
     return {"type": "wkv", "mlp": _mlp(ff, experts, top), "mixer": {"heads": heads, "dim": dim}}, rank
 
 
-def make_config(layers, vocab=96, width=48, eps=1e-2, loop=None):
+def make_config(layers, vocab=96, width=48, eps=5e-2, loop=None):
     """(config, ranks of the decay projections by layer); ``layers`` may hold (layer, rank) pairs."""
     ranks = {i: l[1] for i, l in enumerate(layers) if isinstance(l, tuple)}
     cfg = {"architecture": "Tilulorn", "vocab": vocab, "width": width, "norm": {"eps": eps},
@@ -252,7 +252,7 @@ def make_weights(cfg, ranks, seed=0):
         return 1.0 + rnd(*shape, s=0.15)
     W = {"embed": rnd(V, Wd), "head": lin(V, Wd, 4.0), "final.norm": near1(Wd)}
     if cfg.get("loop"):
-        W["loop.in"] = torch.cat([0.7 * torch.eye(Wd) + lin(Wd, Wd, 0.4), lin(Wd, Wd, 0.6)], -1)
+        W["loop.in"] = torch.cat([0.6 * torch.eye(Wd) + lin(Wd, Wd, 0.3), lin(Wd, Wd, 0.8)], -1)
         W["loop.step"] = rnd(cfg["loop"]["times"], Wd, s=0.6)
     for i, L in enumerate(cfg["layers"]):
         p, m = f"l{i}.", L["mixer"]
@@ -260,7 +260,7 @@ def make_weights(cfg, ranks, seed=0):
         W[p + "norm1"] = near1(Wd)
         if L["type"] == "wkv":
             H, D = m["heads"], m["dim"]
-            W.update({x + s: lin(H * D, Wd, 2.0) for s in "rkvg"})
+            W.update({x + s: lin(H * D, Wd, 1.0 if s in "rk" else 2.0) for s in "rkvg"})
             W.update({x + "mu." + s: torch.rand(Wd, generator=g) * 0.9 for s in "rkvgw"})
             W.update({x + "w1": lin(ranks[i], Wd, 1.5), x + "w2": lin(H * D, ranks[i], 1.5), x + "w0": rnd(H * D) - 2.5,
                       x + "u": 0.5 + rnd(H, D, s=0.5), x + "norm": near1(H * D), x + "o": lin(Wd, H * D)})
@@ -271,15 +271,15 @@ def make_weights(cfg, ranks, seed=0):
                       x + "o": lin(Wd, H * D)})
         else:
             H, D, P, E, R, Q = (m[n] for n in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank"))
-            W.update({x + "dq": lin(Q, Wd, 2.0), x + "dq.norm": near1(Q), x + "uq": lin(H * (D + P), Q, 2.0),
-                      x + "dkv": lin(R + P, Wd, 2.0), x + "dkv.norm": near1(R), x + "uk": lin(H * D, R, 2.0),
-                      x + "uv": lin(H * E, R, 2.0), x + "g": lin(H, Wd, 2.0), x + "o": lin(Wd, H * E, 1.5)})
+            W.update({x + "dq": lin(Q, Wd, 2.0), x + "dq.norm": near1(Q), x + "uq": lin(H * (D + P), Q, 1.5),
+                      x + "dkv": lin(R + P, Wd, 2.0), x + "dkv.norm": near1(R), x + "uk": lin(H * D, R, 1.5),
+                      x + "uv": lin(H * E, R, 2.0), x + "g": lin(H, Wd, 2.0), x + "o": lin(Wd, H * E)})
         if L.get("mlp"):
             ff, n, top = L["mlp"]["expert"]["ff"], L["mlp"]["router"]["experts"], L["mlp"]["router"]["top"]
             W[p + "norm2"] = near1(Wd)
             for e in range(n):
                 W.update({p + f"mlp.e{e}.gate": lin(ff, Wd, 2.0), p + f"mlp.e{e}.up": lin(ff, Wd, 2.0),
-                          p + f"mlp.e{e}.down": lin(Wd, ff, 1.5)})
+                          p + f"mlp.e{e}.down": lin(Wd, ff)})
             W[p + "mlp.table"] = torch.stack([torch.randperm(n, generator=g)[:top] for _ in range(V)]).to(torch.int32)
     # the checkpoint holds bfloat16: round once, so that oracle and engine read the same numbers
     return {k: v.to(torch.bfloat16) if v.is_floating_point() else v for k, v in W.items()}
